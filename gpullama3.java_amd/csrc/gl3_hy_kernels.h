@@ -51,17 +51,28 @@ __device__ __forceinline__ float hy_block_sum(float v, float* red) {
 }
 
 // step record in device memory (read by the kernels, so that a captured step can be replayed at another position):
-// dyn[0] = position of the step's first token, dyn[1] = sequence slot
+// dyn[0] = position of the step's first token, dyn[1] = sequence slot, dyn[2] = the sequence's token before the step's first one
 constexpr int HY_MAX_STREAMS = 8;
 
-// ---- embedding: every stream starts as the token's row times `scale`; copy != null keeps the embedding output for the depth average --
+// ---- embedding: every stream starts as the token's row times `scale`, plus (bg.table) a row picked by the token pair,
+// (previous mul_prev + token mul_cur) mod buckets, or row `buckets` for a sequence's first token; copy != null keeps the embedding output
+// for the depth average ----
+struct HyBigram { const void* table; int buckets, mul_prev, mul_cur; };
 template <typename T>
 static __global__ __launch_bounds__(256) void hy_embed_kernel(const int* __restrict__ tokens, const T* __restrict__ emb, float* __restrict__ X,
-                                                              int W, int S, size_t sstride, float scale, float* __restrict__ copy) {
-    const int t = blockIdx.x;
-    const T* row = emb + (size_t)tokens[t] * W;
+                                                              int W, int S, size_t sstride, float scale, float* __restrict__ copy, HyBigram bg = HyBigram{},
+                                                              const int* __restrict__ dyn = nullptr) {
+    const int t = blockIdx.x, tok = tokens[t];
+    const T* row = emb + (size_t)tok * W;
+    const T* pair = nullptr;
+    if (bg.table) {
+        const int prev = t > 0 ? tokens[t - 1] : dyn[2];
+        const int b = (t == 0 && dyn[0] == 0) ? bg.buckets : (int)(((long long)prev * bg.mul_prev + (long long)tok * bg.mul_cur) % bg.buckets);
+        pair = (const T*)bg.table + (size_t)b * W;
+    }
     for (int w = blockIdx.y * 256 + threadIdx.x; w < W; w += 256 * gridDim.y) {
-        const float v = hy_ld(row + w) * scale;
+        float v = hy_ld(row + w) * scale;
+        if (pair) v += hy_ld(pair + w);
         for (int s = 0; s < S; ++s) X[s * sstride + (size_t)t * W + w] = v;
         if (copy) copy[(size_t)t * W + w] = v;
     }
@@ -426,24 +437,44 @@ static __global__ __launch_bounds__(256) void hy_matvec_kernel(const T* __restri
 // in place, key heads likewise on their way to the key rows of the slot, value heads are normalised (optional), turned (optional) and
 // written to the value rows.  proj row = [.. q (H x D) .. k (G x D) .. v (G x V) ..].
 // Rotary turn: entry i of the first `dims` pairs with entry i + dims / 2 (interleaved: entry 2 i with entry 2 i + 1) and the pair (u, v)
-// becomes (u cos a - v sin a, v cos a + u sin a), a = pos * freq[i] in float32; freq is a table the host made (base^(-2 i / dims),
-// divided for q / k by the position scaling).  An entry is (src + bias) * r * weight before it turns (bias, weight: null = absent).
+// becomes (u cos a - v sin a, v cos a + u sin a), a = pos * freq[i]; freq is a table the host made (base^(-2 i / dims), for q / k with the
+// position scaling applied).  An entry is (src + bias) * r * weight before it turns (bias, weight: null = absent).
+// q / k: the angle is formed and brought into (-pi, pi] in double (a float holds an angle of a thousand radians to 1e-4 only), sine and
+// cosine are float32; values (turned by j, their sum turned back by i with the same table): float32.
+__device__ __forceinline__ void hy_sincos_pos(int pos, double freq, float mscale, float* sn, float* cs) {
+    const double a = (double)pos * freq;
+    const float r = (float)(a - 6.283185307179586476925 * rint(a * 0.15915494309189533577));
+    sincosf(r, sn, cs);
+    *sn *= mscale; *cs *= mscale;
+}
+__device__ __forceinline__ void hy_turn_angle(int pos, const double* freq, int i, float* sn, float* cs) { hy_sincos_pos(pos, freq[i], 1.f, sn, cs); }
+__device__ __forceinline__ void hy_turn_angle(int pos, const float* freq, int i, float* sn, float* cs) { sincosf((float)pos * freq[i], sn, cs); }
 struct HyRot {
-    int qk_dims; const float* qk_freq;       // q / k: first qk_dims entries turn; 0 = none
+    int qk_dims; const double* qk_freq;      // q / k: first qk_dims entries turn; 0 = none
     int v_norm;                              // values: unit root mean square per head
     const float* v_freq;                     // values: all V entries turn (null = none)
     int interleaved;                         // q / k pairs are (2 i, 2 i + 1)
 };
-// further inputs of the cache writers (null = absent): a bias per projection row, added first; weights of the norm over a whole
-// projection (unit_norm = 2)
-struct HyPrepX { const float* bias; const float* qn; const float* kn; const float* rowr; };
-__device__ __forceinline__ void hy_turn_store(float* __restrict__ dst, const float* __restrict__ src, int D, int dims, const float* __restrict__ freq, float pos, float r, int lane,
+// further inputs of the cache writers (null / 0 = absent): a bias per projection row, added first; weights of the norm over a whole
+// projection (unit_norm = 2) or per head, shared by the heads (unit_norm = 3); values taken from the keys; and a causal depthwise
+// convolution over time on the q and k channels (C = (H + G) D of them, taps as rows [taps][C], last row = current token), which reads the
+// raw projections of the step's earlier tokens and the slot's tail (the last taps - 1 raw rows before the step, [taps - 1][C]): q then goes
+// to qout (row stride ldq) because other tokens still read the raw row.  A step of one token also moves the tail on (every thread the
+// channels it has read); longer steps leave that to hy_conv_tail_kernel.
+constexpr int HY_PREP_MAXD = 1024;
+struct HyPrepX {
+    const float* bias; const float* qn; const float* kn; const float* rowr;
+    int v_from_k;
+    const float* conv_w; int taps; float* tail; float* qout; int ldq; int n;
+};
+template <typename F>
+__device__ __forceinline__ void hy_turn_store(float* __restrict__ dst, const float* __restrict__ src, int D, int dims, const F* __restrict__ freq, int pos, float r, int lane,
                                               int interleaved = 0, const float* __restrict__ bias = nullptr, const float* __restrict__ w = nullptr) {
     const int half = dims >> 1;
     auto val = [&](int d) { return (src[d] + (bias ? bias[d] : 0.f)) * r * (w ? w[d] : 1.f); };
     for (int d = lane; d < half; d += 64) {
         float sn, cs;
-        sincosf(pos * freq[d], &sn, &cs);
+        hy_turn_angle(pos, freq, d, &sn, &cs);
         const int i0 = interleaved ? 2 * d : d, i1 = interleaved ? 2 * d + 1 : d + half;
         const float u = val(i0), v = val(i1);
         dst[i0] = u * cs - v * sn;
@@ -454,14 +485,37 @@ __device__ __forceinline__ void hy_turn_store(float* __restrict__ dst, const flo
 static __global__ __launch_bounds__(64) void hy_attn_prep_kernel(float* __restrict__ proj, int ld, int q_off, int k_off, int v_off, int H, int G, int D, int V,
                                                                  int unit_norm, float eps, float* __restrict__ kc, float* __restrict__ vc, size_t slot_stride,
                                                                  const int* __restrict__ dyn, HyRot rot, HyPrepX x = HyPrepX{}) {
+    __shared__ float crow[HY_PREP_MAXD];
     const int t = blockIdx.x, hh = blockIdx.y, lane = threadIdx.x;
     const int pos = dyn[0] + t;
     const size_t slot = (size_t)dyn[1] * slot_stride;
     if (hh < H + G) {
         const bool isq = hh < H;
         const int col = isq ? q_off + hh * D : k_off + (hh - H) * D;
-        float* src = proj + (size_t)t * ld + col;
+        const float* src = proj + (size_t)t * ld + col;
         const float* bias = x.bias ? x.bias + col : nullptr;
+        float* dst = isq ? proj + (size_t)t * ld + col : kc + slot + (size_t)pos * (G * D) + (hh - H) * D;
+        if (x.taps > 0) {
+            const int C = (H + G) * D, c0 = hh * D, keep = x.taps - 1;
+            float* tl = x.tail + slot + c0;
+            const bool fresh = dyn[0] == 0;
+            for (int d = lane; d < D; d += 64) {
+                float a = 0.f;
+                for (int j = 0; j < x.taps; ++j) {
+                    const int tau = t - keep + j;
+                    const float u = tau >= 0 ? proj[(size_t)tau * ld + col + d] : fresh ? 0.f : tl[(size_t)(keep + tau) * C + d];
+                    a = fmaf(x.conv_w[(size_t)j * C + c0 + d], u, a);
+                }
+                crow[d] = a;
+                if (x.n == 1) {
+                    for (int i = 0; i + 1 < keep; ++i) tl[(size_t)i * C + d] = fresh ? 0.f : tl[(size_t)(i + 1) * C + d];
+                    if (keep > 0) tl[(size_t)(keep - 1) * C + d] = src[d];
+                }
+            }
+            __syncthreads();
+            src = crow;
+            if (isq) dst = x.qout + (size_t)t * x.ldq + hh * D;
+        }
         const float* w = nullptr;
         float r = 1.f;
         if (unit_norm == 2) {          // over the whole projection: hy_rowrms_kernel has left 1 / rms of the token's q and k rows
@@ -472,10 +526,14 @@ static __global__ __launch_bounds__(64) void hy_attn_prep_kernel(float* __restri
             for (int d = lane; d < D; d += 64) { const float v = src[d] + (bias ? bias[d] : 0.f); ss += v * v; }
             ss = hy_wave_sum(ss);
             r = 1.f / sqrtf(ss / (float)D + eps);
+            if (unit_norm == 3) w = isq ? x.qn : x.kn;
         }
-        float* dst = isq ? src : kc + slot + (size_t)pos * (G * D) + (hh - H) * D;
-        if (isq && !unit_norm && !rot.qk_dims && !bias) return;
-        hy_turn_store(dst, src, D, rot.qk_dims, rot.qk_freq, (float)pos, r, lane, rot.interleaved, bias, w);      // a lane reads both entries of its pairs before it writes them
+        if (!isq && x.v_from_k) {          // V = D: the value is the key as it came in
+            float* vd = vc + slot + (size_t)pos * (G * V) + (hh - H) * V;
+            for (int d = lane; d < D; d += 64) vd[d] = src[d] + (bias ? bias[d] : 0.f);
+        }
+        if (isq && !unit_norm && !rot.qk_dims && !bias && dst == src) return;
+        hy_turn_store(dst, src, D, rot.qk_dims, rot.qk_freq, pos, r, lane, rot.interleaved, bias, w);      // a lane reads both entries of its pairs before it writes them
     } else {
         const int g = hh - H - G;
         const float* src = proj + (size_t)t * ld + v_off + g * V;
@@ -488,7 +546,7 @@ static __global__ __launch_bounds__(64) void hy_attn_prep_kernel(float* __restri
             ss = hy_wave_sum(ss);
             r = 1.f / sqrtf(ss / (float)V + eps);
         }
-        hy_turn_store(dst, src, V, rot.v_freq ? V : 0, rot.v_freq, (float)pos, r, lane, 0, bias);
+        hy_turn_store(dst, src, V, rot.v_freq ? V : 0, rot.v_freq, pos, r, lane, 0, bias);
     }
 }
 
@@ -555,14 +613,7 @@ static __global__ __launch_bounds__(64) void hy_latent_norm_kernel(const float* 
 // cached behind the latent).  blockIdx.y = 0: the first R entries of the token's down projection are RMS-normed with their weight into
 // the slot row's [0, R), the P entries behind them turn by the position into [R, R + P) (nothing when cc == null: a layer that reads
 // another layer's cache).  blockIdx.y = 1 + h: the last P entries of query head h turn in place.  Turn: pair (i, i + P / 2) becomes
-// (u c - v s, v c + u s), c = mscale cos(pos freq[i]), s = mscale sin(pos freq[i]).  The angle is formed and brought into (-pi, pi] in double
-// (a float holds an angle of a thousand radians to 1e-4 only), sine and cosine are float32.
-__device__ __forceinline__ void hy_sincos_pos(int pos, double freq, float mscale, float* sn, float* cs) {
-    const double a = (double)pos * freq;
-    const float r = (float)(a - 6.283185307179586476925 * rint(a * 0.15915494309189533577));
-    sincosf(r, sn, cs);
-    *sn *= mscale; *cs *= mscale;
-}
+// (u c - v s, v c + u s), c = mscale cos(pos freq[i]), s = mscale sin(pos freq[i]) (hy_sincos_pos).
 static __global__ __launch_bounds__(64) void hy_latent_prep_kernel(float* __restrict__ q, int ldq, int D, int P, const float* __restrict__ proj, int ld, int c_off, int R,
                                                                    const float* __restrict__ cnorm, float eps, float* __restrict__ cc, size_t slot_stride,
                                                                    const int* __restrict__ dyn, const double* __restrict__ freq, float mscale) {
@@ -968,9 +1019,11 @@ static __global__ __launch_bounds__(256) void hy_conv_tail_kernel(const float* _
 }
 
 // Recurrence S_t = a_t S_(t-1) + b_t k_t x_t^T,  y_t = S_t^T q_t + D x_t  per head, S = N x P (keys / queries of N entries, values of P).
-// Three sources of a_t, b_t (HyScanArgs.mode): 0, a state-space layer: dt = softplus(raw + bias), a = e^(-e^(A_log) dt), b = dt, keys
+// Sources of a_t, b_t (HyScanArgs.mode): 0, a state-space layer: dt = softplus(raw + bias), a = e^(-e^(A_log) dt), b = dt, keys
 // and queries shared by the heads of a group; 1, gates that a kernel before this one left per (token, head) (hy_mem_gates_kernel);
-// 2, a fixed decay per head, b = 1.  Keys, queries and x may pass through silu on the way into LDS (act); keys and queries are
+// 2, a fixed decay per head, b = 1; 3, one gate per key channel: with g = (1 - lower) sigmoid(-(source + bias)) made on the way into LDS in
+// the key's place, S_t = diag(1 - g) S_(t-1) + g x^T, walked as S += g (x - S): the small complement of a gate near one keeps its
+// relative precision.  Keys, queries and x may pass through silu on the way into LDS (act); keys and queries are
 // multiplied by k_mul / q_mul there and may turn by their
 // position (rot: first `dims` entries, pairs (i, i + dims / 2) or (2 i, 2 i + 1), angle = position * freq[i]).  ones_col: the last of
 // the P columns has x = 1 whatever the token (it then carries n_t = a n + b k, the normaliser of a matrix memory, and y's last column
@@ -987,12 +1040,13 @@ struct HyScanArgs {
     const float* qsrc; int ldq, q_off, q_hstride;
     const float* xsrc; int ldx, x_off;                 // x of (t, head, column): xsrc + t ldx + x_off + head Px + column, Px = P - ones_col
     float k_mul, q_mul;
-    int act;                                           // 1: keys, queries and x are silu(source) (before the multipliers)
+    int act;                                           // sum of 1: keys, 2: queries, 4: x are silu(source) (before the multipliers)
     HyScanRot rot;
     int mode;
     const float* dtsrc; int ld_dt, dt_off; const float* dt_bias; const float* A_log; const float* Dp;      // mode 0 (Dp: null = no skip term)
     const float* ga; const float* gb;                  // mode 1: [n][heads]
     const float* decay;                                // mode 2: [heads]
+    const float* fbias; const float* lower;            // mode 3: [heads N] each
     int ones_col;
     int heads, P, N, G, NG, TB;
     float* state; size_t slot_stride; const int* dyn; int n;
@@ -1015,6 +1069,26 @@ __device__ __forceinline__ void hy_scan_stage(float* __restrict__ dst, const flo
         }
     }
 }
+// mode 3: (1 - lower) sigmoid(-(row + bias)), zero behind N; eight loads in flight per thread
+__device__ __forceinline__ void hy_scan_stage_gate(float* __restrict__ dst, const float* __restrict__ base, int ld, int t0, int tb, int N, int Ns, const float* __restrict__ bias,
+                                                   const float* __restrict__ lower) {
+    const int total = tb * Ns;
+    for (int i0 = threadIdx.x; i0 < total; i0 += 8 * 256) {
+        float v[8], lo[8];
+#pragma unroll
+        for (int u = 0; u < 8; ++u) {
+            const int i = i0 + u * 256, t = i / Ns, nn = i - t * Ns;
+            const bool live = i < total && nn < N;
+            v[u] = live ? base[(size_t)(t0 + t) * ld + nn] + bias[nn] : 0.f;
+            lo[u] = live ? lower[nn] : 1.f;
+        }
+#pragma unroll
+        for (int u = 0; u < 8; ++u) {
+            const int i = i0 + u * 256;
+            if (i < total) dst[i] = (1.f - lo[u]) * hy_sigmoid(-v[u]);
+        }
+    }
+}
 // the staged rows turn in place by their position: one thread per pair
 __device__ __forceinline__ void hy_scan_turn(float* __restrict__ rows, int tb, int Ns, const HyScanRot& rot, int pos) {
     const int half = rot.dims >> 1;
@@ -1029,7 +1103,7 @@ __device__ __forceinline__ void hy_scan_turn(float* __restrict__ rows, int tb, i
         r[i1] = v * cs + u * sn;
     }
 }
-template <int NL>
+template <int NL, int CG>          // CG = 1: mode 3
 static __global__ __launch_bounds__(256) void hy_ssm_scan_kernel(HyScanArgs a) {
     extern __shared__ __attribute__((aligned(16))) float smem[];
     const int P = a.P, N = a.N, NG = a.NG, TB = a.TB, n = a.n, Px = P - (a.ones_col ? 1 : 0);
@@ -1059,14 +1133,15 @@ static __global__ __launch_bounds__(256) void hy_ssm_scan_kernel(HyScanArgs a) {
     for (int t0 = 0; t0 < n; t0 += TB) {
         const int tb = min(TB, n - t0);
         __syncthreads();
-        hy_scan_stage(sB, kbase, a.ldk, t0, tb, N, Ns, a.k_mul, a.act);
-        hy_scan_stage(sC, qbase, a.ldq, t0, tb, N, Ns, a.q_mul, a.act);
+        if constexpr (CG) hy_scan_stage_gate(sB, kbase, a.ldk, t0, tb, N, Ns, a.fbias + (size_t)head * N, a.lower + (size_t)head * N);
+        else hy_scan_stage(sB, kbase, a.ldk, t0, tb, N, Ns, a.k_mul, a.act & 1);
+        hy_scan_stage(sC, qbase, a.ldq, t0, tb, N, Ns, a.q_mul, a.act & 2);
         for (int i = tid; i < tb * cols; i += 256) {
             const int t = i / cols, c = i - t * cols;
-            if (col0 + c < Px) { const float xv = xbase[(size_t)(t0 + t) * a.ldx + col0 + c]; sX[i] = a.act ? hy_silu(xv) : xv; }
+            if (col0 + c < Px) { const float xv = xbase[(size_t)(t0 + t) * a.ldx + col0 + c]; sX[i] = (a.act & 4) ? hy_silu(xv) : xv; }
             else sX[i] = col0 + c < P ? 1.f : 0.f;
         }
-        if (tid < tb) {
+        if (!CG && tid < tb) {
             if (a.mode == 0) {
                 const float dt = hy_softplus(a.dtsrc[(size_t)(t0 + tid) * a.ld_dt + a.dt_off + head] + dtb);
                 sDt[tid] = dt;
@@ -1086,17 +1161,17 @@ static __global__ __launch_bounds__(256) void hy_ssm_scan_kernel(HyScanArgs a) {
         }
         __syncthreads();
         for (int t = 0; t < tb; ++t) {
-            const float dx = sDt[t] * sX[t * cols + myc], decay = sDt[TB + t];
+            const float dx = CG ? sX[t * cols + myc] : sDt[t] * sX[t * cols + myc], decay = CG ? 0.f : sDt[TB + t];
             const float4* b4 = reinterpret_cast<const float4*>(sB + t * Ns + ng * NL);
             const float4* c4 = reinterpret_cast<const float4*>(sC + t * Ns + ng * NL);
             float a0 = 0.f, a1 = 0.f;
 #pragma unroll
             for (int q = 0; q < NL / 4; ++q) {
                 const float4 bv = b4[q], cv = c4[q];
-                s[4 * q] = fmaf(decay, s[4 * q], bv.x * dx);         a0 = fmaf(s[4 * q], cv.x, a0);
-                s[4 * q + 1] = fmaf(decay, s[4 * q + 1], bv.y * dx); a1 = fmaf(s[4 * q + 1], cv.y, a1);
-                s[4 * q + 2] = fmaf(decay, s[4 * q + 2], bv.z * dx); a0 = fmaf(s[4 * q + 2], cv.z, a0);
-                s[4 * q + 3] = fmaf(decay, s[4 * q + 3], bv.w * dx); a1 = fmaf(s[4 * q + 3], cv.w, a1);
+                s[4 * q] = CG ? fmaf(bv.x, dx - s[4 * q], s[4 * q]) : fmaf(decay, s[4 * q], bv.x * dx);         a0 = fmaf(s[4 * q], cv.x, a0);
+                s[4 * q + 1] = CG ? fmaf(bv.y, dx - s[4 * q + 1], s[4 * q + 1]) : fmaf(decay, s[4 * q + 1], bv.y * dx); a1 = fmaf(s[4 * q + 1], cv.y, a1);
+                s[4 * q + 2] = CG ? fmaf(bv.z, dx - s[4 * q + 2], s[4 * q + 2]) : fmaf(decay, s[4 * q + 2], bv.z * dx); a0 = fmaf(s[4 * q + 2], cv.z, a0);
+                s[4 * q + 3] = CG ? fmaf(bv.w, dx - s[4 * q + 3], s[4 * q + 3]) : fmaf(decay, s[4 * q + 3], bv.w * dx); a1 = fmaf(s[4 * q + 3], cv.w, a1);
             }
             sY[t * 256 + tid] = a0 + a1;
         }
@@ -1159,15 +1234,16 @@ static __global__ __launch_bounds__(256) void hy_mem_gates_kernel(const float* _
 
 // What leaves a matrix memory: one wavefront per (token, head).  o = y[0 .. V) of the head (row stride ldy, P = V or V + 1 columns per
 // head), divided by max(|y[V]|, ge[t][head]) + 1e-6 where the memory has a normaliser (ge != null); then o / sqrt(mean(o^2) + eps), times
-// w[head V + c] (null = none), times act(gate[t][g_off + head V + c]) (act = silu, or sigmoid for gate_act 1), times out_mul, stored in the
-// matrix type at out[t ldo + head V + c].
+// w[head w_stride + c] (null = none; w_stride = V, or 0 for a weight the heads share), times act(gate[t][g_off + head V + c]) (act = silu, or
+// sigmoid for gate_act 1; gate = null: none), times out_mul, stored in the matrix type at out[t ldo + head V + c].
 // NT threads per (token, head): 64 for portions of many tokens, 256 for a few (a thread's column loop is a chain of load round trips).
 template <typename TO, int NT>
 static __global__ __launch_bounds__(NT) void hy_mem_out_kernel(const float* __restrict__ y, int ldy, int P, int V, const float* __restrict__ ge, int heads,
                                                                const float* __restrict__ w, const float* __restrict__ gate, int ldg, int g_off, int gate_act,
-                                                               float eps, float out_mul, TO* __restrict__ out, int ldo) {
+                                                               float eps, float out_mul, TO* __restrict__ out, int ldo, int w_stride) {
     __shared__ float red[NT / 64];
     const int t = blockIdx.x, head = blockIdx.y, tid = threadIdx.x;
+    auto act = [&](float z) { return !gate ? 1.f : gate_act == 1 ? hy_sigmoid(z) : hy_silu(z); };
     const float* row = y + (size_t)t * ldy + (size_t)head * P;
     float inv = 1.f;
     if (ge) inv = 1.f / (fmaxf(fabsf(row[V]), ge[(size_t)t * heads + head]) + 1e-6f);
@@ -1177,8 +1253,8 @@ static __global__ __launch_bounds__(NT) void hy_mem_out_kernel(const float* __re
     for (int u = 0; u < 2; ++u) {
         const int c = tid + u * NT;
         keep[u] = c < V ? row[c] * inv : 0.f;
-        kz[u] = c < V ? gate[(size_t)t * ldg + g_off + head * V + c] : 0.f;
-        kw[u] = (c < V && w) ? w[head * V + c] : 1.f;
+        kz[u] = (c < V && gate) ? gate[(size_t)t * ldg + g_off + head * V + c] : 0.f;
+        kw[u] = (c < V && w) ? w[head * w_stride + c] : 1.f;
     }
     float ss = keep[0] * keep[0] + keep[1] * keep[1];
     for (int c = tid + 2 * NT; c < V; c += NT) { const float v = row[c] * inv; ss += v * v; }
@@ -1188,12 +1264,11 @@ static __global__ __launch_bounds__(NT) void hy_mem_out_kernel(const float* __re
 #pragma unroll
     for (int u = 0; u < 2; ++u) {
         const int c = tid + u * NT;
-        if (c < V) hy_st(out + (size_t)t * ldo + head * V + c, keep[u] * r * kw[u] * (gate_act == 1 ? hy_sigmoid(kz[u]) : hy_silu(kz[u])) * out_mul);
+        if (c < V) hy_st(out + (size_t)t * ldo + head * V + c, keep[u] * r * kw[u] * act(kz[u]) * out_mul);
     }
     for (int c = tid + 2 * NT; c < V; c += NT) {
-        const float z = gate[(size_t)t * ldg + g_off + head * V + c];
-        const float gv = gate_act == 1 ? hy_sigmoid(z) : hy_silu(z);
-        hy_st(out + (size_t)t * ldo + head * V + c, row[c] * inv * r * (w ? w[head * V + c] : 1.f) * gv * out_mul);
+        const float gv = act(gate ? gate[(size_t)t * ldg + g_off + head * V + c] : 0.f);
+        hy_st(out + (size_t)t * ldo + head * V + c, row[c] * inv * r * (w ? w[head * w_stride + c] : 1.f) * gv * out_mul);
     }
 }
 
@@ -1214,4 +1289,53 @@ static __global__ __launch_bounds__(256) void hy_gated_norm_kernel(const float* 
         const float v = y[(size_t)t * inner + c0 + i] * hy_silu(proj[(size_t)t * ld + z_off + c0 + i]);
         hy_st(out + (size_t)t * ldo + c0 + i, v * r * w[c0 + i]);
     }
+}
+
+// Feed-forward activation over a token's whole vector: z[0 .. ff) (the sum of `parts` K-split partial products, pstride apart) becomes
+// c0 N(z) + c1 N(z^2) + c2 N(z^3) + c3, powers element by element, N(x) = x / sqrt(mean(x^2) + eps); written in the matrix type, zeros in
+// the columns ff .. ld - 1.  One workgroup per token; the first HY_PN_RC chunks of four columns of a thread stay in registers between the sums
+// (of z^2, z^4 and z^6) and the polynomial.  ld is a multiple of 4.
+constexpr int HY_PN_RC = 4;
+template <typename TO, int NT>
+static __global__ __launch_bounds__(NT) void hy_polynorm_kernel(const float* __restrict__ z, int ld, int ff, int parts, size_t pstride, const float* __restrict__ coef, float eps,
+                                                                TO* __restrict__ out) {
+    __shared__ float red[NT / 64];
+    const int t = blockIdx.x;
+    const float* row = z + (size_t)t * ld;
+    auto load = [&](int c) {
+        float4 v = *reinterpret_cast<const float4*>(row + c);
+        for (int p = 1; p < parts; ++p) { const float4 q = *reinterpret_cast<const float4*>(row + p * pstride + c); v.x += q.x; v.y += q.y; v.z += q.z; v.w += q.w; }
+        return v;
+    };
+    float s2 = 0.f, s4 = 0.f, s6 = 0.f;
+    auto add = [&](const float4& v) {          // (columns behind ff are products with zero rows)
+        const float e[4] = {v.x, v.y, v.z, v.w};
+#pragma unroll
+        for (int i = 0; i < 4; ++i) { const float q = e[i] * e[i], c = q * e[i]; s2 += q; s4 = fmaf(q, q, s4); s6 = fmaf(c, c, s6); }
+    };
+    float4 keep[HY_PN_RC];
+#pragma unroll
+    for (int u = 0; u < HY_PN_RC; ++u) {
+        const int c = (threadIdx.x + u * NT) * 4;
+        keep[u] = c < ld ? load(c) : make_float4(0.f, 0.f, 0.f, 0.f);
+    }
+#pragma unroll
+    for (int u = 0; u < HY_PN_RC; ++u) add(keep[u]);
+    for (int c = (threadIdx.x + HY_PN_RC * NT) * 4; c < ld; c += NT * 4) add(load(c));
+    s2 = hy_block_sum<NT>(s2, red);
+    s4 = hy_block_sum<NT>(s4, red);
+    s6 = hy_block_sum<NT>(s6, red);
+    const float m = 1.f / (float)ff;
+    const float k1 = coef[0] / sqrtf(s2 * m + eps), k2 = coef[1] / sqrtf(s4 * m + eps), k3 = coef[2] / sqrtf(s6 * m + eps), k0 = coef[3];
+    auto put = [&](int c, const float4& v) {
+        const float e[4] = {v.x, v.y, v.z, v.w};
+#pragma unroll
+        for (int i = 0; i < 4; ++i) hy_st(out + (size_t)t * ld + c + i, c + i < ff ? fmaf(fmaf(fmaf(k3, e[i], k2), e[i], k1), e[i], k0) : 0.f);
+    };
+#pragma unroll
+    for (int u = 0; u < HY_PN_RC; ++u) {
+        const int c = (threadIdx.x + u * NT) * 4;
+        if (c < ld) put(c, keep[u]);
+    }
+    for (int c = (threadIdx.x + HY_PN_RC * NT) * 4; c < ld; c += NT * 4) put(c, load(c));
 }

@@ -9,21 +9,27 @@
 // One workgroup per token.  In this order, every part optional (null pointer = absent):
 //   d  = ya_mul * ga * sum_z ya[z]              ya: a sublayer's output (or several sublayers' outputs), possibly as K-split parts; ga = sigmoid(gate_z[t * gate_ld]) or 1
 //   d += sum_k ew[t top + k] eo[pair_row[t top + k]]   the routed experts' down projections of this token (ew: a weight per pair, null = 1)
-//   x += d, or with post_w: x += d / sqrt(mean(d^2) + eps) * post_w    (the sublayer's output passes a norm of its own before it joins the residual)
+//   x += d, or with post_w: x += d / sqrt(mean(d^2) + eps) * post_w    (the sublayer's output passes a norm of its own before it joins the residual);
+//                                               with lw the addend is multiplied by lw[w] first (a scale per column)
 //   x += yc / sqrt(mean(yc^2) + eps) * cw       a unit-RMS normed input with a plain weight
 //   hist_out[t] = x;  x = sum_j mix[j] hist[j][t], j < n_mix, where hist[n_mix - 1] is hist_out (what the layer leaves is an average over
 //                                               the embedding output and every layer's result so far)
 //   x is written back; xt = x in the matrix type (operand of a following product); tap = x
-//   h = x / sqrt(mean(x^2) + eps) * norm_w in the matrix type (the next sublayer's input; norm_w already holds any offset)
+//   h = x / sqrt(mean(x^2) + eps) * norm_w in the matrix type (the next sublayer's input; norm_w already holds any offset); hf != null: in
+//                                               float32 to hf instead (hy_shift_kernel reads it)
+//   with shift_mu (a step of ONE token): h + (h' - h) shift_mu[w] is written instead, h' = the slot's row shift_prev (zeros at position 0),
+//                                               which becomes h
 struct HyResid {
     float* x; int W;
     const float* ya; int ya_parts; size_t ya_stride; const float* gate_z; int gate_ld; float ya_mul;
     const float* eo; const int* pair_row; int top; const float* ew;
-    const float* post_w;
+    const float* post_w; const float* lw;
     const float* yc; const float* cw;
     float* hist; size_t hist_stride; int n_mix; const float* mix;      // hist_out = hist + (n_mix - 1) hist_stride
     float* tap;
     const float* norm_w; float eps;
+    float* hf;
+    const float* shift_mu; float* shift_prev; size_t slot_stride; const int* dyn;
 };
 // V = 4: rows are read and written 16 bytes at a time (W a multiple of 4); every load of a chunk is issued before the first use, so one
 // round trip to memory covers them all.  The first HY_RC chunks of a thread stay in registers for the norm's second pass.
@@ -127,7 +133,20 @@ static __global__ __launch_bounds__(NT) void hy_resid_kernel(HyResid a, TO* __re
             float pw[V];
             hy_ldv<V>(a.post_w + w, pw);
 #pragma unroll
-            for (int i = 0; i < V; ++i) x[i] += (ga * y[i] + e[i]) * pr * pw[i];
+            for (int i = 0; i < V; ++i) y[i] = (ga * y[i] + e[i]) * pr * pw[i];
+            if (a.lw) {
+                float lw[V];
+                hy_ldv<V>(a.lw + w, lw);
+#pragma unroll
+                for (int i = 0; i < V; ++i) y[i] *= lw[i];
+            }
+#pragma unroll
+            for (int i = 0; i < V; ++i) x[i] += y[i];
+        } else if (a.lw) {
+            float lw[V];
+            hy_ldv<V>(a.lw + w, lw);
+#pragma unroll
+            for (int i = 0; i < V; ++i) x[i] = fmaf(ga * y[i] + e[i], lw[i], x[i]);
         } else {
 #pragma unroll
             for (int i = 0; i < V; ++i) {
@@ -176,6 +195,8 @@ static __global__ __launch_bounds__(NT) void hy_resid_kernel(HyResid a, TO* __re
     if (!a.norm_w) return;
     ss = hy_block_sum<NT>(ss, red);
     const float r = 1.f / sqrtf(ss / (float)W + a.eps);
+    float* prev = a.shift_mu ? a.shift_prev + (size_t)a.dyn[1] * a.slot_stride : nullptr;
+    const bool fresh = a.shift_mu && a.dyn[0] == 0;
     it = 0;
     for (int w = threadIdx.x * V; w < W; w += NT * V, ++it) {
         float x[V], nw[V];
@@ -189,7 +210,45 @@ static __global__ __launch_bounds__(NT) void hy_resid_kernel(HyResid a, TO* __re
         hy_ldv<V>(a.norm_w + w, nw);
 #pragma unroll
         for (int i = 0; i < V; ++i) x[i] = x[i] * r * nw[i];
-        hy_stv<V>(h_out + row + w, x);
+        if (a.shift_mu) {
+            float p[V], mu[V];
+            hy_ldv<V>(a.shift_mu + w, mu);
+#pragma unroll
+            for (int i = 0; i < V; ++i) p[i] = 0.f;
+            if (!fresh) hy_ldv<V>(prev + w, p);
+            hy_stv<V>(prev + w, x);
+#pragma unroll
+            for (int i = 0; i < V; ++i) x[i] = fmaf(p[i] - x[i], mu[i], x[i]);
+        }
+        if (a.hf) hy_stv<V>(a.hf + row + w, x);
+        else hy_stv<V>(h_out + row + w, x);
+    }
+}
+
+// Token shift of a step of n tokens: out[t] = h[t] + (h[t - 1] - h[t]) mu in the matrix type, h[-1] = the slot's row prev (zeros at position
+// 0), which becomes h[n - 1] (by the threads that have read it: token 0's).  Grid (n, column blocks).
+template <typename TO, int V>
+static __global__ __launch_bounds__(256) void hy_shift_kernel(const float* __restrict__ hf, int W, int n, const float* __restrict__ mu, float* __restrict__ prev, size_t slot_stride,
+                                                              const int* __restrict__ dyn, TO* __restrict__ out) {
+    const int t = blockIdx.x;
+    const float* row = hf + (size_t)t * W;
+    float* sp = prev + (size_t)dyn[1] * slot_stride;
+    for (int w = (blockIdx.y * 256 + threadIdx.x) * V; w < W; w += gridDim.y * 256 * V) {
+        float x[V], p[V], m[V];
+        hy_ldv<V>(row + w, x);
+        hy_ldv<V>(mu + w, m);
+        if (t > 0) hy_ldv<V>(row - W + w, p);
+        else {
+#pragma unroll
+            for (int i = 0; i < V; ++i) p[i] = 0.f;
+            if (dyn[0] > 0) hy_ldv<V>(sp + w, p);
+            float last[V];
+            hy_ldv<V>(hf + (size_t)(n - 1) * W + w, last);
+            hy_stv<V>(sp + w, last);
+        }
+#pragma unroll
+        for (int i = 0; i < V; ++i) x[i] = fmaf(p[i] - x[i], m[i], x[i]);
+        hy_stv<V>(out + (size_t)t * W + w, x);
     }
 }
 
@@ -212,13 +271,15 @@ static __global__ __launch_bounds__(256) void hy_side_act_kernel(const float* __
 // pstride apart); score = sigmoid(z), or softmax(z) over all E experts (HyRoute.softmax); the `top` largest of score (+ bias[e], where
 // bias != null: it decides the choice only) are taken in descending order (the lowest index wins a tie): sel[t top + k], wgt[t top + k] =
 // the chosen expert's score (without the bias), divided by the chosen scores' sum + 1e-20 (renorm), times mul.  E <= 64 * HY_RT_PER, top <= 64.
+// groups > 0: the experts form that many equal runs of neighbours; a run's score is the sum of its two largest choice scores, and only
+// experts of the `keep` best runs (the lowest index wins a tie) can be chosen (top <= keep E / groups).
 // pair_row != null (a few tokens): the pairs keep their own order, pair_row[p] = p.  extra_out != null: column E of z (the shared
 // expert's gate logit) is summed into extra_out[t].
 constexpr int HY_RT_PER = 16;
-struct HyRoute { int softmax; const float* bias; int renorm; float mul; };
+struct HyRoute { int softmax; const float* bias; int renorm; float mul; int groups, keep; };
 static __global__ __launch_bounds__(64) void hy_route_kernel(const float* __restrict__ z, int ldz, int parts, size_t pstride, int E, int top, int* __restrict__ sel,
                                                              float* __restrict__ wgt, int* __restrict__ pair_row, float* __restrict__ extra_out,
-                                                             HyRoute rt = HyRoute{0, nullptr, 0, 1.f}) {
+                                                             HyRoute rt = HyRoute{0, nullptr, 0, 1.f, 0, 0}) {
     const int t = blockIdx.x, lane = threadIdx.x;
     constexpr float GONE = -3.0e38f;
     float s[HY_RT_PER], c[HY_RT_PER];          // score; what the choice goes by
@@ -249,6 +310,35 @@ static __global__ __launch_bounds__(64) void hy_route_kernel(const float* __rest
     for (int i = 0; i < HY_RT_PER; ++i) {
         const int e = lane + 64 * i;
         c[i] = e < E ? s[i] + (rt.bias ? rt.bias[e] : 0.f) : GONE;
+    }
+    if (rt.groups > 0) {
+        __shared__ float cs[64 * HY_RT_PER], gsc[64 * HY_RT_PER];
+        const int gs = E / rt.groups;
+#pragma unroll
+        for (int i = 0; i < HY_RT_PER; ++i)
+            if (lane + 64 * i < E) cs[lane + 64 * i] = c[i];
+        __syncthreads();
+        for (int g = lane; g < rt.groups; g += 64) {
+            float b1 = cs[g * gs], b2 = GONE;
+            for (int j = 1; j < gs; ++j) {
+                const float v = cs[g * gs + j];
+                if (v > b1) { b2 = b1; b1 = v; } else if (v > b2) b2 = v;
+            }
+            gsc[g] = gs > 1 ? b1 + b2 : b1;
+        }
+        __syncthreads();
+        // an expert stays open if fewer than `keep` groups stand before its own
+#pragma unroll
+        for (int i = 0; i < HY_RT_PER; ++i) {
+            const int e = lane + 64 * i;
+            if (e < E) {
+                const int g = e / gs;
+                const float mine = gsc[g];
+                int before = 0;
+                for (int o = 0; o < rt.groups; ++o) before += (gsc[o] > mine || (gsc[o] == mine && o < g)) ? 1 : 0;
+                if (before >= rt.keep) c[i] = GONE;
+            }
+        }
     }
     float wsum = 0.f, myw = 0.f;          // lane k keeps the weight of choice k (top <= 64) until the sum is known
     int mysel = 0;

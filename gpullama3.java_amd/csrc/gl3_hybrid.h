@@ -1,5 +1,6 @@
 // gl3_hybrid.h — plan state of the layer-list family (GL3_ARCH_LAYERLIST) and the entry points the C-ABI dispatches to.
 #pragma once
+#include <bitset>
 #include <string>
 #include <vector>
 
@@ -7,6 +8,8 @@
 
 constexpr int HY_KSPLIT = 4;     // most partial sums a K-split output / down projection leaves for the streams kernel to add
 constexpr int HY_YPARTS = 2 * HY_KSPLIT;      // copies of y: in a parallel block the mixer's and the feed-forward's parts lie side by side
+
+typedef std::bitset<GL3_T_COUNT> HyHave;      // tensors that have arrived, by id
 
 struct HyMat {                 // [rows][ld] of the plan's matrix type (bfloat16 or float32), K-contiguous, zero padded
     void* w = nullptr;
@@ -27,7 +30,11 @@ struct HyLayer {
     HyLayer* side = nullptr;   // owned
     HyMat o;                   // the mixer's output projection [width x mo_total]
     float* pbias = nullptr;    // bias per row of the fused projection (null: no mixer of the layer has biases)
-    float *qn = nullptr, *kn = nullptr, *sink = nullptr;      // attention: weights of the whole-projection q / k norms, learned sink logits
+    float *qn = nullptr, *kn = nullptr, *sink = nullptr;      // attention: weights of the q / k norms (whole projection or per head), learned sink logits
+    float* qk_conv_w = nullptr;                               // attention: taps of the q and k channels, [taps][(heads + kv_heads) dim]
+    float* mem_lower = nullptr;                               // matrix memory, channel gates: lower bounds [heads dim]
+    float *shift_mu = nullptr, *ls1 = nullptr, *ls2 = nullptr, *poly = nullptr;      // token shift, layer scales, coefficients of the polynomial activation
+    size_t off_shift = 0;                                     // float offset inside a slot: the previous token's normed row
     float* decay = nullptr;    // matrix memory: fixed decay per head
     size_t off_pk = 0, off_pv = 0, off_m = 0;                 // float offsets inside a slot: pooled key / value rows, running maxima of the gates
     HyMat gu, down;            // feed-forward (in a mixture of experts: the shared expert): gate / up rows in blocks of 32 + 32 (2 ff_pad rows), down [width x ff_pad]
@@ -41,7 +48,9 @@ struct HyLayer {
     float* depth_mix = nullptr;
     HyMat side_gate, side_proj;
     float* side_norm = nullptr;
-    float *rot_freq = nullptr, *vrot_freq = nullptr;       // rotary tables: [rot_dims / 2] (position scaling applied), [vdim / 2]
+    // rotary tables: [rot_dims / 2] (position scaling applied; attention in double, matrix memory in float32), [vdim / 2]
+    double* rot_freq64 = nullptr;
+    float *rot_freq = nullptr, *vrot_freq = nullptr;
     float *norm1 = nullptr, *norm2 = nullptr;
     float* hc[2][3] = {};      // per sublayer: in [S], out [S], mix [S x S]
     // latent: norm weight; key expansion [H D][R] (as stored: rows for the expansion GEMM, and [h][d][r] for carrying a query into the latent's
@@ -59,7 +68,7 @@ struct HyLayer {
     float* route_bias = nullptr;                     // mixture of experts: added to the scores for the choice
     float *conv_w = nullptr, *conv_b = nullptr, *dt_bias = nullptr, *a_log = nullptr, *dskip = nullptr, *ssm_norm = nullptr;
     size_t off_k = 0, off_v = 0, off_state = 0, off_tail = 0;       // float offsets inside a sequence slot
-    uint64_t have = 0;
+    HyHave have;
 };
 
 struct gl3_hybrid_state {
@@ -71,6 +80,10 @@ struct gl3_hybrid_state {
     float emb_scale = 1.f, norm_offset = 0.f;
     int side_dim = 0, side_ld = 0, max_top = 0;
     bool depth = false;
+    bool shift = false, lscale = false;              // token shift in front of every mixer; a scale per column behind every sublayer
+    HyMat bigram;              // rows of token pairs [buckets + 1][W] (buckets = 0: none)
+    int bg_buckets = 0, bg_prev = 0, bg_cur = 0;
+    float *hf = nullptr, *ffz = nullptr;             // normed rows in float32 [mb][W]; up products of a polynomial feed-forward, K-split parts of [mb][ff_pad]
     bool post_norms = false;   // every sublayer's output passes an RMS norm with its own weight before it joins the residual
     float softcap = 0.f;       // logits <- cap tanh(logits / cap); 0 = none
     void* cq = nullptr;        // latent with q_rank: the normed query latents [mb][max q_rank], matrix type
@@ -83,12 +96,13 @@ struct gl3_hybrid_state {
     std::vector<HyLayer> L;
     HyMat emb, head;
     float* final_norm = nullptr;
-    uint64_t have = 0;
+    HyHave have;
     // sequence slots: cache rows and recurrent state of every layer, [n_seqs][slot_floats]
     float* slots = nullptr;
     size_t slot_floats = 0;
     std::vector<char> busy;
     std::vector<int> len;      // tokens a slot holds
+    std::vector<int> last_tok; // the last of them
     // scratch of one portion of a step (<= mb tokens)
     float *X = nullptr, *proj = nullptr, *y = nullptr, *conv = nullptr, *ssm_y = nullptr, *qa = nullptr, *oc = nullptr, *kx = nullptr, *vx = nullptr, *part_acc = nullptr, *part_ml = nullptr;
     float *gates = nullptr, *rowr = nullptr;     // matrix memory: a, b, e^(-m) per (token, head), [3][mb][max heads]; attention: 1 / rms of the whole q and k rows [mb][2]

@@ -1,10 +1,11 @@
 // gl3_hybrid.hip — the layer-list family (GL3_ARCH_LAYERLIST) behind the C-ABI: a model is a list of layers, each with its own token mixer
 // (softmax attention over cached keys / values, attention over a cached low-rank latent — optionally with a query latent, a rotated key
 // part shared by all heads and rows that a later layer reads too —, a state-space recurrence, a matrix memory with a fixed decay or
-// exponential gates), an optional feed-forward (gated or relu^2, dense or a mixture of experts with a shared expert and a sigmoid or
-// softmax router), and either several residual streams that per-sublayer tables read from and write to, or one plain residual stream
-// with an optional per-layer token input, a weighted average over all earlier layers' results, one norm for both sublayers of a layer, or
-// a norm behind every sublayer as well as in front of it.
+// exponential gates or a gate per key channel), an optional feed-forward (gated, relu^2 or a normed polynomial, dense or a mixture of
+// experts with a shared expert and a sigmoid or softmax router, optionally over groups of experts), and either several residual streams
+// that per-sublayer tables read from and write to, or one plain residual stream with an optional per-layer token input, a weighted average
+// over all earlier layers' results, one norm for both sublayers of a layer, a norm or a scale per column behind every sublayer, a token
+// shift in front of every mixer, and an embedding row per token pair.
 //
 // Plan: matrices live in HBM as bfloat16 (default) or widened to float32 (GL3_FLAG_F32_COMPUTE); every sequence slot owns the cache
 // rows and the recurrent state of all layers; a step runs the next n tokens of one slot in portions of at most max_batch tokens:
@@ -23,6 +24,7 @@
 using gl3::AMX_WGS;
 using gl3::argmax_kernel;
 
+#define HY_BIT(id) (HyHave().set(id))
 #define HY_HIP(call)                                                                                   \
     do {                                                                                               \
         hipError_t e_ = (call);                                                                        \
@@ -56,20 +58,22 @@ static int32_t hy_alloc_mat(gl3_ctx* ctx, HyMat& m, int rows, int k, int ld) {
 }
 
 // ---- shapes -----------------------------------------------------------------------------------------------------------------------
-static int hy_gate_rows(const gl3_layer_desc& d) { return d.mixer == GL3_MIX_MEMORY ? d.heads * d.vdim : d.out_gate == 2 ? d.heads : d.out_gate ? d.heads * d.vdim : 0; }
+static int hy_gate_rows(const gl3_layer_desc& d) { return d.mixer == GL3_MIX_MEMORY ? (d.mem_gate_act == 2 ? 0 : d.heads * d.vdim) : d.out_gate == 2 ? d.heads : d.out_gate ? d.heads * d.vdim : 0; }
 // rows of ONE mixer's part of the fused input projection
 static int hy_proj_rows(const gl3_layer_desc& d) {
     switch (d.mixer) {
-        case GL3_MIX_ATTENTION: return d.heads * d.dim + d.kv_heads * d.dim + d.kv_heads * d.vdim + hy_gate_rows(d);
+        case GL3_MIX_ATTENTION: return d.heads * d.dim + d.kv_heads * d.dim + (d.v_from_k ? 0 : d.kv_heads * d.vdim) + hy_gate_rows(d);
         case GL3_MIX_LATENT: return (d.q_rank > 0 ? d.q_rank : d.heads * (d.dim + d.rot_dim)) + (d.kv_share > 0 ? 0 : d.kv_rank + d.rot_dim) + hy_gate_rows(d);
-        case GL3_MIX_MEMORY: return 2 * d.heads * d.dim + 2 * d.heads * d.vdim + (d.mem_gates == GL3_MEM_EXP_GATES ? 2 * d.heads : 0);
+        case GL3_MIX_MEMORY: return 2 * d.heads * d.dim + d.heads * d.vdim + hy_gate_rows(d) + (d.mem_gates == GL3_MEM_EXP_GATES ? 2 * d.heads : 0);
         default: return 2 * d.heads * d.vdim + 2 * d.groups * d.state + d.heads;
     }
 }
 static int hy_mix_out(const gl3_layer_desc& d) { return d.heads * d.vdim; }
 // the fused input projection may come in K-split parts (room for HY_KSPLIT copies in the plan's scratch)
 static bool hy_narrow_proj(const gl3_layer_desc& d) { return d.mixer == GL3_MIX_LATENT && d.q_rank > 0; }
-static bool hy_has_bias(const gl3_layer_desc& d) { return (d.mixer == GL3_MIX_ATTENTION && d.qk_bias) || (d.mixer == GL3_MIX_MEMORY && d.mem_gates == GL3_MEM_EXP_GATES); }
+static bool hy_has_bias(const gl3_layer_desc& d) { return (d.mixer == GL3_MIX_ATTENTION && d.qk_bias) || (d.mixer == GL3_MIX_MEMORY && d.mem_gates != GL3_MEM_DECAY); }
+static bool hy_ungated(const gl3_layer_desc& d) { return d.ff_act >= 2; }          // the feed-forward (experts and shared expert too) has up rows alone
+static int hy_qk_ch(const gl3_layer_desc& d) { return (d.heads + d.kv_heads) * d.dim; }
 static int hy_conv_ch(const gl3_layer_desc& d) { return d.heads * d.vdim + 2 * d.groups * d.state; }
 
 static const char* hy_check_layer(const gl3_layer_desc& d) {
@@ -79,15 +83,22 @@ static const char* hy_check_layer(const gl3_layer_desc& d) {
     if (d.experts < 0 || d.shared_ff < 0) return "experts and shared_ff must be >= 0";
     if (d.experts > 0) {
         if (d.ff < 1) return "mixture of experts: ff (one expert's width) must be positive";
-        if (d.ff_act == 2) return "mixture of experts: the experts are gated (ff_act 0 or 1)";
+        if (d.ff_act == 3) return "mixture of experts: the polynomial activation is for dense feed-forwards";
+        if (d.ff_act == 2 && !d.route_on_output) return "mixture of experts: experts without a gate are weighted at their output (route_on_output)";
         if (d.experts + (d.shared_ff > 0 ? 1 : 0) > 64 * HY_RT_PER) return "mixture of experts: at most 1024 router rows (experts, plus one for a shared expert's gate)";
         if (d.top < 1 || d.top > d.experts || d.top > 64) return "mixture of experts: 1 <= top <= min(experts, 64)";
+        if (d.route_groups < 0 || (d.route_groups > 0 && (d.experts % d.route_groups || d.route_keep < 1 || d.route_keep > d.route_groups ||
+                                                          d.top > d.route_keep * (d.experts / d.route_groups))))
+            return "mixture of experts: route_groups must divide the experts and the route_keep best groups must hold at least top of them";
     } else if (d.shared_ff > 0)
         return "a shared expert needs a mixture of experts";
     if (d.mixer != GL3_MIX_ATTENTION && (d.v_unit_norm || d.v_rot || d.window > 0 || d.keep_first > 0 || d.pool > 0 || d.qk_bias))
         return "value norm / rotation, windows, pooled blocks and q / k / v biases belong to the attention mixer";
     if (d.mixer != GL3_MIX_ATTENTION && d.mixer != GL3_MIX_MEMORY && d.rot_dims) return "rotary positions belong to the attention and matrix-memory mixers";
-    if (d.ff_act < 0 || d.ff_act > 2) return "ff_act must be 0, 1 or 2";
+    if (d.mixer != GL3_MIX_ATTENTION && (d.qk_conv || d.v_from_k)) return "q / k convolutions and values taken from the keys belong to the attention mixer";
+    if (d.ff_act < 0 || d.ff_act > 3) return "ff_act must be 0, 1, 2 or 3";
+    if (d.rot_wave_factor < 0.f || (d.rot_wave_factor > 0.f && !(d.rot_wave_low > 0.f && d.rot_wave_high >= d.rot_wave_low && d.rot_wave_original > 0.f)))
+        return "frequencies rescaled by wavelength need original > 0 and 0 < low <= high";
     if (d.mixer != GL3_MIX_LATENT && (d.q_rank || d.rot_dim || d.kv_share)) return "q_rank, rot_dim and kv_share belong to the latent attention";
     if (d.mixer != GL3_MIX_MEMORY && (d.mem_qkv_act || d.mem_norm_whole)) return "mem_qkv_act and mem_norm_whole belong to the matrix memory";
     if (d.mixer == GL3_MIX_ATTENTION) {
@@ -98,7 +109,10 @@ static const char* hy_check_layer(const gl3_layer_desc& d) {
         if ((d.rot_dims || d.v_rot) && !(d.rot_base > 0.f)) return "attention: rot_base must be positive";
         if (d.v_rot && (d.vdim & 1)) return "attention: rotated values need an even vdim";
         if (d.keep_first < 0) return "attention: keep_first must be >= 0";
-        if (d.qk_unit_norm < 0 || d.qk_unit_norm > 2 || d.softmax_sink < 0 || d.softmax_sink > 2) return "attention: qk_unit_norm and softmax_sink must be 0, 1 or 2";
+        if (d.qk_unit_norm < 0 || d.qk_unit_norm > 3 || d.softmax_sink < 0 || d.softmax_sink > 2) return "attention: qk_unit_norm must be 0 .. 3, softmax_sink 0 .. 2";
+        if (d.qk_conv < 0 || d.qk_conv > 64) return "attention: 0 <= qk_conv <= 64";
+        if (d.v_from_k && (d.vdim != d.dim || d.v_unit_norm || d.v_rot)) return "attention: values taken from the keys need vdim = dim and no value norm or rotation";
+        if (d.qk_conv > 0 && (d.qk_unit_norm == 2 || d.qk_bias)) return "attention: q / k convolutions go without biases and without norms over a whole projection";
         if (d.pool < 0 || (d.pool > 0 && d.window <= 0)) return "attention: pooled blocks need a window";
         if (d.pool > 0 && d.slope_log2 != 0.f) return "attention: pooled blocks have no distance term";
     } else if (d.mixer == GL3_MIX_LATENT) {
@@ -113,7 +127,11 @@ static const char* hy_check_layer(const gl3_layer_desc& d) {
         if (d.dim < 1 || d.dim > 2048) return "matrix memory: 1 <= dim <= 2048";
         if (d.rot_dims < 0 || d.rot_dims > d.dim || (d.rot_dims & 1)) return "matrix memory: rot_dims must be even and at most dim";
         if (d.rot_dims && !(d.rot_base > 0.f)) return "matrix memory: rot_base must be positive";
-        if (d.mem_gates != GL3_MEM_DECAY && d.mem_gates != GL3_MEM_EXP_GATES) return "matrix memory: unknown mem_gates";
+        if (d.mem_gates != GL3_MEM_DECAY && d.mem_gates != GL3_MEM_EXP_GATES && d.mem_gates != GL3_MEM_CHANNEL_GATES) return "matrix memory: unknown mem_gates";
+        if (d.mem_gate_act < 0 || d.mem_gate_act > 2 || d.mem_norm_weight < 0 || d.mem_norm_weight > 2 || d.mem_qkv_act < 0 || d.mem_qkv_act > 2)
+            return "matrix memory: mem_gate_act, mem_norm_weight and mem_qkv_act must be 0, 1 or 2";
+        if (d.mem_norm_whole && d.mem_norm_weight == 2) return "matrix memory: one norm over all heads has a weight per entry";
+        if (d.mem_gates == GL3_MEM_CHANNEL_GATES && (d.rot_dims || d.mem_qkv_act == 1 || d.mem_norm_whole)) return "matrix memory: channel gates go without rotation, activated keys and a norm over all heads";
         if (d.mem_gates == GL3_MEM_DECAY && !d.mem_decay) return "matrix memory: a fixed decay needs mem_decay";
         if (d.mem_gates == GL3_MEM_EXP_GATES && !(d.mem_gate_cap > 0.f)) return "matrix memory: mem_gate_cap must be positive";
     } else if (d.mixer == GL3_MIX_SSM) {
@@ -137,6 +155,9 @@ int32_t gl3_hy_create(const gl3_model_desc* desc, gl3_ctx** out, std::string& er
     if (desc->weight_type != GL3_TYPE_BF16 && desc->weight_type != GL3_TYPE_F32) { err = "layer-list family: weight_type must be GL3_TYPE_BF16 (or GL3_TYPE_F32)"; return GL3_E_UNSUPPORTED; }
     if (desc->tp_size > 1) { err = "layer-list family: tensor parallelism is not built"; return GL3_E_UNSUPPORTED; }
     if (desc->post_norms && (desc->streams > 0 || desc->side_dim || desc->depth_mix || desc->parallel_block)) { err = "layer-list family: post norms need the plain residual without token input, depth average and parallel block"; return GL3_E_ARG; }
+    if (desc->streams > 0 && (desc->token_shift || desc->layer_scale || desc->bigram_buckets)) { err = "layer-list family: token shift, layer scales and token-pair embeddings need the plain residual (streams = 0)"; return GL3_E_ARG; }
+    if (desc->parallel_block && (desc->token_shift || desc->layer_scale)) { err = "layer-list family: token shift and layer scales need separate sublayers (no parallel block)"; return GL3_E_ARG; }
+    if (desc->bigram_buckets < 0 || desc->bigram_mul_prev < 0 || desc->bigram_mul_cur < 0) { err = "layer-list family: token-pair embedding: buckets and multipliers must be >= 0"; return GL3_E_ARG; }
     if (desc->logit_softcap < 0.f) { err = "layer-list family: logit_softcap must be >= 0"; return GL3_E_ARG; }
     if (desc->parallel_block && (desc->streams > 0 || desc->side_dim || desc->depth_mix)) { err = "layer-list family: the parallel block needs the plain residual without token input and depth average"; return GL3_E_ARG; }
     for (int l = 0; l < desc->n_layers; ++l) {
@@ -173,9 +194,11 @@ int32_t gl3_hy_create(const gl3_model_desc* desc, gl3_ctx** out, std::string& er
     h->depth = desc->depth_mix != 0;
     h->post_norms = desc->post_norms != 0;
     h->softcap = desc->logit_softcap;
+    h->shift = desc->token_shift != 0; h->lscale = desc->layer_scale != 0;
+    h->bg_buckets = desc->bigram_buckets; h->bg_prev = desc->bigram_mul_prev; h->bg_cur = desc->bigram_mul_cur;
     h->S = std::max(1, desc->streams); h->W = desc->dim; h->mb = std::max(1, desc->max_batch); h->n_seqs = ctx->n_seqs;
     h->want_cap = std::min(h->mb, 256);
-    h->busy.assign(h->n_seqs, 0); h->len.assign(h->n_seqs, 0);
+    h->busy.assign(h->n_seqs, 0); h->len.assign(h->n_seqs, 0); h->last_tok.assign(h->n_seqs, 0);
     auto fail = [&](int32_t code) { err = ctx->err; gl3_hy_destroy(ctx); if (ctx->stream) hipStreamDestroy(ctx->stream); if (ctx->argmax) hipFree(ctx->argmax);
                                     if (ctx->h_argmax) hipHostFree(ctx->h_argmax); if (ctx->h_dyn) hipHostFree(ctx->h_dyn); delete ctx; return code; };
 #define TRY(x) do { int32_t r_ = (x); if (r_ != GL3_OK) return fail(r_); } while (0)
@@ -187,9 +210,10 @@ int32_t gl3_hy_create(const gl3_model_desc* desc, gl3_ctx** out, std::string& er
     TRY(hy_alloc_mat(ctx, h->emb, V, W, W));
     TRY(hy_alloc_mat(ctx, h->head, V, W, W));
     TRY(hy_alloc(ctx, &h->final_norm, (size_t)W * 4));
+    if (h->bg_buckets > 0) TRY(hy_alloc_mat(ctx, h->bigram, h->bg_buckets + 1, W, W));
     h->L.resize(desc->n_layers);
     size_t slot = 0;
-    int max_proj = 1, max_mix = W, max_ch = 1, max_inner = 1, max_hr = 1, max_hdv = 1, max_kx = 0, max_vx = 0, max_rz = 0, max_top = 0, max_eff = 0, max_e = 0;
+    int max_proj = 1, max_mix = W, max_ch = 1, max_inner = 1, max_hr = 1, max_hdv = 1, max_kx = 0, max_vx = 0, max_rz = 0, max_top = 0, max_eff = 0, max_e = 0, max_poly = 0;
     if (h->side_dim > 0) TRY(hy_alloc_mat(ctx, h->side_emb, V, desc->n_layers * h->side_dim, desc->n_layers * h->side_dim));
     int max_heads = 1, max_qr = 0, max_qfull = 0;
     bool long_latent = false;
@@ -201,18 +225,48 @@ int32_t gl3_hy_create(const gl3_model_desc* desc, gl3_ctx** out, std::string& er
         Ly.out_mul = d.out_scale != 0.f ? d.out_scale : 1.f;
         max_heads = std::max(max_heads, d.heads);
 #define TRYM(x) do { int32_t r_ = (x); if (r_ != GL3_OK) return r_; } while (0)
-        // rotary tables, made in double: entry i turns by pos * base^(-2 i / dims) (q / k: divided by the position scaling)
-        auto table = [&](float** dst, int dims, double divide) -> int32_t {
-            std::vector<float> f(dims / 2);
-            for (int i = 0; i < dims / 2; ++i) f[i] = (float)(std::pow((double)d.rot_base, -2.0 * i / dims) / divide);
-            int32_t r_ = hy_alloc(ctx, dst, f.size() * 4);
+        // rotary tables, made in double: entry i turns by pos * f, f = base^(-2 i / dims); q / k with the position scaling: divided by a number,
+        // or rescaled by wavelength (long waves divided by the factor, short ones kept, a blend in between)
+        auto frequencies = [&](int dims, bool scaled) {
+            std::vector<double> f(dims / 2);
+            for (int i = 0; i < dims / 2; ++i) {
+                f[i] = std::pow((double)d.rot_base, -2.0 * i / dims);
+                if (!scaled) continue;
+                if (d.rot_divide > 0.f) f[i] /= (double)d.rot_divide;
+                if (d.rot_wave_factor > 0.f) {
+                    const double factor = d.rot_wave_factor, low = d.rot_wave_low, high = d.rot_wave_high, turns = d.rot_wave_original * f[i] / (2.0 * M_PI);          // original / wavelength
+                    if (turns < low) f[i] /= factor;
+                    else if (turns <= high && high > low) {
+                        const double s = (turns - low) / (high - low);
+                        f[i] = (1.0 - s) * f[i] / factor + s * f[i];
+                    }
+                }
+            }
+            return f;
+        };
+        auto put_table = [&](void** dst, const void* src, size_t bytes) -> int32_t {
+            int32_t r_ = hy_alloc(ctx, (uint8_t**)dst, bytes);
             if (r_ != GL3_OK) return r_;
-            return hipMemcpy(*dst, f.data(), f.size() * 4, hipMemcpyHostToDevice) == hipSuccess ? GL3_OK : GL3_E_HIP;
+            return hipMemcpy(*dst, src, bytes, hipMemcpyHostToDevice) == hipSuccess ? GL3_OK : GL3_E_HIP;
+        };
+        auto table = [&](float** dst, int dims, bool scaled) -> int32_t {
+            const std::vector<double> f = frequencies(dims, scaled);
+            const std::vector<float> f32(f.begin(), f.end());
+            return put_table((void**)dst, f32.data(), f32.size() * 4);
         };
         if (d.mixer == GL3_MIX_ATTENTION) {
-            Ly.q_off = p0; Ly.k_off = Ly.q_off + d.heads * d.dim; Ly.v_off = Ly.k_off + d.kv_heads * d.dim; Ly.g_off = Ly.v_off + d.kv_heads * d.vdim;
-            if (d.rot_dims > 0) TRYM(table(&Ly.rot_freq, d.rot_dims, d.rot_divide > 0.f ? (double)d.rot_divide : 1.0));
-            if (d.v_rot) TRYM(table(&Ly.vrot_freq, d.vdim, 1.0));
+            Ly.q_off = p0; Ly.k_off = Ly.q_off + d.heads * d.dim; Ly.v_off = Ly.k_off + d.kv_heads * d.dim; Ly.g_off = Ly.v_off + (d.v_from_k ? 0 : d.kv_heads * d.vdim);
+            if (d.rot_dims > 0) {
+                const std::vector<double> f = frequencies(d.rot_dims, true);
+                TRYM(put_table((void**)&Ly.rot_freq64, f.data(), f.size() * 8));
+            }
+            if (d.v_rot) TRYM(table(&Ly.vrot_freq, d.vdim, false));
+            if (d.qk_conv > 0) {
+                Ly.off_tail = slot; slot += (size_t)(d.qk_conv - 1) * hy_qk_ch(d);
+                slot = (slot + 63) & ~(size_t)63;          // (the cache rows behind it stay aligned)
+                TRYM(hy_alloc(ctx, &Ly.qk_conv_w, (size_t)d.qk_conv * hy_qk_ch(d) * 4));
+                max_ch = std::max(max_ch, d.heads * d.dim);          // the convolved, normed and turned queries
+            }
             Ly.off_k = slot; slot += (size_t)C * d.kv_heads * d.dim;
             Ly.off_v = slot; slot += (size_t)C * d.kv_heads * d.vdim;
             if (d.pool > 0) {          // one pooled row per complete block of `pool` positions
@@ -222,6 +276,10 @@ int32_t gl3_hy_create(const gl3_model_desc* desc, gl3_ctx** out, std::string& er
             if (d.qk_unit_norm == 2) {
                 TRYM(hy_alloc(ctx, &Ly.qn, (size_t)d.heads * d.dim * 4));
                 TRYM(hy_alloc(ctx, &Ly.kn, (size_t)d.kv_heads * d.dim * 4));
+            }
+            if (d.qk_unit_norm == 3) {
+                TRYM(hy_alloc(ctx, &Ly.qn, (size_t)d.dim * 4));
+                TRYM(hy_alloc(ctx, &Ly.kn, (size_t)d.dim * 4));
             }
             if (d.softmax_sink == 2) TRYM(hy_alloc(ctx, &Ly.sink, (size_t)d.heads * 4));
             max_hdv = std::max(max_hdv, d.heads * d.vdim);
@@ -270,16 +328,17 @@ int32_t gl3_hy_create(const gl3_model_desc* desc, gl3_ctx** out, std::string& er
             const bool eg = d.mem_gates == GL3_MEM_EXP_GATES;
             Ly.d.kv_heads = d.heads;
             Ly.q_off = p0; Ly.k_off = Ly.q_off + d.heads * d.dim; Ly.v_off = Ly.k_off + d.heads * d.dim; Ly.g_off = Ly.v_off + d.heads * d.vdim;
-            Ly.i_off = Ly.g_off + d.heads * d.vdim; Ly.f_off = Ly.i_off + d.heads;
-            if (d.rot_dims > 0) TRYM(table(&Ly.rot_freq, d.rot_dims, d.rot_divide > 0.f ? (double)d.rot_divide : 1.0));
+            Ly.i_off = Ly.g_off + hy_gate_rows(d); Ly.f_off = d.mem_gates == GL3_MEM_CHANNEL_GATES ? Ly.k_off : Ly.i_off + d.heads;          // channel gates stand in the keys' place
+            if (d.rot_dims > 0) TRYM(table(&Ly.rot_freq, d.rot_dims, true));
             const int P = d.vdim + (eg ? 1 : 0);             // exponential gates: one more state column carries the normaliser
             Ly.off_state = slot; slot += (size_t)d.heads * d.dim * P;
             if (eg) { Ly.off_m = slot; slot += (size_t)d.heads; }
+            else if (d.mem_gates == GL3_MEM_CHANNEL_GATES) TRYM(hy_alloc(ctx, &Ly.mem_lower, (size_t)d.heads * d.dim * 4));
             else {
                 TRYM(hy_alloc(ctx, &Ly.decay, (size_t)d.heads * 4));
                 if (hipMemcpy(Ly.decay, d.mem_decay, (size_t)d.heads * 4, hipMemcpyHostToDevice) != hipSuccess) { ctx->err = "copy of mem_decay failed"; return GL3_E_HIP; }
             }
-            if (d.mem_norm_weight) TRYM(hy_alloc(ctx, &Ly.ssm_norm, (size_t)d.heads * d.vdim * 4));
+            if (d.mem_norm_weight) TRYM(hy_alloc(ctx, &Ly.ssm_norm, (size_t)(d.mem_norm_weight == 2 ? 1 : d.heads) * d.vdim * 4));
             max_inner = std::max(max_inner, d.heads * P);
         } else {
             const int ch = hy_conv_ch(d), inner = d.heads * d.vdim;
@@ -321,6 +380,14 @@ int32_t gl3_hy_create(const gl3_model_desc* desc, gl3_ctx** out, std::string& er
             TRY(hy_alloc(ctx, &Ly.hc[q][2], (size_t)S * S * 4));
         }
         max_proj = std::max(max_proj, (hy_narrow_proj(d) && !bd ? HY_KSPLIT : 1) * np); max_mix = std::max(max_mix, mo);
+        if (h->shift) {          // first in the layer's part of the slot: 16-byte aligned
+            TRY(hy_alloc(ctx, &Ly.shift_mu, (size_t)W * 4));
+            Ly.off_shift = slot; slot += ((size_t)W + 63) & ~(size_t)63;
+        }
+        if (h->lscale) {
+            TRY(hy_alloc(ctx, &Ly.ls1, (size_t)W * 4));
+            if (d.ff > 0) TRY(hy_alloc(ctx, &Ly.ls2, (size_t)W * 4));
+        }
         TRY(setup_mixer(Ly, 0, 0));
         if (Ly.side) {
             Ly.side->pbias = Ly.pbias; Ly.side->mo_total = mo;
@@ -335,15 +402,16 @@ int32_t gl3_hy_create(const gl3_model_desc* desc, gl3_ctx** out, std::string& er
         }
         if (Ly.dense_ff > 0) {
             Ly.ff_pad = hy_cdiv(Ly.dense_ff, 32) * 32;
-            TRY(hy_alloc_mat(ctx, Ly.gu, (d.experts == 0 && d.ff_act == 2 ? 1 : 2) * Ly.ff_pad, W, W));          // without a gate: the up rows alone
+            TRY(hy_alloc_mat(ctx, Ly.gu, (hy_ungated(d) ? 1 : 2) * Ly.ff_pad, W, W));          // without a gate: the up rows alone
             TRY(hy_alloc_mat(ctx, Ly.down, W, Ly.ff_pad, Ly.ff_pad));
             max_mix = std::max(max_mix, Ly.ff_pad);
+            if (d.ff_act == 3) { TRY(hy_alloc(ctx, &Ly.poly, 4 * 4)); max_poly = std::max(max_poly, Ly.ff_pad); }
         }
         if (d.experts > 0) {
             Ly.eff_pad = hy_cdiv(d.ff, 32) * 32;
             TRY(hy_alloc_mat(ctx, Ly.router, d.experts + (d.shared_ff > 0 && !d.shared_ungated ? 1 : 0), W, W));
             if (d.route_bias) TRY(hy_alloc(ctx, &Ly.route_bias, (size_t)d.experts * 4));
-            TRY(hy_alloc_mat(ctx, Ly.egu, d.experts * 2 * Ly.eff_pad, W, W));
+            TRY(hy_alloc_mat(ctx, Ly.egu, d.experts * (hy_ungated(d) ? 1 : 2) * Ly.eff_pad, W, W));
             TRY(hy_alloc_mat(ctx, Ly.edown, d.experts * W, Ly.eff_pad, Ly.eff_pad));
             max_rz = std::max(max_rz, Ly.router.rows); max_top = std::max(max_top, d.top); max_eff = std::max(max_eff, Ly.eff_pad); max_e = std::max(max_e, d.experts);
         }
@@ -361,6 +429,8 @@ int32_t gl3_hy_create(const gl3_model_desc* desc, gl3_ctx** out, std::string& er
     TRY(hy_alloc(ctx, &h->h, (size_t)mb * W * es));
     TRY(hy_alloc(ctx, &h->proj, (size_t)mb * max_proj * 4));
     TRY(hy_alloc(ctx, &h->y, (size_t)HY_YPARTS * mb * W * 4));          // K-split partial sums of the output / down projections
+    if (h->shift) TRY(hy_alloc(ctx, &h->hf, (size_t)mb * W * 4));
+    if (max_poly > 0) TRY(hy_alloc(ctx, &h->ffz, (size_t)HY_KSPLIT * mb * max_poly * 4));
     h->max_heads = max_heads;
     TRY(hy_alloc(ctx, &h->gates, (size_t)3 * mb * max_heads * 4));
     TRY(hy_alloc(ctx, &h->rowr, (size_t)2 * mb * 4));
@@ -446,15 +516,16 @@ void gl3_hy_destroy(gl3_ctx* ctx) {
             if (!M) continue;
             f(M->lat_norm); f(M->wk); f(M->wv); f(M->wvT); f(M->conv_w); f(M->conv_b); f(M->dt_bias); f(M->a_log); f(M->dskip); f(M->ssm_norm);
             f(M->rot_freq); f(M->vrot_freq); f(M->qn); f(M->kn); f(M->sink); f(M->decay); f(M->uq.w); f(M->qlat_norm); f(M->lat_freq);
+            f(M->rot_freq64); f(M->qk_conv_w); f(M->mem_lower);
         }
         delete L.side;
         L.side = nullptr;
-        f(L.norm1b); f(L.norm2b); f(L.route_bias);
+        f(L.norm1b); f(L.norm2b); f(L.route_bias); f(L.shift_mu); f(L.ls1); f(L.ls2); f(L.poly);
         f(L.router.w); f(L.egu.w); f(L.edown.w); f(L.depth_mix); f(L.side_gate.w); f(L.side_proj.w); f(L.side_norm);
     }
     f(h->side_emb.w); f(h->sgz); f(h->hist); f(h->side_z); f(h->moe_z); f(h->wsel); f(h->eout); f(h->xb); f(h->side_g); f(h->ea); f(h->eact); f(h->sel); f(h->pair_row); f(h->tiles); f(h->ntiles);
     f(h->slots); f(h->X); f(h->h); f(h->proj); f(h->y); f(h->mixo); f(h->conv); f(h->ssm_y); f(h->qa); f(h->oc); f(h->kx); f(h->vx); f(h->part_acc); f(h->part_ml); f(h->gates); f(h->rowr);
-    f(h->cq); f(h->qfull);
+    f(h->cq); f(h->qfull); f(h->bigram.w); f(h->hf); f(h->ffz);
     f(h->xw); f(h->logits); f(h->taps); f(h->ones); f(h->dyn);
     hf(h->h_dyn); hf(h->h_logits);
     if (ctx->logits == h->logits) ctx->logits = nullptr;
@@ -519,14 +590,17 @@ int32_t gl3_hy_upload(gl3_ctx* ctx, int32_t id, int32_t layer, const void* host,
     const int W = h->W, S = h->S;
     constexpr int32_t NOT_MINE = -1000;
     int32_t r = NOT_MINE;
-    if (id == GL3_T_TOKEN_EMBD || id == GL3_T_OUTPUT || id == GL3_T_OUTPUT_NORM || id == GL3_T_SIDE_EMBD) {
+    if (id == GL3_T_TOKEN_EMBD || id == GL3_T_OUTPUT || id == GL3_T_OUTPUT_NORM || id == GL3_T_SIDE_EMBD || id == GL3_T_BIGRAM_EMBD) {
         if (id == GL3_T_TOKEN_EMBD) r = hy_put_rows(ctx, h->emb, 0, ctx->d.vocab, W, host, bytes, type, 0);
         else if (id == GL3_T_OUTPUT) r = hy_put_rows(ctx, h->head, 0, ctx->d.vocab, W, host, bytes, type, 0);
-        else if (id == GL3_T_SIDE_EMBD) {
+        else if (id == GL3_T_BIGRAM_EMBD) {
+            if (h->bg_buckets < 1) GL3_FAIL(GL3_E_ARG, "the model has no token-pair embedding");
+            r = hy_put_rows(ctx, h->bigram, 0, h->bg_buckets + 1, W, host, bytes, type, 0);
+        } else if (id == GL3_T_SIDE_EMBD) {
             if (h->side_dim < 1) GL3_FAIL(GL3_E_ARG, "the model has no per-layer token input");
             r = hy_put_rows(ctx, h->side_emb, 0, ctx->d.vocab, h->side_emb.k, host, bytes, type, 0);
         } else r = hy_put_vec(ctx, h->final_norm, W, host, bytes, type, h->norm_offset);
-        if (r == GL3_OK) h->have |= 1ull << id;
+        if (r == GL3_OK) h->have.set(id);
         return r;
     }
     const bool beside = layer >= 0 && (layer & GL3_LAYER_BESIDE);
@@ -537,7 +611,7 @@ int32_t gl3_hy_upload(gl3_ctx* ctx, int32_t id, int32_t layer, const void* host,
     HyLayer& L = beside ? *L0.side : L0;             // the mixer the tensor belongs to
     const gl3_layer_desc& d = L.d;
     const bool att = d.mixer == GL3_MIX_ATTENTION, lat = d.mixer == GL3_MIX_LATENT, ssm = d.mixer == GL3_MIX_SSM, mem = d.mixer == GL3_MIX_MEMORY;
-    const bool memg = mem && d.mem_gates == GL3_MEM_EXP_GATES;
+    const bool memg = mem && d.mem_gates == GL3_MEM_EXP_GATES, memc = mem && d.mem_gates == GL3_MEM_CHANNEL_GATES;
     const int mo = hy_mix_out(d);
     HyMat& proj = L0.proj;
     const size_t tes = type == GL3_TYPE_BF16 ? 2 : 4;          // bytes per element of the source
@@ -555,20 +629,36 @@ int32_t gl3_hy_upload(gl3_ctx* ctx, int32_t id, int32_t layer, const void* host,
         case GL3_T_Q_DOWN: if (lat && d.q_rank > 0) r = hy_put_rows(ctx, proj, L.q_off, d.q_rank, W, host, bytes, type, 0); break;
         case GL3_T_Q_DOWN_NORM: if (lat && d.q_rank > 0) r = hy_put_vec(ctx, L.qlat_norm, d.q_rank, host, bytes, type); break;
         case GL3_T_FFN_ROUTE_BIAS: if (d.experts > 0 && d.route_bias) r = hy_put_vec(ctx, L.route_bias, d.experts, host, bytes, type); break;
-        case GL3_T_WK: if (att || mem) r = hy_put_rows(ctx, proj, L.k_off, d.kv_heads * d.dim, W, host, bytes, type, 0); break;
-        case GL3_T_WV: if (att || mem) r = hy_put_rows(ctx, proj, L.v_off, d.kv_heads * d.vdim, W, host, bytes, type, 0); break;
-        case GL3_T_ATTN_GATE: if (((att || lat) && d.out_gate) || mem) r = hy_put_rows(ctx, proj, L.g_off, hy_gate_rows(d), W, host, bytes, type, 0); break;
+        case GL3_T_WK: if (att || (mem && !memc)) r = hy_put_rows(ctx, proj, L.k_off, d.kv_heads * d.dim, W, host, bytes, type, 0); break;
+        case GL3_T_WV: if ((att && !d.v_from_k) || mem) r = hy_put_rows(ctx, proj, L.v_off, d.kv_heads * d.vdim, W, host, bytes, type, 0); break;
+        case GL3_T_ATTN_GATE: if (hy_gate_rows(d) > 0 && !ssm) r = hy_put_rows(ctx, proj, L.g_off, hy_gate_rows(d), W, host, bytes, type, 0); break;
         case GL3_T_WO: r = hy_put_rows(ctx, L0.o, 0, W, mo, host, bytes, type, 0, L.o0); break;
         case GL3_T_BQ: if (att && d.qk_bias) r = hy_put_vec(ctx, L.pbias + L.q_off, (size_t)d.heads * d.dim, host, bytes, type); break;
         case GL3_T_BK: if (att && d.qk_bias) r = hy_put_vec(ctx, L.pbias + L.k_off, (size_t)d.kv_heads * d.dim, host, bytes, type); break;
         case GL3_T_BV: if (att && d.qk_bias) r = hy_put_vec(ctx, L.pbias + L.v_off, (size_t)d.kv_heads * d.vdim, host, bytes, type); break;
-        case GL3_T_ATTN_Q_NORM: if (att && d.qk_unit_norm == 2) r = hy_put_vec(ctx, L.qn, (size_t)d.heads * d.dim, host, bytes, type); break;
-        case GL3_T_ATTN_K_NORM: if (att && d.qk_unit_norm == 2) r = hy_put_vec(ctx, L.kn, (size_t)d.kv_heads * d.dim, host, bytes, type); break;
+        case GL3_T_ATTN_Q_NORM: if (att && d.qk_unit_norm >= 2) r = hy_put_vec(ctx, L.qn, (size_t)(d.qk_unit_norm == 3 ? 1 : d.heads) * d.dim, host, bytes, type); break;
+        case GL3_T_ATTN_K_NORM: if (att && d.qk_unit_norm >= 2) r = hy_put_vec(ctx, L.kn, (size_t)(d.qk_unit_norm == 3 ? 1 : d.kv_heads) * d.dim, host, bytes, type); break;
         case GL3_T_ATTN_SINK: if (att && d.softmax_sink == 2) r = hy_put_vec(ctx, L.sink, d.heads, host, bytes, type); break;
         case GL3_T_MEM_IGATE: if (memg) r = hy_put_rows(ctx, proj, L.i_off, d.heads, W, host, bytes, type, 0); break;
-        case GL3_T_MEM_FGATE: if (memg) r = hy_put_rows(ctx, proj, L.f_off, d.heads, W, host, bytes, type, 0); break;
+        case GL3_T_MEM_FGATE: if (memg || memc) r = hy_put_rows(ctx, proj, L.f_off, memc ? d.heads * d.dim : d.heads, W, host, bytes, type, 0); break;
         case GL3_T_MEM_IGATE_BIAS: if (memg) r = hy_put_vec(ctx, L.pbias + L.i_off, d.heads, host, bytes, type); break;
-        case GL3_T_MEM_FGATE_BIAS: if (memg) r = hy_put_vec(ctx, L.pbias + L.f_off, d.heads, host, bytes, type); break;
+        case GL3_T_MEM_FGATE_BIAS: if (memg || memc) r = hy_put_vec(ctx, L.pbias + L.f_off, memc ? (size_t)d.heads * d.dim : d.heads, host, bytes, type); break;
+        case GL3_T_MEM_LOWER: if (memc) r = hy_put_vec(ctx, L.mem_lower, (size_t)d.heads * d.dim, host, bytes, type); break;
+        case GL3_T_Q_CONV: case GL3_T_K_CONV:
+            if (att && d.qk_conv > 0) {          // [channels][taps] -> columns of [taps][all channels]
+                const int taps = d.qk_conv, C = hy_qk_ch(d), c0 = id == GL3_T_Q_CONV ? 0 : d.heads * d.dim, nc = (id == GL3_T_Q_CONV ? d.heads : d.kv_heads) * d.dim;
+                if (!hy_to_f32(host, bytes, type, (size_t)nc * taps, f)) GL3_FAIL(GL3_E_ARG, "tensor size or type mismatch");
+                std::vector<float> tr((size_t)nc * taps);
+                for (int c = 0; c < nc; ++c)
+                    for (int j = 0; j < taps; ++j) tr[(size_t)j * nc + c] = f[(size_t)c * taps + j];
+                HY_HIP(hipMemcpy2D(L.qk_conv_w + c0, (size_t)C * 4, tr.data(), (size_t)nc * 4, (size_t)nc * 4, taps, hipMemcpyHostToDevice));
+                r = GL3_OK;
+            }
+            break;
+        case GL3_T_TOKEN_SHIFT: if (!beside && h->shift) r = hy_put_vec(ctx, L.shift_mu, W, host, bytes, type); break;
+        case GL3_T_ATTN_SCALE: if (!beside && h->lscale) r = hy_put_vec(ctx, L.ls1, W, host, bytes, type); break;
+        case GL3_T_FFN_SCALE: if (L.ls2) r = hy_put_vec(ctx, L.ls2, W, host, bytes, type); break;
+        case GL3_T_FFN_POLY: if (L.poly) r = hy_put_vec(ctx, L.poly, 4, host, bytes, type); break;
         case GL3_T_KV_DOWN: if (lat && d.kv_share == 0) r = hy_put_rows(ctx, proj, L.c_off, L.Re, W, host, bytes, type, 0); break;
         case GL3_T_KV_DOWN_NORM: if (lat && d.kv_share == 0) r = hy_put_vec(ctx, L.lat_norm, d.kv_rank, host, bytes, type); break;
         case GL3_T_K_UP:
@@ -608,9 +698,9 @@ int32_t gl3_hy_upload(gl3_ctx* ctx, int32_t id, int32_t layer, const void* host,
         case GL3_T_SSM_DT_BIAS: if (ssm) r = hy_put_vec(ctx, L.dt_bias, d.heads, host, bytes, type); break;
         case GL3_T_SSM_A_LOG: if (ssm) r = hy_put_vec(ctx, L.a_log, d.heads, host, bytes, type); break;
         case GL3_T_SSM_D: if (ssm) r = hy_put_vec(ctx, L.dskip, d.heads, host, bytes, type); break;
-        case GL3_T_SSM_NORM: if (ssm || (mem && d.mem_norm_weight)) r = hy_put_vec(ctx, L.ssm_norm, mo, host, bytes, type); break;
-        case GL3_T_W1: if (L.dense_ff > 0 && (d.experts > 0 || d.ff_act != 2)) r = hy_put_rows(ctx, L.gu, 0, L.dense_ff, W, host, bytes, type, 1); break;
-        case GL3_T_W3: if (L.dense_ff > 0) r = hy_put_rows(ctx, L.gu, 0, L.dense_ff, W, host, bytes, type, (d.experts == 0 && d.ff_act == 2) ? 0 : 2); break;
+        case GL3_T_SSM_NORM: if (ssm || (mem && d.mem_norm_weight)) r = hy_put_vec(ctx, L.ssm_norm, (mem && d.mem_norm_weight == 2) ? d.vdim : mo, host, bytes, type); break;
+        case GL3_T_W1: if (L.dense_ff > 0 && !hy_ungated(d)) r = hy_put_rows(ctx, L.gu, 0, L.dense_ff, W, host, bytes, type, 1); break;
+        case GL3_T_W3: if (L.dense_ff > 0) r = hy_put_rows(ctx, L.gu, 0, L.dense_ff, W, host, bytes, type, hy_ungated(d) ? 0 : 2); break;
         case GL3_T_W2:
             if (L.dense_ff > 0) {          // [W][ff] into rows of ff_pad
                 if (!hy_to_f32(host, bytes, type, (size_t)W * L.dense_ff, f)) GL3_FAIL(GL3_E_ARG, "tensor size or type mismatch");
@@ -623,11 +713,11 @@ int32_t gl3_hy_upload(gl3_ctx* ctx, int32_t id, int32_t layer, const void* host,
         case GL3_T_FFN_GATE_INP: if (d.experts > 0) r = hy_put_rows(ctx, L.router, 0, d.experts, W, host, bytes, type, 0); break;
         case GL3_T_FFN_GATE_INP_SHEXP: if (d.experts > 0 && d.shared_ff > 0 && !d.shared_ungated) r = hy_put_rows(ctx, L.router, d.experts, 1, W, host, bytes, type, 0); break;
         case GL3_T_FFN_GATE_EXPS: case GL3_T_FFN_UP_EXPS:
-            if (d.experts > 0) {
+            if (d.experts > 0 && !(hy_ungated(d) && id == GL3_T_FFN_GATE_EXPS)) {
                 const size_t per = (size_t)d.ff * W * tes;
                 if (bytes != per * d.experts) GL3_FAIL(GL3_E_ARG, "tensor size or type mismatch");
                 for (int e = 0; e < d.experts; ++e) {
-                    r = hy_put_rows(ctx, L.egu, e * 2 * L.eff_pad, d.ff, W, (const uint8_t*)host + e * per, per, type, id == GL3_T_FFN_GATE_EXPS ? 1 : 2);
+                    r = hy_put_rows(ctx, L.egu, e * (hy_ungated(d) ? 1 : 2) * L.eff_pad, d.ff, W, (const uint8_t*)host + e * per, per, type, hy_ungated(d) ? 0 : id == GL3_T_FFN_GATE_EXPS ? 1 : 2);
                     if (r != GL3_OK) break;
                 }
             }
@@ -654,55 +744,67 @@ int32_t gl3_hy_upload(gl3_ctx* ctx, int32_t id, int32_t layer, const void* host,
         default: break;
     }
     if (r == NOT_MINE) GL3_FAIL(GL3_E_ARG, "tensor id " + std::to_string(id) + " does not belong to layer " + std::to_string(layer));
-    if (r == GL3_OK) L.have |= 1ull << id;
+    if (r == GL3_OK) L.have.set(id);
     return r;
 }
 
 // tensors of one mixer (second = the mixer beside the layer's first: it has no norm, tables or feed-forward of its own)
-static uint64_t hy_needed(const gl3_hybrid_state* h, const gl3_layer_desc& d, bool second = false) {
-    uint64_t m = 1ull << GL3_T_WO;
-    if (d.mixer == GL3_MIX_ATTENTION) m |= (1ull << GL3_T_WQ) | (1ull << GL3_T_WK) | (1ull << GL3_T_WV);
-    if (d.mixer == GL3_MIX_ATTENTION && d.qk_bias) m |= (1ull << GL3_T_BQ) | (1ull << GL3_T_BK) | (1ull << GL3_T_BV);
-    if (d.mixer == GL3_MIX_ATTENTION && d.qk_unit_norm == 2) m |= (1ull << GL3_T_ATTN_Q_NORM) | (1ull << GL3_T_ATTN_K_NORM);
-    if (d.mixer == GL3_MIX_ATTENTION && d.softmax_sink == 2) m |= 1ull << GL3_T_ATTN_SINK;
-    if (d.mixer == GL3_MIX_MEMORY) m |= (1ull << GL3_T_WQ) | (1ull << GL3_T_WK) | (1ull << GL3_T_WV) | (1ull << GL3_T_ATTN_GATE);
-    if (d.mixer == GL3_MIX_MEMORY && d.mem_norm_weight) m |= 1ull << GL3_T_SSM_NORM;
+static HyHave hy_needed(const gl3_hybrid_state* h, const gl3_layer_desc& d, bool second = false) {
+    HyHave m = HY_BIT(GL3_T_WO);
+    if (d.mixer == GL3_MIX_ATTENTION) m |= HY_BIT(GL3_T_WQ) | HY_BIT(GL3_T_WK);
+    if (d.mixer == GL3_MIX_ATTENTION && !d.v_from_k) m.set(GL3_T_WV);
+    if (d.mixer == GL3_MIX_ATTENTION && d.qk_conv > 0) m |= HY_BIT(GL3_T_Q_CONV) | HY_BIT(GL3_T_K_CONV);
+    if (d.mixer == GL3_MIX_ATTENTION && d.qk_bias) m |= (HY_BIT(GL3_T_BQ)) | (HY_BIT(GL3_T_BK)) | (HY_BIT(GL3_T_BV));
+    if (d.mixer == GL3_MIX_ATTENTION && d.qk_unit_norm >= 2) m |= (HY_BIT(GL3_T_ATTN_Q_NORM)) | (HY_BIT(GL3_T_ATTN_K_NORM));
+    if (d.mixer == GL3_MIX_ATTENTION && d.softmax_sink == 2) m |= HY_BIT(GL3_T_ATTN_SINK);
+    if (d.mixer == GL3_MIX_MEMORY) m |= HY_BIT(GL3_T_WQ) | HY_BIT(GL3_T_WV);
+    if (d.mixer == GL3_MIX_MEMORY && d.mem_gate_act != 2) m.set(GL3_T_ATTN_GATE);
+    if (d.mixer == GL3_MIX_MEMORY && d.mem_gates != GL3_MEM_CHANNEL_GATES) m.set(GL3_T_WK);
+    if (d.mixer == GL3_MIX_MEMORY && d.mem_gates == GL3_MEM_CHANNEL_GATES) m |= HY_BIT(GL3_T_MEM_FGATE) | HY_BIT(GL3_T_MEM_FGATE_BIAS) | HY_BIT(GL3_T_MEM_LOWER);
+    if (d.mixer == GL3_MIX_MEMORY && d.mem_norm_weight) m |= HY_BIT(GL3_T_SSM_NORM);
     if (d.mixer == GL3_MIX_MEMORY && d.mem_gates == GL3_MEM_EXP_GATES)
-        m |= (1ull << GL3_T_MEM_IGATE) | (1ull << GL3_T_MEM_FGATE) | (1ull << GL3_T_MEM_IGATE_BIAS) | (1ull << GL3_T_MEM_FGATE_BIAS);
+        m |= (HY_BIT(GL3_T_MEM_IGATE)) | (HY_BIT(GL3_T_MEM_FGATE)) | (HY_BIT(GL3_T_MEM_IGATE_BIAS)) | (HY_BIT(GL3_T_MEM_FGATE_BIAS));
     if (second) return m;
-    m |= 1ull << GL3_T_ATTN_NORM;
-    if (!h->plain) m |= (1ull << GL3_T_HC1_IN) | (1ull << GL3_T_HC1_OUT) | (1ull << GL3_T_HC1_MIX);
-    if (h->depth) m |= 1ull << GL3_T_DEPTH_MIX;
-    if (h->side_dim > 0) m |= (1ull << GL3_T_SIDE_GATE) | (1ull << GL3_T_SIDE_PROJ) | (1ull << GL3_T_SIDE_NORM);
-    if (d.mixer == GL3_MIX_LATENT) m |= (1ull << GL3_T_WQ) | (1ull << GL3_T_K_UP) | (1ull << GL3_T_V_UP);
-    if (d.mixer == GL3_MIX_LATENT && d.kv_share == 0) m |= (1ull << GL3_T_KV_DOWN) | (1ull << GL3_T_KV_DOWN_NORM);
-    if (d.mixer == GL3_MIX_LATENT && d.q_rank > 0) m |= (1ull << GL3_T_Q_DOWN) | (1ull << GL3_T_Q_DOWN_NORM);
-    if (h->post_norms) m |= (1ull << GL3_T_ATTN_POST_NORM) | (d.ff > 0 ? 1ull << GL3_T_FFN_POST_NORM : 0);
-    if (d.experts > 0 && d.route_bias) m |= 1ull << GL3_T_FFN_ROUTE_BIAS;
-    if ((d.mixer == GL3_MIX_ATTENTION || d.mixer == GL3_MIX_LATENT) && d.out_gate) m |= 1ull << GL3_T_ATTN_GATE;
+    m |= HY_BIT(GL3_T_ATTN_NORM);
+    if (!h->plain) m |= (HY_BIT(GL3_T_HC1_IN)) | (HY_BIT(GL3_T_HC1_OUT)) | (HY_BIT(GL3_T_HC1_MIX));
+    if (h->depth) m |= HY_BIT(GL3_T_DEPTH_MIX);
+    if (h->side_dim > 0) m |= (HY_BIT(GL3_T_SIDE_GATE)) | (HY_BIT(GL3_T_SIDE_PROJ)) | (HY_BIT(GL3_T_SIDE_NORM));
+    if (d.mixer == GL3_MIX_LATENT) m |= (HY_BIT(GL3_T_WQ)) | (HY_BIT(GL3_T_K_UP)) | (HY_BIT(GL3_T_V_UP));
+    if (d.mixer == GL3_MIX_LATENT && d.kv_share == 0) m |= (HY_BIT(GL3_T_KV_DOWN)) | (HY_BIT(GL3_T_KV_DOWN_NORM));
+    if (d.mixer == GL3_MIX_LATENT && d.q_rank > 0) m |= (HY_BIT(GL3_T_Q_DOWN)) | (HY_BIT(GL3_T_Q_DOWN_NORM));
+    if (h->post_norms) m |= (HY_BIT(GL3_T_ATTN_POST_NORM)) | (d.ff > 0 ? HY_BIT(GL3_T_FFN_POST_NORM) : HyHave());
+    if (d.experts > 0 && d.route_bias) m |= HY_BIT(GL3_T_FFN_ROUTE_BIAS);
+    if ((d.mixer == GL3_MIX_ATTENTION || d.mixer == GL3_MIX_LATENT) && d.out_gate) m |= HY_BIT(GL3_T_ATTN_GATE);
     if (d.mixer == GL3_MIX_SSM)
-        m |= (1ull << GL3_T_SSM_IN) | (1ull << GL3_T_SSM_CONV) | (1ull << GL3_T_SSM_CONV_BIAS) | (1ull << GL3_T_SSM_DT_BIAS) | (1ull << GL3_T_SSM_A_LOG) |
-             (1ull << GL3_T_SSM_D) | (1ull << GL3_T_SSM_NORM);
-    if (d.ff > 0 && !h->parallel) m |= 1ull << GL3_T_FFN_NORM;
-    if (d.ff > 0 && !h->plain) m |= (1ull << GL3_T_HC2_IN) | (1ull << GL3_T_HC2_OUT) | (1ull << GL3_T_HC2_MIX);
-    if (d.experts > 0) m |= (1ull << GL3_T_FFN_GATE_INP) | (1ull << GL3_T_FFN_GATE_EXPS) | (1ull << GL3_T_FFN_UP_EXPS) | (1ull << GL3_T_FFN_DOWN_EXPS);
-    if (d.experts > 0 && d.shared_ff > 0 && !d.shared_ungated) m |= 1ull << GL3_T_FFN_GATE_INP_SHEXP;
-    if (d.experts > 0 ? d.shared_ff > 0 : d.ff > 0) m |= (1ull << GL3_T_W2) | (1ull << GL3_T_W3) | ((d.experts > 0 || d.ff_act != 2) ? 1ull << GL3_T_W1 : 0);
+        m |= (HY_BIT(GL3_T_SSM_IN)) | (HY_BIT(GL3_T_SSM_CONV)) | (HY_BIT(GL3_T_SSM_CONV_BIAS)) | (HY_BIT(GL3_T_SSM_DT_BIAS)) | (HY_BIT(GL3_T_SSM_A_LOG)) |
+             (HY_BIT(GL3_T_SSM_D)) | (HY_BIT(GL3_T_SSM_NORM));
+    if (d.ff > 0 && !h->parallel) m |= HY_BIT(GL3_T_FFN_NORM);
+    if (h->shift) m.set(GL3_T_TOKEN_SHIFT);
+    if (h->lscale) { m.set(GL3_T_ATTN_SCALE); if (d.ff > 0) m.set(GL3_T_FFN_SCALE); }
+    if (d.ff > 0 && d.ff_act == 3) m.set(GL3_T_FFN_POLY);
+    if (d.ff > 0 && !h->plain) m |= (HY_BIT(GL3_T_HC2_IN)) | (HY_BIT(GL3_T_HC2_OUT)) | (HY_BIT(GL3_T_HC2_MIX));
+    if (d.experts > 0) m |= HY_BIT(GL3_T_FFN_GATE_INP) | HY_BIT(GL3_T_FFN_UP_EXPS) | HY_BIT(GL3_T_FFN_DOWN_EXPS);
+    if (d.experts > 0 && !hy_ungated(d)) m.set(GL3_T_FFN_GATE_EXPS);
+    if (d.experts > 0 && d.shared_ff > 0 && !d.shared_ungated) m |= HY_BIT(GL3_T_FFN_GATE_INP_SHEXP);
+    if (d.experts > 0 ? d.shared_ff > 0 : d.ff > 0) {
+        m |= HY_BIT(GL3_T_W2) | HY_BIT(GL3_T_W3);
+        if (!hy_ungated(d)) m.set(GL3_T_W1);
+    }
     return m;
 }
 
 int32_t gl3_hy_finalize(gl3_ctx* ctx) {
     gl3_hybrid_state* h = ctx->hy;
-    const uint64_t g = (1ull << GL3_T_TOKEN_EMBD) | (1ull << GL3_T_OUTPUT_NORM) | (h->side_dim > 0 ? 1ull << GL3_T_SIDE_EMBD : 0);
-    if ((h->have & g) != g) GL3_FAIL(GL3_E_STATE, "missing global tensors (token embedding / output norm / side embedding)");
-    if (!(h->have & (1ull << GL3_T_OUTPUT))) {           // tied head
+    const HyHave g = (HY_BIT(GL3_T_TOKEN_EMBD)) | (HY_BIT(GL3_T_OUTPUT_NORM)) | (h->side_dim > 0 ? HY_BIT(GL3_T_SIDE_EMBD) : HyHave()) | (h->bg_buckets > 0 ? HY_BIT(GL3_T_BIGRAM_EMBD) : HyHave());
+    if ((h->have & g) != g) GL3_FAIL(GL3_E_STATE, "missing global tensors (token embedding / output norm / side embedding / token-pair embedding)");
+    if (!h->have.test(GL3_T_OUTPUT)) {           // tied head
         HY_HIP(hipMemcpy(h->head.w, h->emb.w, (size_t)h->emb.rows * h->emb.ld * (h->f32 ? 4 : 2), hipMemcpyDeviceToDevice));
     }
     for (size_t l = 0; l < h->L.size(); ++l) {
-        const uint64_t need = hy_needed(h, h->L[l].d);
+        const HyHave need = hy_needed(h, h->L[l].d);
         if ((h->L[l].have & need) != need) GL3_FAIL(GL3_E_STATE, "layer " + std::to_string(l) + ": missing tensors");
         if (h->L[l].side) {
-            const uint64_t need2 = hy_needed(h, h->L[l].side->d, true);
+            const HyHave need2 = hy_needed(h, h->L[l].side->d, true);
             if ((h->L[l].side->have & need2) != need2) GL3_FAIL(GL3_E_STATE, "layer " + std::to_string(l) + ", second mixer: missing tensors");
         }
     }
@@ -843,7 +945,11 @@ static void hy_scan(gl3_ctx* ctx, HyScanArgs& a) {
     const size_t smem = ((size_t)TB * (2 * Ns + cols + 256) + 2 * TB) * 4;
     a.NG = NG; a.TB = TB;
     const dim3 grid(hy_cdiv(a.P, cols), a.heads);
-#define HY_SCAN(NLT) hipLaunchKernelGGL((hy_ssm_scan_kernel<NLT>), grid, dim3(256), smem, ctx->stream, a)
+#define HY_SCAN(NLT)                                                                                                       \
+    do {                                                                                                                   \
+        if (a.mode == 3) hipLaunchKernelGGL((hy_ssm_scan_kernel<NLT, 1>), grid, dim3(256), smem, ctx->stream, a);            \
+        else hipLaunchKernelGGL((hy_ssm_scan_kernel<NLT, 0>), grid, dim3(256), smem, ctx->stream, a);                        \
+    } while (0)
     if (NL == 4) HY_SCAN(4); else if (NL == 8) HY_SCAN(8); else if (NL == 16) HY_SCAN(16); else HY_SCAN(32);
 #undef HY_SCAN
 }
@@ -863,28 +969,37 @@ static int32_t hy_mixer_core(gl3_ctx* ctx, HyLayer& L, int np, int ldo, int n, i
         float* vc = h->slots + L.off_v;
         float* pk = d.pool > 0 ? h->slots + L.off_pk : nullptr;
         float* pv = d.pool > 0 ? h->slots + L.off_pv : nullptr;
-        const HyRot rot{d.rot_dims, L.rot_freq, d.v_unit_norm, d.v_rot ? L.vrot_freq : nullptr, d.rot_interleaved};
-        const HyPrepX px{d.qk_bias ? L.pbias : nullptr, L.qn, L.kn, h->rowr};
+        const HyRot rot{d.rot_dims, L.rot_freq64, d.v_unit_norm, d.v_rot ? L.vrot_freq : nullptr, d.rot_interleaved};
+        HyPrepX px{d.qk_bias ? L.pbias : nullptr, L.qn, L.kn, h->rowr, d.v_from_k};
+        const float* q = h->proj + L.q_off;
+        int ldq = np;
+        if (d.qk_conv > 0) {
+            px.conv_w = L.qk_conv_w; px.taps = d.qk_conv; px.tail = h->slots + L.off_tail; px.qout = h->conv; px.ldq = d.heads * d.dim; px.n = n;
+            q = h->conv; ldq = px.ldq;
+        }
         if (d.qk_unit_norm == 2) {
             if (n <= 32) hipLaunchKernelGGL((hy_rowrms_kernel<1024>), dim3(n, 2), dim3(1024), 0, st, h->proj, np, L.q_off, d.heads * d.dim, L.k_off, d.kv_heads * d.dim, px.bias, eps, h->rowr);
             else hipLaunchKernelGGL((hy_rowrms_kernel<256>), dim3(n, 2), dim3(256), 0, st, h->proj, np, L.q_off, d.heads * d.dim, L.k_off, d.kv_heads * d.dim, px.bias, eps, h->rowr);
         }
-        hipLaunchKernelGGL(hy_attn_prep_kernel, dim3(n, d.heads + 2 * d.kv_heads), dim3(64), 0, st, h->proj, np, L.q_off, L.k_off, L.v_off, d.heads, d.kv_heads, d.dim,
+        hipLaunchKernelGGL(hy_attn_prep_kernel, dim3(n, d.heads + (d.v_from_k ? 1 : 2) * d.kv_heads), dim3(64), 0, st, h->proj, np, L.q_off, L.k_off, L.v_off, d.heads, d.kv_heads, d.dim,
                            d.vdim, d.qk_unit_norm, eps, kc, vc, h->slot_floats, h->dyn, rot, px);
+        if (d.qk_conv > 1 && n > 1)          // (q and k stand side by side in the projection row; a single token's tail moved on above)
+            hipLaunchKernelGGL(hy_conv_tail_kernel, dim3(hy_cdiv(hy_qk_ch(d), 256)), dim3(256), 0, st, h->proj, np, L.q_off, hy_qk_ch(d), d.qk_conv, h->slots + L.off_tail,
+                               h->slot_floats, h->dyn, n);
         if (d.pool > 0) {
             const int done = (pos0 + n) / d.pool - pos0 / d.pool;          // blocks whose last position lies in this portion
             if (done > 0)
                 hipLaunchKernelGGL(hy_pool_kernel, dim3(done, 2, done <= 8 ? std::min(16, hy_cdiv(d.kv_heads * std::max(d.dim, d.vdim), 256)) : 1), dim3(256), 0, st, kc, vc, pk, pv,
                                    d.kv_heads * d.dim, d.kv_heads * d.vdim, d.pool, h->slot_floats, h->dyn, n);
         }
-        int32_t r = hy_attention(ctx, h->proj + L.q_off, np, kc, vc, d.heads, d.kv_heads, d.dim, d.vdim, d.scale, d.slope_log2, n, pos0, &nsplit, true, d.window, d.keep_first,
+        int32_t r = hy_attention(ctx, q, ldq, kc, vc, d.heads, d.kv_heads, d.dim, d.vdim, d.scale, d.slope_log2, n, pos0, &nsplit, true, d.window, d.keep_first,
                                  pk, pv, d.pool);
         if (r != GL3_OK) return r;
         hipLaunchKernelGGL((hy_attn_merge_kernel<T>), dim3(n, d.heads), dim3(64), 0, st, h->part_acc, h->part_ml, d.heads, d.vdim, nsplit, d.softmax_sink,
                            d.out_gate ? h->proj + L.g_off : nullptr, np, d.out_gate, mixo, ldo, d.v_rot ? L.vrot_freq : nullptr, h->dyn,
                            d.softmax_sink == 2 ? L.sink : nullptr, L.out_mul);
     } else if (d.mixer == GL3_MIX_MEMORY) {
-        const bool eg = d.mem_gates == GL3_MEM_EXP_GATES;
+        const bool eg = d.mem_gates == GL3_MEM_EXP_GATES, cg = d.mem_gates == GL3_MEM_CHANNEL_GATES;
         const int P = d.vdim + (eg ? 1 : 0), ldy = d.heads * P;
         float *ga = h->gates, *gb = ga + (size_t)h->mb * h->max_heads, *ge = gb + (size_t)h->mb * h->max_heads;
         if (eg)
@@ -895,29 +1010,32 @@ static int32_t hy_mixer_core(gl3_ctx* ctx, HyLayer& L, int np, int ldo, int n, i
         a.qsrc = h->proj; a.ldq = np; a.q_off = L.q_off; a.q_hstride = d.dim;
         a.xsrc = h->proj; a.ldx = np; a.x_off = L.v_off;
         a.k_mul = d.mem_k_mul != 0.f ? d.mem_k_mul : 1.f; a.q_mul = d.mem_q_mul != 0.f ? d.mem_q_mul : 1.f;
-        a.act = d.mem_qkv_act;
+        a.act = d.mem_qkv_act == 1 ? 7 : d.mem_qkv_act == 2 ? 2 : 0;
         a.rot = HyScanRot{d.rot_dims, L.rot_freq, d.rot_interleaved};
-        a.mode = eg ? 1 : 2; a.ga = ga; a.gb = gb; a.decay = L.decay; a.ones_col = eg ? 1 : 0;
+        a.mode = eg ? 1 : cg ? 3 : 2; if (cg) { a.fbias = L.pbias + L.f_off; a.lower = L.mem_lower; }
+        a.ga = ga; a.gb = gb; a.decay = L.decay; a.ones_col = eg ? 1 : 0;
         a.heads = d.heads; a.P = P; a.N = d.dim; a.G = d.heads;
         a.state = h->slots + L.off_state; a.slot_stride = h->slot_floats; a.dyn = h->dyn; a.n = n; a.y = h->ssm_y; a.ldy = ldy;
         hy_scan(ctx, a);
+        const float* gate = d.mem_gate_act == 2 ? nullptr : h->proj;
+        const int w_stride = d.mem_norm_weight == 2 ? 0 : d.vdim;
         if (d.mem_norm_whole && !eg) {          // one norm over the heads side by side: the kernel's "head" is the token's whole row
             // (a row is heads x vdim wide: 1024 threads for a few tokens, 256 for many)
             if (n <= 32 && ldy > 512)
                 hipLaunchKernelGGL((hy_mem_out_kernel<T, 1024>), dim3(n, 1), dim3(1024), 0, st, h->ssm_y, ldy, ldy, ldy, (const float*)nullptr, 1,
-                                   d.mem_norm_weight ? L.ssm_norm : nullptr, h->proj, np, L.g_off, d.mem_gate_act, eps, L.out_mul, mixo, ldo);
+                                   d.mem_norm_weight ? L.ssm_norm : nullptr, gate, np, L.g_off, d.mem_gate_act, eps, L.out_mul, mixo, ldo, w_stride);
             else if (ldy > 128)
                 hipLaunchKernelGGL((hy_mem_out_kernel<T, 256>), dim3(n, 1), dim3(256), 0, st, h->ssm_y, ldy, ldy, ldy, (const float*)nullptr, 1,
-                                   d.mem_norm_weight ? L.ssm_norm : nullptr, h->proj, np, L.g_off, d.mem_gate_act, eps, L.out_mul, mixo, ldo);
+                                   d.mem_norm_weight ? L.ssm_norm : nullptr, gate, np, L.g_off, d.mem_gate_act, eps, L.out_mul, mixo, ldo, w_stride);
             else
                 hipLaunchKernelGGL((hy_mem_out_kernel<T, 64>), dim3(n, 1), dim3(64), 0, st, h->ssm_y, ldy, ldy, ldy, (const float*)nullptr, 1,
-                                   d.mem_norm_weight ? L.ssm_norm : nullptr, h->proj, np, L.g_off, d.mem_gate_act, eps, L.out_mul, mixo, ldo);
+                                   d.mem_norm_weight ? L.ssm_norm : nullptr, gate, np, L.g_off, d.mem_gate_act, eps, L.out_mul, mixo, ldo, w_stride);
         } else if (n <= 32 && d.vdim > 128)
             hipLaunchKernelGGL((hy_mem_out_kernel<T, 256>), dim3(n, d.heads), dim3(256), 0, st, h->ssm_y, ldy, P, d.vdim, eg ? ge : nullptr, d.heads,
-                               d.mem_norm_weight ? L.ssm_norm : nullptr, h->proj, np, L.g_off, d.mem_gate_act, eps, L.out_mul, mixo, ldo);
+                               d.mem_norm_weight ? L.ssm_norm : nullptr, gate, np, L.g_off, d.mem_gate_act, eps, L.out_mul, mixo, ldo, w_stride);
         else
             hipLaunchKernelGGL((hy_mem_out_kernel<T, 64>), dim3(n, d.heads), dim3(64), 0, st, h->ssm_y, ldy, P, d.vdim, eg ? ge : nullptr, d.heads,
-                               d.mem_norm_weight ? L.ssm_norm : nullptr, h->proj, np, L.g_off, d.mem_gate_act, eps, L.out_mul, mixo, ldo);
+                               d.mem_norm_weight ? L.ssm_norm : nullptr, gate, np, L.g_off, d.mem_gate_act, eps, L.out_mul, mixo, ldo, w_stride);
     } else if (d.mixer == GL3_MIX_LATENT) {
         // De entries per query / key head, Re per cached row (= dim, kv_rank without a rotated part)
         float* cc = h->slots + L.off_k;
@@ -1015,6 +1133,23 @@ static int32_t hy_mixer(gl3_ctx* ctx, HyLayer& L, int n, int pos0, int seq) {
     return GL3_OK;
 }
 
+// Up (and gate) product of the layer's dense feed-forward (in a mixture of experts: of the shared expert) with its activation: act [n][ff_pad]
+// in the matrix type, the down projection's operand.
+template <typename T>
+static void hy_ff_up(gl3_ctx* ctx, const T* hb, HyLayer& L, int n, T* act) {
+    gl3_hybrid_state* h = ctx->hy;
+    const int act_id = L.d.ff_act;
+    if (act_id == 3) {          // the activation needs the token's whole vector: float32 products (K-split parts), then one pass
+        int parts = 1;
+        hy_gemm<T>(ctx, hb, h->W, L.gu, n, h->ffz, L.ff_pad, false, nullptr, 0, HyGlu{}, &parts);
+        if (L.ff_pad > 1024)
+            hipLaunchKernelGGL((hy_polynorm_kernel<T, 1024>), dim3(n), dim3(1024), 0, ctx->stream, h->ffz, L.ff_pad, L.dense_ff, parts, (size_t)n * L.ff_pad, L.poly, ctx->d.rms_eps, act);
+        else
+            hipLaunchKernelGGL((hy_polynorm_kernel<T, 256>), dim3(n), dim3(256), 0, ctx->stream, h->ffz, L.ff_pad, L.dense_ff, parts, (size_t)n * L.ff_pad, L.poly, ctx->d.rms_eps, act);
+    } else if (act_id == 2) hy_gemm<T>(ctx, hb, h->W, L.gu, n, nullptr, 0, false, act, L.ff_pad, HyGlu{0.f, 0.f, 0.f, nullptr, nullptr, 0, 0, 2});      // no gate: relu(up)^2
+    else hy_gemm<T>(ctx, hb, h->W, L.gu, n, nullptr, 0, true, act, L.ff_pad, hy_ff_glu(L));
+}
+
 // ---- mixture of experts -------------------------------------------------------------------------------------------------------------
 // One product of every (token, choice) pair with its expert's matrix: w = ONE expert's shape (rows, k, ld) at the base of the stacked
 // matrix, wstride elements apart.  few = a few tokens (decode): pairs in their own order, one matvec per pair (blockIdx.y) with the
@@ -1033,6 +1168,7 @@ static void hy_gemm_grouped(gl3_ctx* ctx, const T* A, int lda, const HyMat& w, s
 #define HY_GMV(KS)                                                                                                                                     \
     do {                                                                                                                                              \
         if (glu) hipLaunchKernelGGL((hy_matvec_kernel<T, T, 1, HY_EPI_GLU, KS, 1>), grid, dim3(256), 0, st, A, lda, Wt, w.ld, 1, N, K, C, ldc, act, ld_act, gp, h->sel, wstride, a_div, row_scale);   \
+        else if (gp.act == 2) hipLaunchKernelGGL((hy_matvec_kernel<T, T, 1, HY_EPI_ACTMUL, KS, 1>), grid, dim3(256), 0, st, A, lda, Wt, w.ld, 1, N, K, C, ldc, act, ld_act, gp, h->sel, wstride, a_div, row_scale);    \
         else hipLaunchKernelGGL((hy_matvec_kernel<T, T, 1, HY_EPI_STORE, KS, 1>), grid, dim3(256), 0, st, A, lda, Wt, w.ld, 1, N, K, C, ldc, act, ld_act, gp, h->sel, wstride, a_div, row_scale);    \
     } while (0)
         if (ksplit) HY_GMV(4); else HY_GMV(1);
@@ -1042,6 +1178,7 @@ static void hy_gemm_grouped(gl3_ctx* ctx, const T* A, int lda, const HyMat& w, s
     const HyGroup grp{h->tiles, h->ntiles, wstride};
     const dim3 grid(hy_cdiv(N, 128), max_tiles, 1);
     if (glu) hipLaunchKernelGGL((hy_gemm_kernel<T, T, HY_MOE_BM, 128, HY_EPI_GLU, 1>), grid, dim3(256), 0, st, A, lda, Wt, w.ld, 0, N, K, C, ldc, act, ld_act, gp, K, grp);
+    else if (gp.act == 2) hipLaunchKernelGGL((hy_gemm_kernel<T, T, HY_MOE_BM, 128, HY_EPI_ACTMUL, 1>), grid, dim3(256), 0, st, A, lda, Wt, w.ld, 0, N, K, C, ldc, act, ld_act, gp, K, grp);
     else hipLaunchKernelGGL((hy_gemm_kernel<T, T, HY_MOE_BM, 128, HY_EPI_STORE, 1>), grid, dim3(256), 0, st, A, lda, Wt, w.ld, 0, N, K, C, ldc, act, ld_act, gp, K, grp);
 }
 
@@ -1060,23 +1197,25 @@ static void hy_moe(gl3_ctx* ctx, HyLayer& L, int n) {
     const int max_tiles = P / HY_MOE_BM + std::min(E, P);
     const bool on_out = d.route_on_output != 0;          // the weights multiply the experts' outputs (in the residual update) instead of their inputs
     hipLaunchKernelGGL(hy_route_kernel, dim3(n), dim3(64), 0, st, h->moe_z, RZ, zparts, (size_t)n * RZ, E, top, h->sel, h->wsel, few ? h->pair_row : nullptr,
-                       (d.shared_ff > 0 && !d.shared_ungated) ? h->sgz : nullptr, HyRoute{d.route_softmax, L.route_bias, d.route_renorm, d.route_scale != 0.f ? d.route_scale : 1.f});
+                       (d.shared_ff > 0 && !d.shared_ungated) ? h->sgz : nullptr, HyRoute{d.route_softmax, L.route_bias, d.route_renorm, d.route_scale != 0.f ? d.route_scale : 1.f, d.route_groups, d.route_keep});
     HyMat one_gu = L.egu, one_down = L.edown;
-    one_gu.rows = 2 * L.eff_pad; one_down.rows = W;
+    const bool glu = !hy_ungated(d);
+    one_gu.rows = (glu ? 2 : 1) * L.eff_pad; one_down.rows = W;
+    const size_t gu_stride = (size_t)one_gu.rows * L.egu.ld;
     if (few) {
         // a few tokens: the pairs of a token read its normed row themselves and the score multiplies the products (W (s h) = s (W h))
-        hy_gemm_grouped<T>(ctx, hb, W, one_gu, (size_t)2 * L.eff_pad * L.egu.ld, P, max_tiles, true, nullptr, 0, true, (T*)h->eact, L.eff_pad,
+        hy_gemm_grouped<T>(ctx, hb, W, one_gu, gu_stride, P, max_tiles, true, nullptr, 0, glu, (T*)h->eact, L.eff_pad,
                            HyGlu{d.ff_limit, d.ff_alpha, d.ff_shift, nullptr, nullptr, 0, 0, d.ff_act}, top, on_out ? nullptr : h->wsel);
     } else {
         hipLaunchKernelGGL(hy_moe_group_kernel, dim3(1), dim3(256), (size_t)2 * E * 4, st, h->sel, P, E, HY_MOE_BM, h->pair_row, h->tiles, h->ntiles);
         hipLaunchKernelGGL((hy_moe_scale_kernel<T>), dim3(P), dim3(256), 0, st, hb, W, top, on_out ? (const float*)nullptr : h->wsel, h->pair_row, (T*)h->ea);
-        hy_gemm_grouped<T>(ctx, (const T*)h->ea, W, one_gu, (size_t)2 * L.eff_pad * L.egu.ld, P, max_tiles, false, nullptr, 0, true, (T*)h->eact, L.eff_pad,
+        hy_gemm_grouped<T>(ctx, (const T*)h->ea, W, one_gu, gu_stride, P, max_tiles, false, nullptr, 0, glu, (T*)h->eact, L.eff_pad,
                            HyGlu{d.ff_limit, d.ff_alpha, d.ff_shift, nullptr, nullptr, 0, 0, d.ff_act});
     }
     hy_gemm_grouped<T>(ctx, (const T*)h->eact, L.eff_pad, one_down, (size_t)W * L.edown.ld, P, max_tiles, few, h->eout, W, false, nullptr, 0, HyGlu{});
     if (d.shared_ff > 0) {
         T* act = (T*)h->mixo;
-        hy_gemm<T>(ctx, hb, W, L.gu, n, nullptr, 0, true, act, L.ff_pad, hy_ff_glu(L));
+        hy_ff_up<T>(ctx, hb, L, n, act);
         hy_gemm<T>(ctx, act, L.ff_pad, L.down, n, h->y, W, false, nullptr, 0, HyGlu{}, &h->y_parts);
     }
 }
@@ -1118,17 +1257,31 @@ static int32_t hy_portion_plain(gl3_ctx* ctx, int seq, const int32_t* tokens, in
     const float eps = ctx->d.rms_eps;
     memcpy(h->h_tokens, tokens, (size_t)n * 4);
     if (nw > 0) memcpy(h->h_want, want, (size_t)nw * 4);
-    h->h_dyn[0] = pos0; h->h_dyn[1] = seq;
+    h->h_dyn[0] = pos0; h->h_dyn[1] = seq; h->h_dyn[2] = h->last_tok[seq];
     HY_HIP(hipMemcpyAsync(h->dyn, h->h_dyn, (size_t)(4 + h->want_cap + n) * 4, hipMemcpyHostToDevice, st));
-    hipLaunchKernelGGL((hy_embed_kernel<T>), dim3(n, n <= 32 ? hy_cdiv(W, 256) : 1), dim3(256), 0, st, h->tokens, (const T*)h->emb.w, h->X, W, 1, lstride, h->emb_scale, h->depth ? h->hist : nullptr);
+    hipLaunchKernelGGL((hy_embed_kernel<T>), dim3(n, n <= 32 ? hy_cdiv(W, 256) : 1), dim3(256), 0, st, h->tokens, (const T*)h->emb.w, h->X, W, 1, lstride, h->emb_scale, h->depth ? h->hist : nullptr,
+                       HyBigram{h->bigram.w, h->bg_buckets, h->bg_prev, h->bg_cur}, h->dyn);
     T* hb = (T*)h->h;
     HyResid base{};
     base.x = h->X; base.W = W; base.eps = eps; base.ya_parts = 1; base.ya_mul = 1.f;
-    {
-        HyResid r = base;
-        r.norm_w = h->L[0].norm1;
+    // a residual update that ends in the norm in front of layer l's mixer (l = nl: the last layer has run, no norm), with the token shift
+    auto resid_to_mixer = [&](HyResid r, int l) {
+        if (l < nl) {
+            HyLayer& N = h->L[l];
+            r.norm_w = N.norm1;
+            if (h->shift && n == 1) { r.shift_mu = N.shift_mu; r.shift_prev = h->slots + N.off_shift; r.slot_stride = h->slot_floats; r.dyn = h->dyn; }
+            else if (h->shift) r.hf = h->hf;
+        }
         hy_resid<T>(ctx, n, r, (T*)nullptr, hb);
-    }
+        if (l < nl && r.hf) {
+            float* prev = h->slots + h->L[l].off_shift;
+            const int v = W % 4 == 0 ? 4 : 1;
+            const dim3 grid(n, hy_cdiv(W, 256 * v));
+            if (v == 4) hipLaunchKernelGGL((hy_shift_kernel<T, 4>), grid, dim3(256), 0, st, h->hf, W, n, h->L[l].shift_mu, prev, h->slot_floats, h->dyn, hb);
+            else hipLaunchKernelGGL((hy_shift_kernel<T, 1>), grid, dim3(256), 0, st, h->hf, W, n, h->L[l].shift_mu, prev, h->slot_floats, h->dyn, hb);
+        }
+    };
+    resid_to_mixer(base, 0);
     for (int l = 0; l < nl; ++l) {
         HyLayer& L = h->L[l];
         const bool last = l + 1 == nl;
@@ -1151,8 +1304,7 @@ static int32_t hy_portion_plain(gl3_ctx* ctx, int seq, const int32_t* tokens, in
             }
             if (h->depth) { r.hist = h->hist; r.hist_stride = lstride; r.n_mix = l + 2; r.mix = L.depth_mix; }
             if (h->taps) r.tap = h->taps + (size_t)l * lstride;
-            if (!last) r.norm_w = h->L[l + 1].norm1;
-            hy_resid<T>(ctx, n, r, (T*)nullptr, hb);
+            resid_to_mixer(r, l + 1);
         };
         int32_t rc = hy_mixer<T>(ctx, L, n, pos0, seq);
         if (rc != GL3_OK) return rc;
@@ -1164,7 +1316,7 @@ static int32_t hy_portion_plain(gl3_ctx* ctx, int seq, const int32_t* tokens, in
             if (L.d.ff > 0) {
                 T* act = (T*)h->mixo;
                 int p2 = 1;
-                hy_gemm<T>(ctx, hb, W, L.gu, n, nullptr, 0, true, act, L.ff_pad, hy_ff_glu(L));
+                hy_ff_up<T>(ctx, hb, L, n, act);
                 hy_gemm<T>(ctx, act, L.ff_pad, L.down, n, h->y + (size_t)h->y_parts * n * W, W, false, nullptr, 0, HyGlu{}, &p2);
                 r.ya_parts += p2;
             }
@@ -1175,11 +1327,13 @@ static int32_t hy_portion_plain(gl3_ctx* ctx, int seq, const int32_t* tokens, in
             continue;
         }
         r.post_w = L.norm1b;          // null without post norms
+        r.lw = L.ls1;                 // null without layer scales
         if (L.d.ff > 0) {
             r.norm_w = L.norm2;
             hy_resid<T>(ctx, n, r, (T*)nullptr, hb);
             r = base;
             r.post_w = L.norm2b;
+            r.lw = L.ls2;
             if (L.d.experts > 0) {
                 hy_moe<T>(ctx, L, n);
                 r.eo = h->eout; r.pair_row = h->pair_row; r.top = L.d.top;
@@ -1190,8 +1344,7 @@ static int32_t hy_portion_plain(gl3_ctx* ctx, int seq, const int32_t* tokens, in
                 }
             } else {
                 T* act = (T*)h->mixo;
-                if (L.d.ff_act == 2) hy_gemm<T>(ctx, hb, W, L.gu, n, nullptr, 0, false, act, L.ff_pad, HyGlu{0.f, 0.f, 0.f, nullptr, nullptr, 0, 0, 2});      // no gate: relu(up)^2
-                else hy_gemm<T>(ctx, hb, W, L.gu, n, nullptr, 0, true, act, L.ff_pad, hy_ff_glu(L));
+                hy_ff_up<T>(ctx, hb, L, n, act);
                 hy_gemm<T>(ctx, act, L.ff_pad, L.down, n, h->y, W, false, nullptr, 0, HyGlu{}, &h->y_parts);
                 r.ya = h->y; r.ya_parts = h->y_parts; r.ya_stride = (size_t)n * W;
             }
@@ -1233,7 +1386,7 @@ static int32_t hy_portion(gl3_ctx* ctx, int seq, const int32_t* tokens, int n, i
         }
         if (ff) {
             T* act = (T*)h->mixo;
-            hy_gemm<T>(ctx, hb, W, L.gu, n, nullptr, 0, true, act, L.ff_pad, hy_ff_glu(L));
+            hy_ff_up<T>(ctx, hb, L, n, act);
             hy_gemm<T>(ctx, act, L.ff_pad, L.down, n, h->y, W, false, nullptr, 0, HyGlu{}, &h->y_parts);
             const float* nin = last ? nullptr : h->L[l + 1].hc[0][0];
             const float* nw_ = last ? nullptr : h->L[l + 1].norm1;
@@ -1288,6 +1441,7 @@ int32_t gl3_hy_step(gl3_ctx* ctx, int32_t seq, const int32_t* tokens, int32_t n,
                 r = GL3_OK;
             }
             if (r != GL3_OK) return r;
+            h->last_tok[seq] = tokens[off + pn - 1];
             if (g > 0 && logits_out) HY_HIP(hipMemcpyAsync(h->h_logits, h->logits, (size_t)g * V * 4, hipMemcpyDeviceToHost, ctx->stream));
             HY_HIP(hipStreamSynchronize(ctx->stream));
             if (g > 0 && logits_out) memcpy(logits_out + (size_t)done * V, h->h_logits, (size_t)g * V * 4);

@@ -223,6 +223,19 @@ bool split_layer_name(const std::string& name, int32_t& layer, std::string& leaf
     return true;
 }
 
+// "mlp.e<k>.gate | up | down": one routed expert's part of a stacked tensor
+bool expert_leaf(const std::string& lf, int32_t& id, int32_t& expert) {
+    static const std::map<std::string, int> part = {{"gate", GL3_T_FFN_GATE_EXPS}, {"up", GL3_T_FFN_UP_EXPS}, {"down", GL3_T_FFN_DOWN_EXPS}};
+    if (lf.compare(0, 5, "mlp.e") != 0) return false;
+    size_t i = 5;
+    while (i < lf.size() && lf[i] >= '0' && lf[i] <= '9') ++i;
+    if (i == 5 || i > 12 || i >= lf.size() || lf[i] != '.') return false;
+    auto pf = part.find(lf.substr(i + 1));
+    if (pf == part.end()) return false;
+    id = pf->second; expert = atoi(lf.substr(5, i - 5).c_str());
+    return true;
+}
+
 bool noditar_tensor(const std::string& name, int32_t& id, int32_t& layer, int32_t& expert) {
     expert = -1;
     static const std::map<std::string, int> global = {{"embed", GL3_T_TOKEN_EMBD}, {"head", GL3_T_OUTPUT}, {"final.norm", GL3_T_OUTPUT_NORM}};
@@ -312,7 +325,6 @@ bool vonulix_tensor(const std::string& name, int32_t& id, int32_t& layer, int32_
         {"mix.o", GL3_T_WO}, {"mlp.router", GL3_T_FFN_GATE_INP}, {"mlp.shared.gate", GL3_T_W1}, {"mlp.shared.up", GL3_T_W3}, {"mlp.shared.down", GL3_T_W2},
         {"mlp.shared.sg", GL3_T_FFN_GATE_INP_SHEXP}, {"dwa", GL3_T_DEPTH_MIX}, {"side.gate", GL3_T_SIDE_GATE}, {"side.proj", GL3_T_SIDE_PROJ},
         {"side.norm", GL3_T_SIDE_NORM}};
-    static const std::map<std::string, int> part = {{"gate", GL3_T_FFN_GATE_EXPS}, {"up", GL3_T_FFN_UP_EXPS}, {"down", GL3_T_FFN_DOWN_EXPS}};
     expert = -1;
     auto g = global.find(name);
     if (g != global.end()) { id = g->second; layer = 0; return true; }
@@ -320,16 +332,7 @@ bool vonulix_tensor(const std::string& name, int32_t& id, int32_t& layer, int32_
     if (!split_layer_name(name, layer, lf)) return false;
     auto f = leaf.find(lf);
     if (f != leaf.end()) { id = f->second; return true; }
-    if (lf.compare(0, 5, "mlp.e") == 0) {          // mlp.e<k>.gate | up | down
-        size_t i = 5;
-        while (i < lf.size() && lf[i] >= '0' && lf[i] <= '9') ++i;
-        if (i == 5 || i > 12 || i >= lf.size() || lf[i] != '.') return false;
-        auto pf = part.find(lf.substr(i + 1));
-        if (pf == part.end()) return false;
-        id = pf->second; expert = atoi(lf.substr(5, i - 5).c_str());
-        return true;
-    }
-    return false;
+    return expert_leaf(lf, id, expert);
 }
 
 // Kosusun: every layer is a parallel block — one RMS norm, whose output feeds the mixer and the feed-forward alike, and
@@ -564,7 +567,6 @@ bool kugadra_tensor(const std::string& name, int32_t& id, int32_t& layer, int32_
         {"mix.dq", GL3_T_Q_DOWN}, {"mix.dq.norm", GL3_T_Q_DOWN_NORM}, {"mix.uq", GL3_T_WQ}, {"mix.dkv", GL3_T_KV_DOWN}, {"mix.dkv.norm", GL3_T_KV_DOWN_NORM},
         {"mix.uk", GL3_T_K_UP}, {"mix.uv", GL3_T_V_UP}, {"mlp.up", GL3_T_W3}, {"mlp.down", GL3_T_W2}, {"mlp.router", GL3_T_FFN_GATE_INP},
         {"mlp.correction", GL3_T_FFN_ROUTE_BIAS}, {"mlp.shared.gate", GL3_T_W1}, {"mlp.shared.up", GL3_T_W3}, {"mlp.shared.down", GL3_T_W2}};
-    static const std::map<std::string, int> part = {{"gate", GL3_T_FFN_GATE_EXPS}, {"up", GL3_T_FFN_UP_EXPS}, {"down", GL3_T_FFN_DOWN_EXPS}};
     expert = -1;
     auto g = global.find(name);
     if (g != global.end()) { id = g->second; layer = 0; return true; }
@@ -572,20 +574,113 @@ bool kugadra_tensor(const std::string& name, int32_t& id, int32_t& layer, int32_
     if (!split_layer_name(name, layer, lf)) return false;
     auto f = leaf.find(lf);
     if (f != leaf.end()) { id = f->second; return true; }
-    if (lf.compare(0, 5, "mlp.e") == 0) {          // mlp.e<k>.gate | up | down
-        size_t i = 5;
-        while (i < lf.size() && lf[i] >= '0' && lf[i] <= '9') ++i;
-        if (i == 5 || i > 12 || i >= lf.size() || lf[i] != '.') return false;
-        auto pf = part.find(lf.substr(i + 1));
-        if (pf == part.end()) return false;
-        id = pf->second; expert = atoi(lf.substr(5, i - 5).c_str());
-        return true;
+    return expert_leaf(lf, id, expert);
+}
+
+// Tutedra: one plain residual stream, x <- x + ls1 * mixer(shift(norm1 x)), x <- x + ls2 * ff(norm2 x), norms with weights kept as their
+// deviation from one; the mixer's input is mixed with the previous token's; the embedding row gains a row chosen by the token pair; the
+// head is the embedding table.  Three layer types.  "hgrn2": a matrix memory whose forget gate (one per head and channel, bounded from
+// below) is also what it writes with, silu queries, heads normed with one shared weight, no gate.  "mlstm": a matrix memory with
+// exponential gates (as Kosusun's).  "attention": grouped-query attention with short convolutions on q and k, values = convolved keys,
+// q / k norms per head with a weight, a partial rotary turn with frequencies rescaled by wavelength.  Feed-forward: W_down PolyNorm(W_up h),
+// or a mixture of relu^2 experts (sigmoid scores, chosen by score + correction among the best groups of neighbours, the plain scores
+// weight the experts' outputs) plus a gated shared expert.  config.json gives every size and the constants; the forms are fixed here.
+bool tutedra_describe(const JVal& cfg, gl3_model_desc& d, std::vector<gl3_layer_desc>& layers, DescStore&, std::string& err) {
+    d.arch = GL3_ARCH_LAYERLIST;
+    d.weight_type = GL3_TYPE_BF16;
+    if (!get_int(cfg, "vocab", d.vocab, err) || !get_int(cfg, "width", d.dim, err)) return false;
+    d.streams = 0;
+    d.norm_offset = 1.f;
+    d.embedding_scale = 1.f;
+    d.token_shift = d.layer_scale = 1;
+    if (const JVal* e = cfg.get("embedding"))
+        if (const JVal* b = e->get("bigram"))
+            if (!b->is_null()) {
+                if (!get_int(*b, "buckets", d.bigram_buckets, err) || !get_int(*b, "mul_prev", d.bigram_mul_prev, err) || !get_int(*b, "mul_cur", d.bigram_mul_cur, err)) return false;
+                if (d.bigram_buckets < 1) { err = "config: bigram.buckets must be positive"; return false; }
+            }
+    const JVal* norm = cfg.get("norm");
+    if (!norm || !get_float(*norm, "eps", d.rms_eps, err)) { if (err.empty()) err = "config: missing norm.eps"; return false; }
+    const JVal* ls = cfg.get("layers");
+    if (!ls || ls->kind != JVal::ARR || ls->arr.empty()) { err = "config: 'layers' must be a non-empty list"; return false; }
+    for (const JVal& l : ls->arr) {
+        gl3_layer_desc ld{};
+        const JVal *ty = l.get("type"), *mx = l.get("mixer"), *mlp = l.get("mlp");
+        if (!ty || ty->kind != JVal::STR || !mx || mx->kind != JVal::OBJ) { err = "config: a layer needs 'type' and 'mixer'"; return false; }
+        if (!get_int(*mx, "heads", ld.heads, err) || !get_int(*mx, "dim", ld.dim, err) || !get_int(*mx, "vdim", ld.vdim, err)) return false;
+        ld.kv_heads = ld.heads;
+        if (ty->str == "hgrn2") {
+            ld.mixer = GL3_MIX_MEMORY;
+            ld.mem_gates = GL3_MEM_CHANNEL_GATES;
+            ld.mem_qkv_act = 2; ld.mem_norm_weight = 2; ld.mem_gate_act = 2;
+        } else if (ty->str == "mlstm") {
+            ld.mixer = GL3_MIX_MEMORY;
+            ld.mem_gates = GL3_MEM_EXP_GATES;
+            if (!get_float(*mx, "gate_cap", ld.mem_gate_cap, err)) return false;
+            ld.mem_q_mul = (float)(1.0 / std::sqrt((double)std::max(1, ld.dim)));
+            ld.mem_gate_act = 1; ld.mem_norm_weight = 1;
+        } else if (ty->str == "attention") {
+            ld.mixer = GL3_MIX_ATTENTION;
+            if (!get_int(*mx, "kv_heads", ld.kv_heads, err) || !get_float(*mx, "scale", ld.scale, err)) return false;
+            if (ld.vdim != ld.dim) { err = "config: the attention's values are its keys, vdim must equal dim"; return false; }
+            ld.v_from_k = 1; ld.qk_unit_norm = 3;
+            if (const JVal* cv = mx->get("conv"))
+                if (!cv->is_null() && !get_int(*mx, "conv", ld.qk_conv, err)) return false;
+            const JVal* rot = mx->get("rot");
+            if (rot && !rot->is_null()) {
+                if (!get_int(*rot, "dims", ld.rot_dims, err) || !get_float(*rot, "base", ld.rot_base, err)) return false;
+                if (const JVal* sc = rot->get("scaling"))
+                    if (!sc->is_null() && (!get_float(*sc, "factor", ld.rot_wave_factor, err) || !get_float(*sc, "low", ld.rot_wave_low, err) ||
+                                           !get_float(*sc, "high", ld.rot_wave_high, err) || !get_float(*sc, "original", ld.rot_wave_original, err)))
+                        return false;
+            }
+        } else { err = "config: unknown layer type '" + ty->str + "'"; return false; }
+        if (mlp && !mlp->is_null()) {
+            const JVal* kind = mlp->get("kind");
+            if (!kind || kind->kind != JVal::STR) { err = "config: mlp needs 'kind'"; return false; }
+            if (kind->str == "dense") {
+                if (!get_int(*mlp, "ff", ld.ff, err)) return false;
+                ld.ff_act = 3;
+            } else if (kind->str == "moe") {
+                const JVal *ex = mlp->get("expert"), *ro = mlp->get("router"), *sh = mlp->get("shared");
+                if (!ex || !ro || !get_int(*ex, "ff", ld.ff, err) || !get_int(*ro, "experts", ld.experts, err) || !get_int(*ro, "top", ld.top, err)) {
+                    if (err.empty()) err = "config: a mixture of experts needs 'expert' and 'router'";
+                    return false;
+                }
+                if (const JVal* gr = ro->get("groups"))
+                    if (!gr->is_null() && (!get_int(*gr, "count", ld.route_groups, err) || !get_int(*gr, "keep", ld.route_keep, err))) return false;
+                if (sh && !sh->is_null() && !get_int(*sh, "ff", ld.shared_ff, err)) return false;
+                ld.ff_act = 2; ld.route_bias = 1; ld.route_on_output = 1;
+            } else { err = "config: mlp.kind must be 'dense' or 'moe'"; return false; }
+        }
+        layers.push_back(ld);
     }
-    return false;
+    d.n_layers = (int32_t)layers.size();
+    return true;
+}
+
+bool tutedra_tensor(const std::string& name, int32_t& id, int32_t& layer, int32_t& expert) {
+    static const std::map<std::string, int> global = {{"embed", GL3_T_TOKEN_EMBD}, {"bigram", GL3_T_BIGRAM_EMBD}, {"final.norm", GL3_T_OUTPUT_NORM}};
+    // "mix.f" / "mix.f.b" are the forget gates of both recurrences, "mix.norm" both recurrences' head norm
+    static const std::map<std::string, int> leaf = {
+        {"norm1", GL3_T_ATTN_NORM}, {"norm2", GL3_T_FFN_NORM}, {"ls1", GL3_T_ATTN_SCALE}, {"ls2", GL3_T_FFN_SCALE}, {"shift", GL3_T_TOKEN_SHIFT},
+        {"mix.q", GL3_T_WQ}, {"mix.k", GL3_T_WK}, {"mix.v", GL3_T_WV}, {"mix.g", GL3_T_ATTN_GATE}, {"mix.o", GL3_T_WO}, {"mix.norm", GL3_T_SSM_NORM},
+        {"mix.i", GL3_T_MEM_IGATE}, {"mix.i.b", GL3_T_MEM_IGATE_BIAS}, {"mix.f", GL3_T_MEM_FGATE}, {"mix.f.b", GL3_T_MEM_FGATE_BIAS}, {"mix.lower", GL3_T_MEM_LOWER},
+        {"mix.q.norm", GL3_T_ATTN_Q_NORM}, {"mix.k.norm", GL3_T_ATTN_K_NORM}, {"mix.q.conv", GL3_T_Q_CONV}, {"mix.k.conv", GL3_T_K_CONV},
+        {"mlp.up", GL3_T_W3}, {"mlp.down", GL3_T_W2}, {"mlp.act", GL3_T_FFN_POLY}, {"mlp.router", GL3_T_FFN_GATE_INP}, {"mlp.correction", GL3_T_FFN_ROUTE_BIAS},
+        {"mlp.shared.up", GL3_T_W3}, {"mlp.shared.down", GL3_T_W2}, {"mlp.shared.sg", GL3_T_FFN_GATE_INP_SHEXP}};
+    expert = -1;
+    auto g = global.find(name);
+    if (g != global.end()) { id = g->second; layer = 0; return true; }
+    std::string lf;
+    if (!split_layer_name(name, layer, lf)) return false;
+    auto f = leaf.find(lf);
+    if (f != leaf.end()) { id = f->second; return true; }
+    return expert_leaf(lf, id, expert);
 }
 
 const Design DESIGNS[] = {{"Noditar", noditar_describe, noditar_tensor}, {"Vonulix", vonulix_describe, vonulix_tensor}, {"Kosusun", kosusun_describe, kosusun_tensor},
-                          {"Kugadra", kugadra_describe, kugadra_tensor}};
+                          {"Kugadra", kugadra_describe, kugadra_tensor}, {"Tutedra", tutedra_describe, tutedra_tensor}};
 
 struct Mapping {
     void* p = MAP_FAILED; size_t n = 0;

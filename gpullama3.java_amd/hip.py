@@ -65,7 +65,9 @@ class LayerDesc(C.Structure):
                 ("q_rank", C.c_int32), ("rot_dim", C.c_int32), ("kv_share", C.c_int32), ("rot_yarn_factor", C.c_float),
                 ("rot_yarn_original", C.c_float), ("rot_yarn_fast", C.c_float), ("rot_yarn_slow", C.c_float),
                 ("mem_qkv_act", C.c_int32), ("mem_norm_whole", C.c_int32), ("route_softmax", C.c_int32), ("route_bias", C.c_int32),
-                ("route_renorm", C.c_int32), ("route_on_output", C.c_int32), ("shared_ungated", C.c_int32), ("route_scale", C.c_float)]
+                ("route_renorm", C.c_int32), ("route_on_output", C.c_int32), ("shared_ungated", C.c_int32), ("route_scale", C.c_float),
+                ("qk_conv", C.c_int32), ("v_from_k", C.c_int32), ("rot_wave_factor", C.c_float), ("rot_wave_low", C.c_float),
+                ("rot_wave_high", C.c_float), ("rot_wave_original", C.c_float), ("route_groups", C.c_int32), ("route_keep", C.c_int32)]
 
 
 class ModelDesc(C.Structure):
@@ -78,7 +80,8 @@ class ModelDesc(C.Structure):
                 ("n_experts", C.c_int32), ("n_experts_used", C.c_int32), ("moe_hidden", C.c_int32),
                 ("streams", C.c_int32), ("layer_descs", C.POINTER(LayerDesc)),
                 ("norm_offset", C.c_float), ("side_dim", C.c_int32), ("depth_mix", C.c_int32), ("parallel_block", C.c_int32),
-                ("post_norms", C.c_int32), ("logit_softcap", C.c_float)]
+                ("post_norms", C.c_int32), ("logit_softcap", C.c_float), ("bigram_buckets", C.c_int32), ("bigram_mul_prev", C.c_int32),
+                ("bigram_mul_cur", C.c_int32), ("token_shift", C.c_int32), ("layer_scale", C.c_int32)]
 
 
 class KernelTimes(C.Structure):

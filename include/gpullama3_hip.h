@@ -71,7 +71,7 @@ enum { GL3_ARCH_LLAMA = 0, GL3_ARCH_QWEN3 = 1, GL3_ARCH_QWEN2 = 2,
                               * gl3_layer_desc; several residual streams mixed by per-sublayer tables, or one plain residual with an optional
                               * weighted average over all earlier layers' results; bfloat16 or float32 matrices
                               * (GL3_TYPE_BF16, GL3_FLAG_F32_COMPUTE); model folders with config.json + model.safetensors (gl3_load_model_dir) */
-       GL3_ARCH_LAYERLIST = 6 /* the same family under its own name: the registered designs (Noditar, Vonulix, Kosusun, Kugadra) differ only in
+       GL3_ARCH_LAYERLIST = 6 /* the same family under its own name: the registered designs (Noditar, Vonulix, Kosusun, Kugadra, Tutedra) differ only in
                               * the parameters of gl3_model_desc / gl3_layer_desc that their `describe` fills in */ };
 
 /* token mixers of a layer-list model (gl3_layer_desc.mixer) */
@@ -81,13 +81,17 @@ enum { GL3_MIX_ATTENTION = 0,   /* grouped-query softmax attention over cached k
        GL3_MIX_LATENT = 1,      /* attention whose keys and values are expanded from one cached low-rank latent per token */
        GL3_MIX_SSM = 2,         /* selective state-space recurrence (scalar decay per head) behind a short causal convolution */
        GL3_MIX_MEMORY = 3 };    /* matrix memory per head, S_t = a_t S_(t-1) + b_t k_t v_t^T, o_t = S_t^T q_t, float32 state carried per sequence:
-                                 * a fixed decay per head (retention) or exponential gates with a running maximum and a normaliser (mLSTM) */
+                                 * a fixed decay per head (retention), exponential gates with a running maximum and a normaliser (mLSTM), or a
+                                 * forget gate per head and channel whose complement is the key (HGRN2) */
 
 /* gl3_layer_desc.mem_gates: how a matrix memory gets a_t and b_t */
 enum { GL3_MEM_DECAY = 0,       /* a = mem_decay[head], b = 1; no normaliser: o = S^T q */
-       GL3_MEM_EXP_GATES = 1 }; /* log gates from two projections with biases: i = cap tanh(z_i / cap), f = logsigmoid(cap tanh(z_f / cap));
+       GL3_MEM_EXP_GATES = 1,  /* log gates from two projections with biases: i = cap tanh(z_i / cap), f = logsigmoid(cap tanh(z_f / cap));
                                  * m_t = max(f + m_(t-1), i), m_0 = 0; a = e^(f + m_(t-1) - m_t), b = e^(i - m_t); n_t = a n + b k;
                                  * o = S^T q / (max(|n . q|, e^(-m_t)) + 1e-6) */
+       GL3_MEM_CHANNEL_GATES = 2 }; /* one forget gate per head and key channel, f = l + (1 - l) sigmoid(z_f + bias); S_t = diag(f) S_(t-1) + (1 - f) v^T,
+                                 * o = S^T q: no key projection; z_f from GL3_T_MEM_FGATE [heads dim x width], GL3_T_MEM_FGATE_BIAS [heads dim], l from
+                                 * GL3_T_MEM_LOWER [heads dim] */
 
 /* gl3_upload_tensor: `layer` + GL3_LAYER_BESIDE addresses the second mixer of a layer (gl3_layer_desc.beside) */
 #define GL3_LAYER_BESIDE (1 << 30)
@@ -138,7 +142,8 @@ typedef struct gl3_layer_desc {
     int32_t qk_bias, rot_interleaved, pool;
     /* matrix memory (GL3_MIX_MEMORY): heads, dim (keys / queries), vdim; rot_* turn q and k as in attention; q and k are multiplied by
      * mem_q_mul / mem_k_mul (0 = 1) after the rotation.  The head's output is divided by its root mean square, multiplied by the weight
-     * GL3_T_SSM_NORM [heads vdim] if mem_norm_weight, and by act(W_g h) (GL3_T_ATTN_GATE, act = silu for mem_gate_act 0, sigmoid for 1).
+     * GL3_T_SSM_NORM [heads vdim] if mem_norm_weight = 1 ([vdim], shared by the heads, if 2), and by act(W_g h) (GL3_T_ATTN_GATE, act = silu for
+     * mem_gate_act 0, sigmoid for 1; 2: no output gate, no W_g).
      * mem_decay: heads values (copied by gl3_create).  GL3_MEM_EXP_GATES: gate projections GL3_T_MEM_IGATE / FGATE [heads x width] and
      * their biases GL3_T_MEM_IGATE_BIAS / FGATE_BIAS [heads], cap = mem_gate_cap */
     int32_t mem_gates;
@@ -163,7 +168,7 @@ typedef struct gl3_layer_desc {
      * rows (and turned key parts) that layer j < this layer writes (same kv_rank and rot_dim), with its own expansions. */
     int32_t q_rank, rot_dim, kv_share;
     float   rot_yarn_factor, rot_yarn_original, rot_yarn_fast, rot_yarn_slow;
-    /* matrix memory, further switches.  mem_qkv_act = 1: q, k and v are silu(projection).  mem_norm_whole = 1: ONE root mean square over
+    /* matrix memory, further switches.  mem_qkv_act = 1: q, k and v are silu(projection), 2: q alone.  mem_norm_whole = 1: ONE root mean square over
      * the token's heads side by side (heads vdim entries) instead of one per head. */
     int32_t mem_qkv_act, mem_norm_whole;
     /* feed-forward, further switches.  ff_act = 2: no gate, act = relu(W_up h)^2 (GL3_T_W3, GL3_T_W2 only).  Mixture of experts:
@@ -173,6 +178,22 @@ typedef struct gl3_layer_desc {
      * shared_ungated = 1: the shared expert has no gate (no GL3_T_FFN_GATE_INP_SHEXP) */
     int32_t route_softmax, route_bias, route_renorm, route_on_output, shared_ungated;
     float   route_scale;
+    /* attention, further switches (each usable alone).  qk_conv > 0: a causal depthwise convolution of that many taps (no bias, no activation) over
+     * time on every channel of the q and k projections, directly behind them (GL3_T_Q_CONV [heads dim x qk_conv], GL3_T_K_CONV [kv_heads dim x
+     * qk_conv], last column = current token); the last qk_conv - 1 projected rows belong to the sequence slot.  qk_unit_norm = 3: root mean
+     * square per head times a weight shared by the heads (GL3_T_ATTN_Q_NORM [dim], GL3_T_ATTN_K_NORM [dim]).  v_from_k = 1: no value
+     * projection, the values are the keys as they leave the projection (and its convolution), before norm and rotation (vdim = dim).
+     * rot_wave_factor > 0 (also read by a matrix memory): rotary frequencies are rescaled by wavelength l = 2 pi / f: f stays where
+     * l < rot_wave_original / rot_wave_high, becomes f / factor where l > original / low, and in between (1 - s) f / factor + s f with
+     * s = (original / l - low) / (high - low) */
+    int32_t qk_conv, v_from_k;
+    float   rot_wave_factor, rot_wave_low, rot_wave_high, rot_wave_original;
+    /* feed-forward, further switches.  ff_act = 3 (dense only): no gate, act(z) = a N(z) + b N(z^2) + c N(z^3) + e over the token's whole vector
+     * z = W_up h, powers element by element, N(x) = x / sqrt(mean(x^2) + eps), a, b, c, e = GL3_T_FFN_POLY [4].  ff_act = 2 in a mixture of experts
+     * (needs route_on_output): experts and shared expert without gates (GL3_T_FFN_UP_EXPS / DOWN_EXPS, W3 / W2).
+     * route_groups > 0: the experts form that many equal runs of neighbours; a run's score is the sum of its two largest choice scores
+     * (score + bias) and only experts of the best route_keep runs can be chosen */
+    int32_t route_groups, route_keep;
 } gl3_layer_desc;
 
 /* ggml tensor types of the wire format (J/tensor/GGMLType.java:5-21) */
@@ -241,7 +262,15 @@ enum {
     GL3_T_Q_DOWN = 54,             /* latent: down projection of the queries         [q_rank x width]                    */
     GL3_T_Q_DOWN_NORM = 55,        /* latent: norm weight of the query latent        [q_rank]                            */
     GL3_T_FFN_ROUTE_BIAS = 56,     /* mixture of experts: added to the scores for the choice only    [experts]           */
-    GL3_T_COUNT = 57
+    GL3_T_BIGRAM_EMBD = 57,        /* gl3_model_desc.bigram_buckets: rows of token pairs, last row = first token of a sequence [buckets + 1 x width] */
+    GL3_T_TOKEN_SHIFT = 58,        /* gl3_model_desc.token_shift: share of the previous token's normed row in the mixer's input  [width] */
+    GL3_T_ATTN_SCALE = 59,         /* gl3_model_desc.layer_scale: multiplies the mixer's output         [width]          */
+    GL3_T_FFN_SCALE = 60,          /*                             multiplies the feed-forward's output  [width]          */
+    GL3_T_FFN_POLY = 61,           /* ff_act = 3: a, b, c, e                         [4]                                 */
+    GL3_T_Q_CONV = 62,             /* attention with qk_conv: taps of the q channels [heads * dim x qk_conv]             */
+    GL3_T_K_CONV = 63,             /*                         taps of the k channels [kv_heads * dim x qk_conv]          */
+    GL3_T_MEM_LOWER = 64,          /* matrix memory, channel gates: lower bound      [heads * dim]                       */
+    GL3_T_COUNT = 65
 };
 
 /* gl3_model_desc.flags */
@@ -318,6 +347,14 @@ typedef struct {
      * logit_softcap > 0: logits <- cap tanh(logits / cap). */
     int32_t post_norms;
     float   logit_softcap;
+    /* layer-list family with streams == 0, each usable alone.  bigram_buckets > 0: the embedding gains row
+     * (previous token * bigram_mul_prev + token * bigram_mul_cur) mod bigram_buckets of GL3_T_BIGRAM_EMBD, its last row (number
+     * bigram_buckets) for a sequence's first token; the previous token belongs to the sequence slot.  token_shift != 0: a mixer reads
+     * h + (h' - h) * mu with h the normed row, h' the previous token's normed row (zeros for the first token; kept in the slot) and mu
+     * = GL3_T_TOKEN_SHIFT of the layer.  layer_scale != 0: a sublayer's output is multiplied element by element by GL3_T_ATTN_SCALE /
+     * GL3_T_FFN_SCALE before it joins the residual. */
+    int32_t bigram_buckets, bigram_mul_prev, bigram_mul_cur;
+    int32_t token_shift, layer_scale;
 } gl3_model_desc;
 
 /* Per-kernel-class device time of one instrumented decode step (HIP events around every launch). */
