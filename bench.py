@@ -115,12 +115,16 @@ def main():
                     "beside retention; mLSTM layers): prefill and decode throughput at layer sizes of a real model beside the family's closest design at "
                     "equal size (Noditar attention and state-space layers, same heads, state sizes and feed-forward); comma list of sizes from 1b,8b; "
                     "prints its own JSON line instead of the tg/pp line")
+    ap.add_argument("--tutedra", default="", help="layer-list family, Tutedra design (bfloat16: HGRN2, mLSTM and attention layers with a token shift in front "
+                    "and a scale behind every sublayer, polynomial feed-forward, relu^2 experts): comma-separated sizes (1b, 8b); prints its own JSON line")
     ap.add_argument("--kugadra", default="", help="layer-list family, Kugadra design (bfloat16: norms on both sides of every sublayer; lightning layers; "
                     "latent attention with a query latent, a shared rotated key part and a cache that the next layer reads; relu^2 feed-forward and a "
                     "mixture of experts with a softmax router): prefill and decode throughput at layer sizes of a real model beside the family's closest "
                     "design at equal size (Noditar latent-attention and state-space layers, same heads, row and state sizes, dense feed-forward of the "
                     "same active width); comma list of sizes from 1b,8b; prints its own JSON line instead of the tg/pp line")
     args = ap.parse_args()
+    if args.tutedra:
+        return bench_tutedra(args)
     if args.kugadra:
         return bench_kugadra(args)
     if args.hybrid:
@@ -803,6 +807,50 @@ def bench_kugadra(args):
     return bench_design_pair(args, "kugadra", "Kugadra", args.kugadra, KUGADRA_SIZES, kugadra_config, kugadra_twin_config,
                              "twin = Noditar latent-attention and state-space layers on one stream with the same heads, row and state sizes and a dense "
                              "feed-forward of the same active width, equal width / layers / vocabulary")
+
+
+TUTEDRA_SIZES = {   # width, dense feed-forward, layers (attention, hgrn2, mlstm, hgrn2, ...; even layers dense, odd ones experts), vocabulary; attention heads / kv
+                    # heads / head size; hgrn2 and mLSTM heads x key size x value size; experts x width, choices, groups (kept), shared expert
+    "1b": dict(width=2048, ff=8192, n_layers=8, vocab=32000, heads=32, kv_heads=8, dim=64, conv=4, h_heads=16, h_dim=128, h_vdim=128, m_heads=8, m_dim=128, m_vdim=256,
+               experts=32, top=4, groups=8, keep=4, expert_ff=1024, shared_ff=4096),
+    "8b": dict(width=4096, ff=14336, n_layers=4, vocab=32000, heads=32, kv_heads=8, dim=128, conv=4, h_heads=32, h_dim=128, h_vdim=128, m_heads=8, m_dim=256, m_vdim=512,
+               experts=32, top=4, groups=8, keep=4, expert_ff=1792, shared_ff=7168),
+}
+
+
+def tutedra_config(z):
+    D = z["dim"]
+    moe = {"kind": "moe", "expert": {"ff": z["expert_ff"]}, "router": {"experts": z["experts"], "top": z["top"], "groups": {"count": z["groups"], "keep": z["keep"]}},
+           "shared": {"ff": z["shared_ff"]}}
+    att = {"type": "attention", "mixer": {"heads": z["heads"], "kv_heads": z["kv_heads"], "dim": D, "vdim": D, "conv": z["conv"], "scale": D ** -0.5,
+                                          "rot": {"base": 500000.0, "dims": D // 2, "scaling": {"factor": 8.0, "high": 4.0, "low": 1.0, "original": 8192}}}}
+    hgrn = {"type": "hgrn2", "mixer": {"heads": z["h_heads"], "dim": z["h_dim"], "vdim": z["h_vdim"]}}
+    mls = {"type": "mlstm", "mixer": {"heads": z["m_heads"], "dim": z["m_dim"], "vdim": z["m_vdim"], "gate_cap": 15.0}}
+    kinds = [att, hgrn, mls, hgrn]
+    return {"architecture": "Tutedra", "vocab": z["vocab"], "width": z["width"], "norm": {"eps": 1e-6},
+            "embedding": {"bigram": {"buckets": 32003, "mul_prev": 8191, "mul_cur": 131}},
+            "layers": [dict(kinds[i % 4], mlp=moe if i % 2 else {"kind": "dense", "ff": z["ff"]}) for i in range(z["n_layers"])]}
+
+
+def tutedra_twin_config(z):
+    """The family's closest design at equal size: Noditar layers on one stream — attention with the same heads; where Tutedra has a recurrence,
+    the state-space mixer with the same heads, state rows (= key size) and head width (= value size); a dense gated feed-forward as wide as
+    what a token uses (the dense layers' own width; elsewhere the chosen experts plus the shared one)."""
+    D = z["dim"]
+    att = {"type": "attention", "mixer": {"heads": z["heads"], "kv_heads": z["kv_heads"], "dim": D, "vdim": D, "scale": D ** -0.5}}
+    ssm = lambda k: {"type": "mamba2", "mixer": {"heads": z[k + "_heads"], "vdim": z[k + "_vdim"], "state": z[k + "_dim"], "groups": z[k + "_heads"],
+                                                 "norm_groups": z[k + "_heads"], "conv": 4}}
+    kinds = [att, ssm("h"), ssm("m"), ssm("h")]
+    return {"architecture": "Noditar", "vocab": z["vocab"], "width": z["width"], "streams": 1, "norm": {"eps": 1e-5},
+            "layers": [dict(kinds[i % 4], mlp={"kind": "dense", "ff": z["top"] * z["expert_ff"] + z["shared_ff"] if i % 2 else z["ff"], "limit": 7.0})
+                       for i in range(z["n_layers"])]}
+
+
+def bench_tutedra(args):
+    """As bench_vonulix, for the Tutedra design beside its twin."""
+    return bench_design_pair(args, "tutedra", "Tutedra", args.tutedra, TUTEDRA_SIZES, tutedra_config, tutedra_twin_config,
+                             "twin = Noditar attention and state-space layers on one stream with the same heads and state sizes and a dense feed-forward of the "
+                             "same active width, equal width / layers / vocabulary")
 
 
 def bench_design_pair(args, label_key, design, sizes_arg, SIZES, config_fn, twin_fn, twin_text):

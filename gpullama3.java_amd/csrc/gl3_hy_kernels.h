@@ -499,19 +499,39 @@ static __global__ __launch_bounds__(64) void hy_attn_prep_kernel(float* __restri
             const int C = (H + G) * D, c0 = hh * D, keep = x.taps - 1;
             float* tl = x.tail + slot + c0;
             const bool fresh = dyn[0] == 0;
-            for (int d = lane; d < D; d += 64) {
-                float a = 0.f;
-                for (int j = 0; j < x.taps; ++j) {
-                    const int tau = t - keep + j;
-                    const float u = tau >= 0 ? proj[(size_t)tau * ld + col + d] : fresh ? 0.f : tl[(size_t)(keep + tau) * C + d];
-                    a = fmaf(x.conv_w[(size_t)j * C + c0 + d], u, a);
+            // two channels and four taps at a time, their loads issued together (taps that are not there read the token's own row, times 0)
+            for (int d0 = lane; d0 < D; d0 += 128) {
+                float a[2] = {0.f, 0.f};
+                for (int j0 = 0; j0 < x.taps; j0 += 4) {
+                    float u[4][2], w[4][2];
+#pragma unroll
+                    for (int k = 0; k < 4; ++k) {
+                        const int j = j0 + k, tau = t - keep + j;
+                        const bool live = j < x.taps && (tau >= 0 || !fresh);
+                        const float* up = !live ? src : tau >= 0 ? proj + (size_t)tau * ld + col : tl + (size_t)(keep + tau) * C;
+                        const float* wp = x.conv_w + (size_t)(j < x.taps ? j : 0) * C + c0;
+#pragma unroll
+                        for (int q = 0; q < 2; ++q) {
+                            const int d = min(d0 + 64 * q, D - 1);
+                            u[k][q] = up[d];
+                            w[k][q] = wp[d];
+                            if (!live) w[k][q] = 0.f;
+                        }
+                    }
+#pragma unroll
+                    for (int k = 0; k < 4; ++k)
+#pragma unroll
+                        for (int q = 0; q < 2; ++q) a[q] = fmaf(w[k][q], u[k][q], a[q]);
                 }
-                crow[d] = a;
-                if (x.n == 1) {
+#pragma unroll
+                for (int q = 0; q < 2; ++q)
+                    if (d0 + 64 * q < D) crow[d0 + 64 * q] = a[q];
+            }
+            if (x.n == 1)
+                for (int d = lane; d < D; d += 64) {
                     for (int i = 0; i + 1 < keep; ++i) tl[(size_t)i * C + d] = fresh ? 0.f : tl[(size_t)(i + 1) * C + d];
                     if (keep > 0) tl[(size_t)(keep - 1) * C + d] = src[d];
                 }
-            }
             __syncthreads();
             src = crow;
             if (isq) dst = x.qout + (size_t)t * x.ldq + hh * D;
@@ -1046,7 +1066,7 @@ struct HyScanArgs {
     const float* dtsrc; int ld_dt, dt_off; const float* dt_bias; const float* A_log; const float* Dp;      // mode 0 (Dp: null = no skip term)
     const float* ga; const float* gb;                  // mode 1: [n][heads]
     const float* decay;                                // mode 2: [heads]
-    const float* fbias; const float* lower;            // mode 3: [heads N] each
+    const float* fbias; const float* lower;            // mode 3: [heads N] each; fbias null: the source holds the gates already
     int ones_col;
     int heads, P, N, G, NG, TB;
     float* state; size_t slot_stride; const int* dyn; int n;
@@ -1067,6 +1087,17 @@ __device__ __forceinline__ void hy_scan_stage(float* __restrict__ dst, const flo
             const int i = i0 + u * 256;
             if (i < total) dst[i] = (act ? hy_silu(v[u]) : v[u]) * mul;
         }
+    }
+}
+// Longer portions of a memory with channel gates: queries and gates of the whole portion are made once, in place, before the scan (whose
+// workgroups would each make them again for their few columns): q <- silu(q) (act_q), f <- (1 - lower) sigmoid(-(f + bias)).
+static __global__ __launch_bounds__(256) void hy_mem_prep_kernel(float* __restrict__ proj, int ld, int q_off, int f_off, int cols, int act_q, const float* __restrict__ bias,
+                                                                 const float* __restrict__ lower) {
+    float* row = proj + (size_t)blockIdx.x * ld;
+    for (int c = blockIdx.y * 256 + threadIdx.x; c < cols; c += 256 * gridDim.y) {
+        const float q = row[q_off + c], z = row[f_off + c] + bias[c], lo = lower[c];
+        if (act_q) row[q_off + c] = hy_silu(q);
+        row[f_off + c] = (1.f - lo) * hy_sigmoid(-z);
     }
 }
 // mode 3: (1 - lower) sigmoid(-(row + bias)), zero behind N; eight loads in flight per thread
@@ -1133,7 +1164,7 @@ static __global__ __launch_bounds__(256) void hy_ssm_scan_kernel(HyScanArgs a) {
     for (int t0 = 0; t0 < n; t0 += TB) {
         const int tb = min(TB, n - t0);
         __syncthreads();
-        if constexpr (CG) hy_scan_stage_gate(sB, kbase, a.ldk, t0, tb, N, Ns, a.fbias + (size_t)head * N, a.lower + (size_t)head * N);
+        if (CG && a.fbias) hy_scan_stage_gate(sB, kbase, a.ldk, t0, tb, N, Ns, a.fbias + (size_t)head * N, a.lower + (size_t)head * N);
         else hy_scan_stage(sB, kbase, a.ldk, t0, tb, N, Ns, a.k_mul, a.act & 1);
         hy_scan_stage(sC, qbase, a.ldq, t0, tb, N, Ns, a.q_mul, a.act & 2);
         for (int i = tid; i < tb * cols; i += 256) {

@@ -1016,6 +1016,10 @@ static int32_t hy_mixer_core(gl3_ctx* ctx, HyLayer& L, int np, int ldo, int n, i
         a.ga = ga; a.gb = gb; a.decay = L.decay; a.ones_col = eg ? 1 : 0;
         a.heads = d.heads; a.P = P; a.N = d.dim; a.G = d.heads;
         a.state = h->slots + L.off_state; a.slot_stride = h->slot_floats; a.dyn = h->dyn; a.n = n; a.y = h->ssm_y; a.ldy = ldy;
+        if (cg && n > 32) {
+            hipLaunchKernelGGL(hy_mem_prep_kernel, dim3(n, hy_cdiv(d.heads * d.dim, 1024)), dim3(256), 0, st, h->proj, np, L.q_off, L.f_off, d.heads * d.dim, a.act & 2, a.fbias, a.lower);
+            a.act &= ~2; a.fbias = nullptr;
+        }
         hy_scan(ctx, a);
         const float* gate = d.mem_gate_act == 2 ? nullptr : h->proj;
         const int w_stride = d.mem_norm_weight == 2 ? 0 : d.vdim;
@@ -1259,7 +1263,7 @@ static int32_t hy_portion_plain(gl3_ctx* ctx, int seq, const int32_t* tokens, in
     if (nw > 0) memcpy(h->h_want, want, (size_t)nw * 4);
     h->h_dyn[0] = pos0; h->h_dyn[1] = seq; h->h_dyn[2] = h->last_tok[seq];
     HY_HIP(hipMemcpyAsync(h->dyn, h->h_dyn, (size_t)(4 + h->want_cap + n) * 4, hipMemcpyHostToDevice, st));
-    hipLaunchKernelGGL((hy_embed_kernel<T>), dim3(n, n <= 32 ? hy_cdiv(W, 256) : 1), dim3(256), 0, st, h->tokens, (const T*)h->emb.w, h->X, W, 1, lstride, h->emb_scale, h->depth ? h->hist : nullptr,
+    hipLaunchKernelGGL((hy_embed_kernel<T>), dim3(n, hy_cdiv(W, n <= 32 ? 256 : 1024)), dim3(256), 0, st, h->tokens, (const T*)h->emb.w, h->X, W, 1, lstride, h->emb_scale, h->depth ? h->hist : nullptr,
                        HyBigram{h->bigram.w, h->bg_buckets, h->bg_prev, h->bg_cur}, h->dyn);
     T* hb = (T*)h->h;
     HyResid base{};
@@ -1368,7 +1372,7 @@ static int32_t hy_portion(gl3_ctx* ctx, int seq, const int32_t* tokens, int n, i
     if (nw > 0) memcpy(h->h_want, want, (size_t)nw * 4);
     h->h_dyn[0] = pos0; h->h_dyn[1] = seq;
     HY_HIP(hipMemcpyAsync(h->dyn, h->h_dyn, (size_t)(4 + h->want_cap + n) * 4, hipMemcpyHostToDevice, st));
-    hipLaunchKernelGGL((hy_embed_kernel<T>), dim3(n, n <= 32 ? hy_cdiv(W, 256) : 1), dim3(256), 0, st, h->tokens, (const T*)h->emb.w, h->X, W, S, sstride, h->emb_scale, (float*)nullptr);
+    hipLaunchKernelGGL((hy_embed_kernel<T>), dim3(n, hy_cdiv(W, n <= 32 ? 256 : 1024)), dim3(256), 0, st, h->tokens, (const T*)h->emb.w, h->X, W, S, sstride, h->emb_scale, (float*)nullptr);
     T* hb = (T*)h->h;
     const int nl = (int)h->L.size();
     hy_streams<T>(ctx, n, h->X, W, S, sstride, (const float*)nullptr, 1, 0, (const float*)nullptr, (const float*)nullptr,

@@ -1,4 +1,4 @@
-"""Host side of the layer-list family (GL3_ARCH_LAYERLIST: the Noditar, Vonulix, Kosusun and Kugadra designs) over the C-ABI: model folders (config.json + model.safetensors), the step
+"""Host side of the layer-list family (GL3_ARCH_LAYERLIST: the Noditar, Vonulix, Kosusun, Kugadra and Tutedra designs) over the C-ABI: model folders (config.json + model.safetensors), the step
 function with sequence slots, greedy / sampled generation.  The compute path is csrc/gl3_hybrid.hip; nothing here computes.
 
     plan = HybridPlan.from_dir("model-folder", dtype="bfloat16", ctx=4096, max_batch=512, n_seqs=2)
@@ -282,20 +282,65 @@ def kugadra_tensor_shapes(config: dict) -> dict:
     return out
 
 
+def tutedra_tensor_shapes(config: dict) -> dict:
+    """{tensor name: shape} of a Tutedra configuration, in file order (the head is the embedding table)."""
+    W, V = config["width"], config["vocab"]
+    out = {"embed": (V, W)}
+    bigram = (config.get("embedding") or {}).get("bigram")
+    if bigram:
+        out["bigram"] = (bigram["buckets"] + 1, W)
+    for i, layer in enumerate(config["layers"]):
+        p, m, ff = "l%d." % i, layer["mixer"], layer.get("mlp")
+        nq, od = m["heads"] * m["dim"], m["heads"] * m["vdim"]
+        out[p + "norm1"] = (W,)
+        if layer["type"] == "hgrn2":
+            mix = {"q": (nq, W), "f": (nq, W), "f.b": (nq,), "lower": (nq,), "v": (od, W), "norm": (m["vdim"],)}
+        elif layer["type"] == "mlstm":
+            mix = {"q": (nq, W), "k": (nq, W), "v": (od, W), "g": (od, W), "norm": (od,), "i": (m["heads"], W), "i.b": (m["heads"],), "f": (m["heads"], W), "f.b": (m["heads"],)}
+        else:
+            nk = m["kv_heads"] * m["dim"]
+            mix = {"q": (nq, W), "k": (nk, W), "q.norm": (m["dim"],), "k.norm": (m["dim"],)}
+            if m.get("conv"):
+                mix.update({"q.conv": (nq, m["conv"]), "k.conv": (nk, m["conv"])})
+        out.update({p + "mix." + k: v for k, v in mix.items()})
+        out[p + "mix.o"] = (W, od)
+        if ff:
+            out[p + "norm2"] = (W,)
+            if ff["kind"] == "dense":
+                out.update({p + "mlp.up": (ff["ff"], W), p + "mlp.down": (W, ff["ff"]), p + "mlp.act": (4,)})
+            else:
+                f = ff["expert"]["ff"]
+                for e in range(ff["router"]["experts"]):
+                    out.update({p + "mlp.e%d.up" % e: (f, W), p + "mlp.e%d.down" % e: (W, f)})
+                out.update({p + "mlp.router": (ff["router"]["experts"], W), p + "mlp.correction": (ff["router"]["experts"],)})
+                if ff.get("shared"):
+                    f = ff["shared"]["ff"]
+                    out.update({p + "mlp.shared.up": (f, W), p + "mlp.shared.down": (W, f), p + "mlp.shared.sg": (1, W)})
+            out[p + "ls2"] = (W,)
+        out.update({p + "ls1": (W,), p + "shift": (W,)})
+    out["final.norm"] = (W,)
+    return out
+
+
 def random_model_dir(path: str, config: dict, seed: int = 0):
     """A model folder with random weights for timing: matrices are random bfloat16 bit patterns of magnitude 2^-9 .. 2^-6 / sqrt-free (cheap to
     make at billions of elements), vectors and tables are benign constants with noise."""
     rng = np.random.default_rng(seed)
     S = config.get("streams", 1)
     t = {}
-    vonulix, kosusun, kugadra = (config["architecture"] == a for a in ("Vonulix", "Kosusun", "Kugadra"))
+    vonulix, kosusun, kugadra, tutedra = (config["architecture"] == a for a in ("Vonulix", "Kosusun", "Kugadra", "Tutedra"))
     shapes = (vonulix_tensor_shapes(config) if vonulix else kosusun_tensor_shapes(config) if kosusun else kugadra_tensor_shapes(config) if kugadra
-              else noditar_tensor_shapes(config))
+              else tutedra_tensor_shapes(config) if tutedra else noditar_tensor_shapes(config))
     for name, shp in shapes.items():
         leaf = name.split(".", 1)[1] if name[0] == "l" and name[1].isdigit() else name
         if kosusun and leaf.endswith((".b", ".sink")):
             t[name] = np.full(shp, 3.0 if leaf.endswith("f.b") else 0.0, np.float32)          # forget gates near one, no other offsets
-        elif vonulix and leaf in ("norm1", "norm2", "final.norm"):
+        elif tutedra and leaf in ("mix.f.b", "mix.i.b", "shift", "mix.lower", "ls1", "ls2", "mlp.act"):
+            v = {"mix.f.b": 3.0, "mix.i.b": 0.0, "shift": 0.25, "mix.lower": 0.5, "ls1": 1.0, "ls2": 1.0, "mlp.act": 0.3}[leaf]
+            t[name] = np.full(shp, v, np.float32)
+        elif leaf in ("mix.q.conv", "mix.k.conv"):
+            t[name] = np.full(shp, 1.0 / shp[1], np.float32)
+        elif (vonulix or tutedra) and leaf in ("norm1", "norm2", "final.norm"):
             t[name] = np.zeros(shp, np.float32)                  # the file holds weight - 1
         elif leaf == "mlp.correction":
             t[name] = np.zeros(shp, np.float32)
