@@ -329,16 +329,17 @@ static __global__ __launch_bounds__(256) void hy_gemm_kernel(const T* __restrict
 // wavefront per pair (4 pairs per workgroup); KS = 4: the workgroup's four wavefronts split K of ONE pair and meet in LDS — four times
 // the wavefronts in flight for matrices with few rows.  EPI_GLU: the pair is (gate row, up row) of one feature in the block layout above.
 // Grouped form (GR = 1, mixture of experts, MT = 1): blockIdx.y = a (token, choice) pair whose expert sel[pair] picks the N rows of the
-// stacked matrix; row `pair` of A, C and act belongs to it.
+// stacked matrix; row `pair` of A, C and act belongs to it.  A choice that is no expert (sel[pair] >= n_sel, identity) has no products.
 template <typename T, typename TO, int MT, int EPI, int KS, int GR = 0>
 static __global__ __launch_bounds__(256) void hy_matvec_kernel(const T* __restrict__ A, int lda, const T* __restrict__ Wt, int ldw, int M, int N, int K,
                                                                float* __restrict__ C, int ldc, TO* __restrict__ act, int ld_act, HyGlu glu,
                                                                const int* __restrict__ sel = nullptr, size_t wstride = 0, int a_div = 1,
-                                                               const float* __restrict__ row_scale = nullptr) {
+                                                               const float* __restrict__ row_scale = nullptr, int n_sel = 0) {
     constexpr int PE = HyPiece<T>::N;
     float rs = 1.f;          // grouped: the pair's products are multiplied by row_scale[pair] (a score that scales the expert's input scales W x)
     if constexpr (GR) {
         const int pair_ = blockIdx.y;
+        if (sel[pair_] >= n_sel) return;
         A += (size_t)(pair_ / a_div) * lda;          // a_div = choices per token: the pairs of a token share its row
         if (row_scale) rs = row_scale[pair_];
         Wt += (size_t)sel[pair_] * wstride;
@@ -467,6 +468,48 @@ struct HyPrepX {
     int v_from_k;
     const float* conv_w; int taps; float* tail; float* qout; int ldq; int n;
 };
+// A causal depthwise convolution over time for `len` (<= HY_PREP_MAXD) channels of one token, by one wavefront: crow[d] = sum_j w[j C + d] u_(t - taps + 1 + j)[d],
+// where u are the raw projections (row stride ld, columns from col on) of the step's tokens and, before them, the slot's tail (the last
+// taps - 1 raw rows before the step, row stride C; zeros when the sequence starts here).  move_tail (a step of one token): the tail
+// moves on by this token (every thread the channels it has read).
+__device__ __forceinline__ void hy_conv_row(float* __restrict__ crow, const float* __restrict__ proj, int ld, int col, int t, int len, const float* __restrict__ w_, int C, int taps,
+                                            float* __restrict__ tl, bool fresh, bool move_tail) {
+    const int lane = threadIdx.x, keep = taps - 1;
+    const float* src = proj + (size_t)t * ld + col;
+    // two channels and four taps at a time, their loads issued together (taps that are not there read the token's own row, times 0)
+    for (int d0 = lane; d0 < len; d0 += 128) {
+        float a[2] = {0.f, 0.f};
+        for (int j0 = 0; j0 < taps; j0 += 4) {
+            float u[4][2], w[4][2];
+#pragma unroll
+            for (int k = 0; k < 4; ++k) {
+                const int j = j0 + k, tau = t - keep + j;
+                const bool live = j < taps && (tau >= 0 || !fresh);
+                const float* up = !live ? src : tau >= 0 ? proj + (size_t)tau * ld + col : tl + (size_t)(keep + tau) * C;
+                const float* wp = w_ + (size_t)(j < taps ? j : 0) * C;
+#pragma unroll
+                for (int q = 0; q < 2; ++q) {
+                    const int d = min(d0 + 64 * q, len - 1);
+                    u[k][q] = up[d];
+                    w[k][q] = wp[d];
+                    if (!live) w[k][q] = 0.f;
+                }
+            }
+#pragma unroll
+            for (int k = 0; k < 4; ++k)
+#pragma unroll
+                for (int q = 0; q < 2; ++q) a[q] = fmaf(w[k][q], u[k][q], a[q]);
+        }
+#pragma unroll
+        for (int q = 0; q < 2; ++q)
+            if (d0 + 64 * q < len) crow[d0 + 64 * q] = a[q];
+    }
+    if (move_tail)
+        for (int d = lane; d < len; d += 64) {
+            for (int i = 0; i + 1 < keep; ++i) tl[(size_t)i * C + d] = fresh ? 0.f : tl[(size_t)(i + 1) * C + d];
+            if (keep > 0) tl[(size_t)(keep - 1) * C + d] = src[d];
+        }
+}
 template <typename F>
 __device__ __forceinline__ void hy_turn_store(float* __restrict__ dst, const float* __restrict__ src, int D, int dims, const F* __restrict__ freq, int pos, float r, int lane,
                                               int interleaved = 0, const float* __restrict__ bias = nullptr, const float* __restrict__ w = nullptr) {
@@ -496,42 +539,7 @@ static __global__ __launch_bounds__(64) void hy_attn_prep_kernel(float* __restri
         const float* bias = x.bias ? x.bias + col : nullptr;
         float* dst = isq ? proj + (size_t)t * ld + col : kc + slot + (size_t)pos * (G * D) + (hh - H) * D;
         if (x.taps > 0) {
-            const int C = (H + G) * D, c0 = hh * D, keep = x.taps - 1;
-            float* tl = x.tail + slot + c0;
-            const bool fresh = dyn[0] == 0;
-            // two channels and four taps at a time, their loads issued together (taps that are not there read the token's own row, times 0)
-            for (int d0 = lane; d0 < D; d0 += 128) {
-                float a[2] = {0.f, 0.f};
-                for (int j0 = 0; j0 < x.taps; j0 += 4) {
-                    float u[4][2], w[4][2];
-#pragma unroll
-                    for (int k = 0; k < 4; ++k) {
-                        const int j = j0 + k, tau = t - keep + j;
-                        const bool live = j < x.taps && (tau >= 0 || !fresh);
-                        const float* up = !live ? src : tau >= 0 ? proj + (size_t)tau * ld + col : tl + (size_t)(keep + tau) * C;
-                        const float* wp = x.conv_w + (size_t)(j < x.taps ? j : 0) * C + c0;
-#pragma unroll
-                        for (int q = 0; q < 2; ++q) {
-                            const int d = min(d0 + 64 * q, D - 1);
-                            u[k][q] = up[d];
-                            w[k][q] = wp[d];
-                            if (!live) w[k][q] = 0.f;
-                        }
-                    }
-#pragma unroll
-                    for (int k = 0; k < 4; ++k)
-#pragma unroll
-                        for (int q = 0; q < 2; ++q) a[q] = fmaf(w[k][q], u[k][q], a[q]);
-                }
-#pragma unroll
-                for (int q = 0; q < 2; ++q)
-                    if (d0 + 64 * q < D) crow[d0 + 64 * q] = a[q];
-            }
-            if (x.n == 1)
-                for (int d = lane; d < D; d += 64) {
-                    for (int i = 0; i + 1 < keep; ++i) tl[(size_t)i * C + d] = fresh ? 0.f : tl[(size_t)(i + 1) * C + d];
-                    if (keep > 0) tl[(size_t)(keep - 1) * C + d] = src[d];
-                }
+            hy_conv_row(crow, proj, ld, col, t, D, x.conv_w + hh * D, (H + G) * D, x.taps, x.tail + slot + hh * D, dyn[0] == 0, x.n == 1);
             __syncthreads();
             src = crow;
             if (isq) dst = x.qout + (size_t)t * x.ldq + hh * D;

@@ -8,7 +8,10 @@
 // ---- residual update ----------------------------------------------------------------------------------------------------------------
 // One workgroup per token.  In this order, every part optional (null pointer = absent):
 //   d  = ya_mul * ga * sum_z ya[z]              ya: a sublayer's output (or several sublayers' outputs), possibly as K-split parts; ga = sigmoid(gate_z[t * gate_ld]) or 1
-//   d += sum_k ew[t top + k] eo[pair_row[t top + k]]   the routed experts' down projections of this token (ew: a weight per pair, null = 1)
+//                                               with bw1 (BR = true): two mixers' outputs, the first ya_first parts and the others, each normed on its own:
+//                                               d = N(first) bw1 + N(others) bw2, N(y) = y / sqrt(mean(y^2) + eps) (the weights hold the mixers' multipliers)
+//   d += sum_k ew[t top + k] eo[pair_row[t top + k]]   the routed experts' down projections of this token (ew: a weight per pair, null = 1); a pair_row
+//                                               of -1 is an identity choice: the sublayer's input row, id_x (float32) or h_out as the sublayer read it
 //   x += d, or with post_w: x += d / sqrt(mean(d^2) + eps) * post_w    (the sublayer's output passes a norm of its own before it joins the residual);
 //                                               with lw the addend is multiplied by lw[w] first (a scale per column)
 //   x += yc / sqrt(mean(yc^2) + eps) * cw       a unit-RMS normed input with a plain weight
@@ -22,7 +25,8 @@
 struct HyResid {
     float* x; int W;
     const float* ya; int ya_parts; size_t ya_stride; const float* gate_z; int gate_ld; float ya_mul;
-    const float* eo; const int* pair_row; int top; const float* ew;
+    const float* bw1; const float* bw2; int ya_first;
+    const float* eo; const int* pair_row; int top; const float* ew; const float* id_x;
     const float* post_w; const float* lw;
     const float* yc; const float* cw;
     float* hist; size_t hist_stride; int n_mix; const float* mix;      // hist_out = hist + (n_mix - 1) hist_stride
@@ -37,6 +41,12 @@ template <int V> __device__ __forceinline__ void hy_ldv(const float* __restrict_
     if constexpr (V == 4) { const float4 t = *reinterpret_cast<const float4*>(p); v[0] = t.x; v[1] = t.y; v[2] = t.z; v[3] = t.w; }
     else v[0] = *p;
 }
+template <int V> __device__ __forceinline__ void hy_ldv(const bf16_t* __restrict__ p, float* v) {
+    if constexpr (V == 4) {
+        const uint2 t = *reinterpret_cast<const uint2*>(p);
+        v[0] = __uint_as_float(t.x << 16); v[1] = __uint_as_float(t.x & 0xffff0000u); v[2] = __uint_as_float(t.y << 16); v[3] = __uint_as_float(t.y & 0xffff0000u);
+    } else v[0] = hy_bf2f(*p);
+}
 template <int V> __device__ __forceinline__ void hy_stv(float* __restrict__ p, const float* v) {
     if constexpr (V == 4) *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]);
     else *p = v[0];
@@ -50,8 +60,8 @@ template <int V> __device__ __forceinline__ void hy_stv(bf16_t* __restrict__ p, 
     } else *p = hy_f2bf(v[0]);
 }
 constexpr int HY_RC = 2, HY_MAX_PARTS = 4, HY_MIX_UNROLL = 4;
-template <typename TO, int NT, int V>
-static __global__ __launch_bounds__(NT) void hy_resid_kernel(HyResid a, TO* __restrict__ xt, TO* __restrict__ h_out) {
+template <typename TO, int NT, int V, bool BR>
+static __global__ __launch_bounds__(NT) void hy_resid_kernel(HyResid a, TO* __restrict__ xt, TO* h_out) {
     __shared__ float red[NT / 64];
     const int t = blockIdx.x, W = a.W;
     const size_t row = (size_t)t * W;
@@ -68,30 +78,79 @@ static __global__ __launch_bounds__(NT) void hy_resid_kernel(HyResid a, TO* __re
         cr = 1.f / sqrtf(ss / (float)W + a.eps);
     }
     const float ga = (a.gate_z ? hy_sigmoid(a.gate_z[(size_t)t * a.gate_ld]) : 1.f) * a.ya_mul;
-    float pr = 0.f;          // post_w: 1 / rms of the sublayer's whole output (the same sums as below, once more)
+    // column w of the sum of parts z0 .. z1 - 1 (the first HY_MAX_PARTS loads issued together)
+    auto parts = [&](int w, int z0, int z1, float* y) {
+        float p[HY_MAX_PARTS][V];
+#pragma unroll
+        for (int i = 0; i < V; ++i) y[i] = 0.f;
+#pragma unroll
+        for (int z = 0; z < HY_MAX_PARTS; ++z)
+            if (z0 + z < z1) hy_ldv<V>(a.ya + (z0 + z) * a.ya_stride + row + w, p[z]);
+#pragma unroll
+        for (int z = 0; z < HY_MAX_PARTS; ++z)
+            if (z0 + z < z1)
+#pragma unroll
+                for (int i = 0; i < V; ++i) y[i] += p[z][i];
+        for (int z = z0 + HY_MAX_PARTS; z < z1; ++z) {
+            float q[V];
+            hy_ldv<V>(a.ya + z * a.ya_stride + row + w, q);
+#pragma unroll
+            for (int i = 0; i < V; ++i) y[i] += q[i];
+        }
+    };
+    float b1 = 0.f, b2 = 0.f;          // two normed mixers: 1 / rms of each one's whole output
+    if constexpr (BR) {
+        for (int w = threadIdx.x * V; w < W; w += NT * V) {
+            float y[V], z[V];
+            parts(w, 0, a.ya_first, y);
+            parts(w, a.ya_first, a.ya_parts, z);
+#pragma unroll
+            for (int i = 0; i < V; ++i) { b1 += y[i] * y[i]; b2 += z[i] * z[i]; }
+        }
+        b1 = hy_block_sum<NT>(b1, red);
+        b2 = hy_block_sum<NT>(b2, red);
+        b1 = 1.f / sqrtf(b1 / (float)W + a.eps);
+        b2 = 1.f / sqrtf(b2 / (float)W + a.eps);
+    }
+    // column w of what joins the residual: y (the sublayer's output) and e (the routed experts')
+    auto addend = [&](int w, float* y, float* e) {
+#pragma unroll
+        for (int i = 0; i < V; ++i) y[i] = e[i] = 0.f;
+        if constexpr (BR) {
+            float z[V], w1[V], w2[V];
+            parts(w, 0, a.ya_first, y);
+            parts(w, a.ya_first, a.ya_parts, z);
+            hy_ldv<V>(a.bw1 + w, w1);
+            hy_ldv<V>(a.bw2 + w, w2);
+#pragma unroll
+            for (int i = 0; i < V; ++i) y[i] = y[i] * b1 * w1[i] + z[i] * b2 * w2[i];
+        } else if (a.ya) parts(w, 0, a.ya_parts, y);
+        if (a.eo)
+            for (int k = 0; k < a.top; ++k) {
+                float q[V];
+                const int pr = a.pair_row[t * a.top + k];
+                if (pr >= 0) hy_ldv<V>(a.eo + (size_t)pr * W + w, q);
+                else if (a.id_x) hy_ldv<V>(a.id_x + row + w, q);
+                else hy_ldv<V>((const TO*)h_out + row + w, q);
+                const float wk = a.ew ? a.ew[t * a.top + k] : 1.f;
+#pragma unroll
+                for (int i = 0; i < V; ++i) e[i] = fmaf(wk, q[i], e[i]);
+            }
+    };
+    float pr = 0.f, kept[HY_RC][V];          // post_w: 1 / rms of the sublayer's whole output; its first chunks stay in registers for the sum below
     if (a.post_w) {
         float sd = 0.f;
-        for (int w = threadIdx.x * V; w < W; w += NT * V) {
+        int it = 0;
+        for (int w = threadIdx.x * V; w < W; w += NT * V, ++it) {
             float y[V], e[V];
+            addend(w, y, e);
 #pragma unroll
-            for (int i = 0; i < V; ++i) y[i] = e[i] = 0.f;
-            if (a.ya)
-                for (int z = 0; z < a.ya_parts; ++z) {
-                    float q[V];
-                    hy_ldv<V>(a.ya + z * a.ya_stride + row + w, q);
+            for (int i = 0; i < V; ++i) { y[i] = ga * y[i] + e[i]; sd += y[i] * y[i]; }
 #pragma unroll
-                    for (int i = 0; i < V; ++i) y[i] += q[i];
-                }
-            if (a.eo)
-                for (int k = 0; k < a.top; ++k) {
-                    float q[V];
-                    hy_ldv<V>(a.eo + (size_t)a.pair_row[t * a.top + k] * W + w, q);
-                    const float wk = a.ew ? a.ew[t * a.top + k] : 1.f;
+            for (int q = 0; q < HY_RC; ++q)
+                if (q == it)
 #pragma unroll
-                    for (int i = 0; i < V; ++i) e[i] = fmaf(wk, q[i], e[i]);
-                }
-#pragma unroll
-            for (int i = 0; i < V; ++i) { const float d = ga * y[i] + e[i]; sd += d * d; }
+                    for (int i = 0; i < V; ++i) kept[q][i] = y[i];
         }
         sd = hy_block_sum<NT>(sd, red);
         pr = 1.f / sqrtf(sd / (float)W + a.eps);
@@ -102,38 +161,25 @@ static __global__ __launch_bounds__(NT) void hy_resid_kernel(HyResid a, TO* __re
         float x[V], y[V], e[V], c[V], cw[V];
         hy_ldv<V>(a.x + row + w, x);
 #pragma unroll
-        for (int i = 0; i < V; ++i) y[i] = e[i] = c[i] = 0.f;
-        if (a.ya) {
-            float p[HY_MAX_PARTS][V];
+        for (int i = 0; i < V; ++i) c[i] = 0.f;
+        if (a.post_w && it < HY_RC) {
 #pragma unroll
-            for (int z = 0; z < HY_MAX_PARTS; ++z)
-                if (z < a.ya_parts) hy_ldv<V>(a.ya + z * a.ya_stride + row + w, p[z]);
+            for (int q = 0; q < HY_RC; ++q)
+                if (q == it)
 #pragma unroll
-            for (int z = 0; z < HY_MAX_PARTS; ++z)
-                if (z < a.ya_parts)
+                    for (int i = 0; i < V; ++i) y[i] = kept[q][i];
+        } else {
+            addend(w, y, e);
+            if (a.post_w)
 #pragma unroll
-                    for (int i = 0; i < V; ++i) y[i] += p[z][i];
-            for (int z = HY_MAX_PARTS; z < a.ya_parts; ++z) {
-                float q[V];
-                hy_ldv<V>(a.ya + z * a.ya_stride + row + w, q);
-#pragma unroll
-                for (int i = 0; i < V; ++i) y[i] += q[i];
-            }
+                for (int i = 0; i < V; ++i) y[i] = ga * y[i] + e[i];
         }
-        if (a.eo)
-            for (int k = 0; k < a.top; ++k) {
-                float q[V];
-                hy_ldv<V>(a.eo + (size_t)a.pair_row[t * a.top + k] * W + w, q);
-                const float wk = a.ew ? a.ew[t * a.top + k] : 1.f;
-#pragma unroll
-                for (int i = 0; i < V; ++i) e[i] = fmaf(wk, q[i], e[i]);
-            }
         if (a.yc) { hy_ldv<V>(a.yc + row + w, c); hy_ldv<V>(a.cw + w, cw); }
         if (a.post_w) {
             float pw[V];
             hy_ldv<V>(a.post_w + w, pw);
 #pragma unroll
-            for (int i = 0; i < V; ++i) y[i] = (ga * y[i] + e[i]) * pr * pw[i];
+            for (int i = 0; i < V; ++i) y[i] = y[i] * pr * pw[i];
             if (a.lw) {
                 float lw[V];
                 hy_ldv<V>(a.lw + w, lw);
@@ -271,15 +317,16 @@ static __global__ __launch_bounds__(256) void hy_side_act_kernel(const float* __
 // pstride apart); score = sigmoid(z), or softmax(z) over all E experts (HyRoute.softmax); the `top` largest of score (+ bias[e], where
 // bias != null: it decides the choice only) are taken in descending order (the lowest index wins a tie): sel[t top + k], wgt[t top + k] =
 // the chosen expert's score (without the bias), divided by the chosen scores' sum + 1e-20 (renorm), times mul.  E <= 64 * HY_RT_PER, top <= 64.
-// groups > 0: the experts form that many equal runs of neighbours; a run's score is the sum of its two largest choice scores, and only
-// experts of the `keep` best runs (the lowest index wins a tie) can be chosen (top <= keep E / groups).
-// pair_row != null (a few tokens): the pairs keep their own order, pair_row[p] = p.  extra_out != null: column E of z (the shared
+// groups > 0: the experts form that many equal runs of neighbours; a run's score is the sum of its two largest choice scores (group_max: its
+// largest alone), and only experts of the `keep` best runs (the lowest index wins a tie) can be chosen (top <= keep E / groups).  The last
+// outputs from `real` on are identity choices (E counts them).
+// pair_row != null (a few tokens): the pairs keep their own order, pair_row[p] = p (-1 for an identity choice).  extra_out != null: column E of z (the shared
 // expert's gate logit) is summed into extra_out[t].
 constexpr int HY_RT_PER = 16;
-struct HyRoute { int softmax; const float* bias; int renorm; float mul; int groups, keep; };
+struct HyRoute { int softmax; const float* bias; int renorm; float mul; int groups, keep; int real, group_max; };
 static __global__ __launch_bounds__(64) void hy_route_kernel(const float* __restrict__ z, int ldz, int parts, size_t pstride, int E, int top, int* __restrict__ sel,
                                                              float* __restrict__ wgt, int* __restrict__ pair_row, float* __restrict__ extra_out,
-                                                             HyRoute rt = HyRoute{0, nullptr, 0, 1.f, 0, 0}) {
+                                                             HyRoute rt) {
     const int t = blockIdx.x, lane = threadIdx.x;
     constexpr float GONE = -3.0e38f;
     float s[HY_RT_PER], c[HY_RT_PER];          // score; what the choice goes by
@@ -324,7 +371,7 @@ static __global__ __launch_bounds__(64) void hy_route_kernel(const float* __rest
                 const float v = cs[g * gs + j];
                 if (v > b1) { b2 = b1; b1 = v; } else if (v > b2) b2 = v;
             }
-            gsc[g] = gs > 1 ? b1 + b2 : b1;
+            gsc[g] = gs > 1 && !rt.group_max ? b1 + b2 : b1;
         }
         __syncthreads();
         // an expert stays open if fewer than `keep` groups stand before its own
@@ -363,13 +410,14 @@ static __global__ __launch_bounds__(64) void hy_route_kernel(const float* __rest
     if (lane < top) {
         sel[t * top + lane] = mysel;
         wgt[t * top + lane] = (rt.renorm || rt.mul != 1.f) ? myw * (rt.mul / (rt.renorm ? wsum + 1e-20f : 1.f)) : myw;
-        if (pair_row) pair_row[t * top + lane] = t * top + lane;
+        if (pair_row) pair_row[t * top + lane] = mysel < rt.real ? t * top + lane : -1;
     }
 }
 
 // Grouping for portions of many tokens: the P = n top (token, choice) pairs are ordered by expert.  pair_row[p] = the pair's row in that
 // order; tiles = {first row, rows (<= BM), expert} per BM rows of an expert, ntiles[0] their count (<= P / BM + min(E, P)).  One
-// workgroup; the order inside an expert's rows is arbitrary (a row's result does not depend on its place).  LDS: 2 E ints.
+// workgroup; the order inside an expert's rows is arbitrary (a row's result does not depend on its place).  A choice sel[p] >= E (identity) has no
+// row: pair_row[p] = -1.  LDS: 2 E ints.
 static __global__ __launch_bounds__(256) void hy_moe_group_kernel(const int* __restrict__ sel, int P, int E, int BM, int* __restrict__ pair_row, int* __restrict__ tiles,
                                                                   int* __restrict__ ntiles) {
     extern __shared__ int gsm[];
@@ -377,7 +425,8 @@ static __global__ __launch_bounds__(256) void hy_moe_group_kernel(const int* __r
     int* off = gsm + E;      // [E] first row of the expert
     for (int e = threadIdx.x; e < E; e += 256) cnt[e] = 0;
     __syncthreads();
-    for (int p = threadIdx.x; p < P; p += 256) atomicAdd(&cnt[sel[p]], 1);
+    for (int p = threadIdx.x; p < P; p += 256)
+        if (sel[p] < E) atomicAdd(&cnt[sel[p]], 1);
     __syncthreads();
     if (threadIdx.x == 0) {
         int row = 0, nt = 0;
@@ -392,13 +441,14 @@ static __global__ __launch_bounds__(256) void hy_moe_group_kernel(const int* __r
     __syncthreads();
     for (int e = threadIdx.x; e < E; e += 256) cnt[e] = off[e];
     __syncthreads();
-    for (int p = threadIdx.x; p < P; p += 256) pair_row[p] = atomicAdd(&cnt[sel[p]], 1);
+    for (int p = threadIdx.x; p < P; p += 256) pair_row[p] = sel[p] < E ? atomicAdd(&cnt[sel[p]], 1) : -1;
 }
 // The experts' operand: row pair_row[p] = wgt[p] * h[token of p] (a score scales its expert's INPUT; wgt = null: the plain row), in the matrix type.
 template <typename T>
 static __global__ __launch_bounds__(256) void hy_moe_scale_kernel(const T* __restrict__ h, int W, int top, const float* __restrict__ wgt, const int* __restrict__ pair_row,
                                                                   T* __restrict__ out) {
     const int p = blockIdx.x, t = p / top;
+    if (pair_row[p] < 0) return;
     const float s = wgt ? wgt[p] : 1.f;
     T* dst = out + (size_t)pair_row[p] * W;
     for (int w = threadIdx.x; w < W; w += 256) hy_st(dst + w, s * hy_ld(h + (size_t)t * W + w));

@@ -28,11 +28,16 @@ struct HyLayer {
     int mo_total = 0;          // columns of o: this mixer's heads * vdim plus the side mixer's
     float out_mul = 1.f;
     HyLayer* side = nullptr;   // owned
-    HyMat o;                   // the mixer's output projection [width x mo_total]
+    HyMat o;                   // the mixer's output projection [width x mo_total]; with out_norm each mixer has one of its own [width x its heads * vdim]
     float* pbias = nullptr;    // bias per row of the fused projection (null: no mixer of the layer has biases)
     float *qn = nullptr, *kn = nullptr, *sink = nullptr;      // attention: weights of the q / k norms (whole projection or per head), learned sink logits
     float* qk_conv_w = nullptr;                               // attention: taps of the q and k channels, [taps][(heads + kv_heads) dim]
     float* mem_lower = nullptr;                               // matrix memory, channel gates: lower bounds [heads dim]
+    // attention: multipliers of the heads' scores [heads], transposed mixing matrix [mix_ld][mix_ld] (zero padded); gated delta rule: taps of the q, k
+    // and v channels in row order, [taps][2 kv_heads dim + heads vdim] (its tail: off_tail); two normed mixers: norm weight of this one's
+    // projected output, times its multiplier [width]
+    float *head_temp = nullptr, *head_mixT = nullptr, *mem_conv_w = nullptr, *branch_norm = nullptr;
+    int mix_ld = 0;
     float *shift_mu = nullptr, *ls1 = nullptr, *ls2 = nullptr, *poly = nullptr;      // token shift, layer scales, coefficients of the polynomial activation
     size_t off_shift = 0;                                     // float offset inside a slot: the previous token's normed row
     float* decay = nullptr;    // matrix memory: fixed decay per head
@@ -84,6 +89,7 @@ struct gl3_hybrid_state {
     HyMat bigram;              // rows of token pairs [buckets + 1][W] (buckets = 0: none)
     int bg_buckets = 0, bg_prev = 0, bg_cur = 0;
     float *hf = nullptr, *ffz = nullptr;             // normed rows in float32 [mb][W]; up products of a polynomial feed-forward, K-split parts of [mb][ff_pad]
+    bool no_pre = false;       // the sublayers read the residual itself
     bool post_norms = false;   // every sublayer's output passes an RMS norm with its own weight before it joins the residual
     float softcap = 0.f;       // logits <- cap tanh(logits / cap); 0 = none
     void* cq = nullptr;        // latent with q_rank: the normed query latents [mb][max q_rank], matrix type
@@ -114,6 +120,7 @@ struct gl3_hybrid_state {
     float* h_logits = nullptr;                                       // pinned [want_cap][vocab]
     size_t part_rows = 0;
     int last_n = 0;
+    int y_first = 1;           // of these, the first mixer's (two normed mixers side by side)
     int y_parts = 1;           // partial sums the last output / down projection left in y (added by the streams kernel)
 };
 

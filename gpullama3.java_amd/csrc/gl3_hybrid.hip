@@ -1,7 +1,7 @@
 // gl3_hybrid.hip — the layer-list family (GL3_ARCH_LAYERLIST) behind the C-ABI: a model is a list of layers, each with its own token mixer
 // (softmax attention over cached keys / values, attention over a cached low-rank latent — optionally with a query latent, a rotated key
 // part shared by all heads and rows that a later layer reads too —, a state-space recurrence, a matrix memory with a fixed decay or
-// exponential gates or a gate per key channel), an optional feed-forward (gated, relu^2 or a normed polynomial, dense or a mixture of
+// exponential gates or a gate per key channel, or the gated delta rule), an optional feed-forward (gated, relu^2 or a normed polynomial, dense or a mixture of
 // experts with a shared expert and a sigmoid or softmax router, optionally over groups of experts), and either several residual streams
 // that per-sublayer tables read from and write to, or one plain residual stream with an optional per-layer token input, a weighted average
 // over all earlier layers' results, one norm for both sublayers of a layer, a norm or a scale per column behind every sublayer, a token
@@ -19,6 +19,7 @@
 #include "gl3_hybrid.h"
 #include "gl3_decode_kernels.h"      // argmax_kernel
 #include "gl3_hy_kernels.h"
+#include "gl3_hy_heads_kernels.h"
 #include "gl3_hy_plain_kernels.h"
 
 using gl3::AMX_WGS;
@@ -59,19 +60,25 @@ static int32_t hy_alloc_mat(gl3_ctx* ctx, HyMat& m, int rows, int k, int ld) {
 
 // ---- shapes -----------------------------------------------------------------------------------------------------------------------
 static int hy_gate_rows(const gl3_layer_desc& d) { return d.mixer == GL3_MIX_MEMORY ? (d.mem_gate_act == 2 ? 0 : d.heads * d.vdim) : d.out_gate == 2 ? d.heads : d.out_gate ? d.heads * d.vdim : 0; }
+// query / key heads of a matrix memory
+static int hy_mem_kvh(const gl3_layer_desc& d) { return d.mem_gates == GL3_MEM_DELTA ? d.kv_heads : d.heads; }
+// channels of the gated delta rule's convolutions
+static int hy_delta_ch(const gl3_layer_desc& d) { return 2 * d.kv_heads * d.dim + d.heads * d.vdim; }
+// attention whose scores need more than hy_attn_kernel makes
+static bool hy_by_heads(const gl3_layer_desc& d) { return d.head_temp || d.head_mix || d.score_softcap > 0.f || d.chunk > 0; }
 // rows of ONE mixer's part of the fused input projection
 static int hy_proj_rows(const gl3_layer_desc& d) {
     switch (d.mixer) {
         case GL3_MIX_ATTENTION: return d.heads * d.dim + d.kv_heads * d.dim + (d.v_from_k ? 0 : d.kv_heads * d.vdim) + hy_gate_rows(d);
         case GL3_MIX_LATENT: return (d.q_rank > 0 ? d.q_rank : d.heads * (d.dim + d.rot_dim)) + (d.kv_share > 0 ? 0 : d.kv_rank + d.rot_dim) + hy_gate_rows(d);
-        case GL3_MIX_MEMORY: return 2 * d.heads * d.dim + d.heads * d.vdim + hy_gate_rows(d) + (d.mem_gates == GL3_MEM_EXP_GATES ? 2 * d.heads : 0);
+        case GL3_MIX_MEMORY: return 2 * hy_mem_kvh(d) * d.dim + d.heads * d.vdim + hy_gate_rows(d) + (d.mem_gates == GL3_MEM_EXP_GATES || d.mem_gates == GL3_MEM_DELTA ? 2 * d.heads : 0);
         default: return 2 * d.heads * d.vdim + 2 * d.groups * d.state + d.heads;
     }
 }
 static int hy_mix_out(const gl3_layer_desc& d) { return d.heads * d.vdim; }
 // the fused input projection may come in K-split parts (room for HY_KSPLIT copies in the plan's scratch)
 static bool hy_narrow_proj(const gl3_layer_desc& d) { return d.mixer == GL3_MIX_LATENT && d.q_rank > 0; }
-static bool hy_has_bias(const gl3_layer_desc& d) { return (d.mixer == GL3_MIX_ATTENTION && d.qk_bias) || (d.mixer == GL3_MIX_MEMORY && d.mem_gates != GL3_MEM_DECAY); }
+static bool hy_has_bias(const gl3_layer_desc& d) { return (d.mixer == GL3_MIX_ATTENTION && d.qk_bias) || (d.mixer == GL3_MIX_MEMORY && (d.mem_gates == GL3_MEM_EXP_GATES || d.mem_gates == GL3_MEM_CHANNEL_GATES)); }
 static bool hy_ungated(const gl3_layer_desc& d) { return d.ff_act >= 2; }          // the feed-forward (experts and shared expert too) has up rows alone
 static int hy_qk_ch(const gl3_layer_desc& d) { return (d.heads + d.kv_heads) * d.dim; }
 static int hy_conv_ch(const gl3_layer_desc& d) { return d.heads * d.vdim + 2 * d.groups * d.state; }
@@ -85,17 +92,23 @@ static const char* hy_check_layer(const gl3_layer_desc& d) {
         if (d.ff < 1) return "mixture of experts: ff (one expert's width) must be positive";
         if (d.ff_act == 3) return "mixture of experts: the polynomial activation is for dense feed-forwards";
         if (d.ff_act == 2 && !d.route_on_output) return "mixture of experts: experts without a gate are weighted at their output (route_on_output)";
-        if (d.experts + (d.shared_ff > 0 ? 1 : 0) > 64 * HY_RT_PER) return "mixture of experts: at most 1024 router rows (experts, plus one for a shared expert's gate)";
-        if (d.top < 1 || d.top > d.experts || d.top > 64) return "mixture of experts: 1 <= top <= min(experts, 64)";
-        if (d.route_groups < 0 || (d.route_groups > 0 && (d.experts % d.route_groups || d.route_keep < 1 || d.route_keep > d.route_groups ||
-                                                          d.top > d.route_keep * (d.experts / d.route_groups))))
-            return "mixture of experts: route_groups must divide the experts and the route_keep best groups must hold at least top of them";
-    } else if (d.shared_ff > 0)
+        if (d.identity < 0 || (d.identity > 0 && !d.route_on_output)) return "mixture of experts: identity choices need route_on_output";
+        const int rows = d.experts + d.identity;
+        if (rows + (d.shared_ff > 0 ? 1 : 0) > 64 * HY_RT_PER) return "mixture of experts: at most 1024 router rows (experts and identity choices, plus one for a shared expert's gate)";
+        if (d.top < 1 || d.top > rows || d.top > 64) return "mixture of experts: 1 <= top <= min(experts + identity, 64)";
+        if (d.route_groups < 0 || (d.route_groups > 0 && (rows % d.route_groups || d.route_keep < 1 || d.route_keep > d.route_groups ||
+                                                          d.top > d.route_keep * (rows / d.route_groups))))
+            return "mixture of experts: route_groups must divide the choices and the route_keep best groups must hold at least top of them";
+    } else if (d.identity)
+        return "identity choices need a mixture of experts";
+    else if (d.shared_ff > 0)
         return "a shared expert needs a mixture of experts";
     if (d.mixer != GL3_MIX_ATTENTION && (d.v_unit_norm || d.v_rot || d.window > 0 || d.keep_first > 0 || d.pool > 0 || d.qk_bias))
         return "value norm / rotation, windows, pooled blocks and q / k / v biases belong to the attention mixer";
     if (d.mixer != GL3_MIX_ATTENTION && d.mixer != GL3_MIX_MEMORY && d.rot_dims) return "rotary positions belong to the attention and matrix-memory mixers";
     if (d.mixer != GL3_MIX_ATTENTION && (d.qk_conv || d.v_from_k)) return "q / k convolutions and values taken from the keys belong to the attention mixer";
+    if (d.mixer != GL3_MIX_ATTENTION && (d.head_temp || d.head_mix || d.score_softcap != 0.f || d.chunk)) return "head temperatures, mixed heads, capped scores and chunks belong to the attention mixer";
+    if ((d.mixer != GL3_MIX_MEMORY || d.mem_gates != GL3_MEM_DELTA) && (d.mem_conv || d.mem_qk_unit)) return "mem_conv and mem_qk_unit belong to the gated delta rule";
     if (d.ff_act < 0 || d.ff_act > 3) return "ff_act must be 0, 1, 2 or 3";
     if (d.rot_wave_factor < 0.f || (d.rot_wave_factor > 0.f && !(d.rot_wave_low > 0.f && d.rot_wave_high >= d.rot_wave_low && d.rot_wave_original > 0.f)))
         return "frequencies rescaled by wavelength need original > 0 and 0 < low <= high";
@@ -115,6 +128,10 @@ static const char* hy_check_layer(const gl3_layer_desc& d) {
         if (d.qk_conv > 0 && (d.qk_unit_norm == 2 || d.qk_bias)) return "attention: q / k convolutions go without biases and without norms over a whole projection";
         if (d.pool < 0 || (d.pool > 0 && d.window <= 0)) return "attention: pooled blocks need a window";
         if (d.pool > 0 && d.slope_log2 != 0.f) return "attention: pooled blocks have no distance term";
+        if (d.chunk < 0 || d.score_softcap < 0.f) return "attention: chunk and score_softcap must be >= 0";
+        if (hy_by_heads(d) && (d.window > 0 || d.keep_first > 0 || d.pool > 0 || d.slope_log2 != 0.f))
+            return "attention: head temperatures, mixed heads, capped scores and chunks go without windows, pooled blocks and a distance term";
+        if (hy_by_heads(d) && d.heads > HY_HEADS_MAX) return "attention: at most 128 heads with head temperatures, mixed heads, capped scores or chunks";
     } else if (d.mixer == GL3_MIX_LATENT) {
         if (d.dim < 1 || d.kv_rank < 1) return "latent attention: dim and kv_rank must be positive";
         if (d.rot_dim < 0 || (d.rot_dim & 1)) return "latent attention: rot_dim must be even and >= 0";
@@ -123,11 +140,18 @@ static const char* hy_check_layer(const gl3_layer_desc& d) {
         if (d.rot_dim > 0 && d.rot_yarn_factor > 0.f && !(d.rot_yarn_original > 0.f && d.rot_yarn_fast > 0.f && d.rot_yarn_slow > 0.f && d.rot_base != 1.f))
             return "latent attention: scaled frequencies need original, fast and slow > 0";
         if (d.q_rank < 0 || d.kv_share < 0) return "latent attention: q_rank and kv_share must be >= 0";
+        if (d.softmax_sink < 0 || d.softmax_sink > 2) return "latent attention: softmax_sink must be 0 .. 2";
     } else if (d.mixer == GL3_MIX_MEMORY) {
         if (d.dim < 1 || d.dim > 2048) return "matrix memory: 1 <= dim <= 2048";
         if (d.rot_dims < 0 || d.rot_dims > d.dim || (d.rot_dims & 1)) return "matrix memory: rot_dims must be even and at most dim";
         if (d.rot_dims && !(d.rot_base > 0.f)) return "matrix memory: rot_base must be positive";
-        if (d.mem_gates != GL3_MEM_DECAY && d.mem_gates != GL3_MEM_EXP_GATES && d.mem_gates != GL3_MEM_CHANNEL_GATES) return "matrix memory: unknown mem_gates";
+        if (d.mem_gates < GL3_MEM_DECAY || d.mem_gates > GL3_MEM_DELTA) return "matrix memory: unknown mem_gates";
+        if (d.mem_gates == GL3_MEM_DELTA) {
+            if (d.kv_heads < 1 || d.heads % d.kv_heads) return "gated delta rule: heads must be a multiple of kv_heads";
+            if (d.mem_conv < 1 || d.mem_conv > 64) return "gated delta rule: 1 <= mem_conv <= 64";
+            if (d.dim > HY_PREP_MAXD || d.vdim > HY_PREP_MAXD) return "gated delta rule: dim and vdim <= 1024";
+            if (d.rot_dims || d.mem_norm_whole || d.mem_qkv_act == 2) return "gated delta rule: no rotation, no norm over all heads, and q, k and v activated alike";
+        }
         if (d.mem_gate_act < 0 || d.mem_gate_act > 2 || d.mem_norm_weight < 0 || d.mem_norm_weight > 2 || d.mem_qkv_act < 0 || d.mem_qkv_act > 2)
             return "matrix memory: mem_gate_act, mem_norm_weight and mem_qkv_act must be 0, 1 or 2";
         if (d.mem_norm_whole && d.mem_norm_weight == 2) return "matrix memory: one norm over all heads has a weight per entry";
@@ -154,7 +178,8 @@ int32_t gl3_hy_create(const gl3_model_desc* desc, gl3_ctx** out, std::string& er
     if (desc->dim < 1 || desc->vocab < 1 || desc->ctx < 1) { err = "layer-list family: dim, vocab and ctx must be positive"; return GL3_E_ARG; }
     if (desc->weight_type != GL3_TYPE_BF16 && desc->weight_type != GL3_TYPE_F32) { err = "layer-list family: weight_type must be GL3_TYPE_BF16 (or GL3_TYPE_F32)"; return GL3_E_UNSUPPORTED; }
     if (desc->tp_size > 1) { err = "layer-list family: tensor parallelism is not built"; return GL3_E_UNSUPPORTED; }
-    if (desc->post_norms && (desc->streams > 0 || desc->side_dim || desc->depth_mix || desc->parallel_block)) { err = "layer-list family: post norms need the plain residual without token input, depth average and parallel block"; return GL3_E_ARG; }
+    if (desc->post_norms && (desc->streams > 0 || desc->depth_mix || desc->parallel_block)) { err = "layer-list family: post norms need the plain residual without depth average and parallel block"; return GL3_E_ARG; }
+    if (desc->no_pre_norms && (!desc->post_norms || desc->token_shift)) { err = "layer-list family: sublayers that read the residual itself need post norms and no token shift"; return GL3_E_ARG; }
     if (desc->streams > 0 && (desc->token_shift || desc->layer_scale || desc->bigram_buckets)) { err = "layer-list family: token shift, layer scales and token-pair embeddings need the plain residual (streams = 0)"; return GL3_E_ARG; }
     if (desc->parallel_block && (desc->token_shift || desc->layer_scale)) { err = "layer-list family: token shift and layer scales need separate sublayers (no parallel block)"; return GL3_E_ARG; }
     if (desc->bigram_buckets < 0 || desc->bigram_mul_prev < 0 || desc->bigram_mul_cur < 0) { err = "layer-list family: token-pair embedding: buckets and multipliers must be >= 0"; return GL3_E_ARG; }
@@ -177,6 +202,11 @@ int32_t gl3_hy_create(const gl3_model_desc* desc, gl3_ctx** out, std::string& er
             }
             if (const char* m = hy_check_layer(*ld.beside)) { err = "layer " + std::to_string(l) + ", second mixer: " + m; return GL3_E_ARG; }
         }
+        if (ld.out_norm || (ld.beside && ld.beside->out_norm)) {
+            if (!ld.beside || !ld.out_norm || !ld.beside->out_norm || desc->streams > 0 || desc->parallel_block) {
+                err = "layer " + std::to_string(l) + ": out_norm is for both of two mixers side by side, on the plain residual without parallel block"; return GL3_E_ARG;
+            }
+        }
     }
     gl3_ctx* ctx = new gl3_ctx();
     ctx->d = *desc;
@@ -193,6 +223,7 @@ int32_t gl3_hy_create(const gl3_model_desc* desc, gl3_ctx** out, std::string& er
     h->side_dim = desc->side_dim; h->side_ld = hy_cdiv(std::max(1, desc->side_dim), 8) * 8;
     h->depth = desc->depth_mix != 0;
     h->post_norms = desc->post_norms != 0;
+    h->no_pre = desc->no_pre_norms != 0;
     h->softcap = desc->logit_softcap;
     h->shift = desc->token_shift != 0; h->lscale = desc->layer_scale != 0;
     h->bg_buckets = desc->bigram_buckets; h->bg_prev = desc->bigram_mul_prev; h->bg_cur = desc->bigram_mul_cur;
@@ -223,6 +254,7 @@ int32_t gl3_hy_create(const gl3_model_desc* desc, gl3_ctx** out, std::string& er
         const gl3_layer_desc& d = Ly.d;
         Ly.o0 = o0;
         Ly.out_mul = d.out_scale != 0.f ? d.out_scale : 1.f;
+        slot = (slot + 63) & ~(size_t)63;
         max_heads = std::max(max_heads, d.heads);
 #define TRYM(x) do { int32_t r_ = (x); if (r_ != GL3_OK) return r_; } while (0)
         // rotary tables, made in double: entry i turns by pos * f, f = base^(-2 i / dims); q / k with the position scaling: divided by a number,
@@ -282,8 +314,14 @@ int32_t gl3_hy_create(const gl3_model_desc* desc, gl3_ctx** out, std::string& er
                 TRYM(hy_alloc(ctx, &Ly.kn, (size_t)d.dim * 4));
             }
             if (d.softmax_sink == 2) TRYM(hy_alloc(ctx, &Ly.sink, (size_t)d.heads * 4));
+            if (d.head_temp) TRYM(hy_alloc(ctx, &Ly.head_temp, (size_t)d.heads * 4));
+            if (d.head_mix) {
+                Ly.mix_ld = hy_cdiv(d.heads, 16) * 16;
+                TRYM(hy_alloc(ctx, &Ly.head_mixT, (size_t)Ly.mix_ld * Ly.mix_ld * 4));
+            }
             max_hdv = std::max(max_hdv, d.heads * d.vdim);
         } else if (d.mixer == GL3_MIX_LATENT) {
+            if (d.softmax_sink == 2) TRYM(hy_alloc(ctx, &Ly.sink, (size_t)d.heads * 4));
             const int De = Ly.De = d.dim + d.rot_dim, Re = Ly.Re = d.kv_rank + d.rot_dim;
             Ly.q_off = p0; Ly.c_off = Ly.q_off + (d.q_rank > 0 ? d.q_rank : d.heads * De); Ly.g_off = Ly.c_off + (d.kv_share > 0 ? 0 : Re);
             if (d.kv_share > 0) Ly.off_k = Ly.off_v = h->L[d.kv_share - 1].off_k;          // another layer's rows
@@ -325,16 +363,22 @@ int32_t gl3_hy_create(const gl3_model_desc* desc, gl3_ctx** out, std::string& er
             max_hdv = std::max(max_hdv, std::max(Re <= HY_LATENT_DIRECT ? d.heads * Re : 0, d.heads * d.vdim));
             max_kx = std::max(max_kx, d.heads * De); max_vx = std::max(max_vx, d.heads * d.vdim);
         } else if (d.mixer == GL3_MIX_MEMORY) {
-            const bool eg = d.mem_gates == GL3_MEM_EXP_GATES;
-            Ly.d.kv_heads = d.heads;
-            Ly.q_off = p0; Ly.k_off = Ly.q_off + d.heads * d.dim; Ly.v_off = Ly.k_off + d.heads * d.dim; Ly.g_off = Ly.v_off + d.heads * d.vdim;
+            const bool eg = d.mem_gates == GL3_MEM_EXP_GATES, delta = d.mem_gates == GL3_MEM_DELTA;
+            Ly.d.kv_heads = hy_mem_kvh(d);
+            Ly.q_off = p0; Ly.k_off = Ly.q_off + d.kv_heads * d.dim; Ly.v_off = Ly.k_off + d.kv_heads * d.dim; Ly.g_off = Ly.v_off + d.heads * d.vdim;
             Ly.i_off = Ly.g_off + hy_gate_rows(d); Ly.f_off = d.mem_gates == GL3_MEM_CHANNEL_GATES ? Ly.k_off : Ly.i_off + d.heads;          // channel gates stand in the keys' place
             if (d.rot_dims > 0) TRYM(table(&Ly.rot_freq, d.rot_dims, true));
             const int P = d.vdim + (eg ? 1 : 0);             // exponential gates: one more state column carries the normaliser
             Ly.off_state = slot; slot += (size_t)d.heads * d.dim * P;
             if (eg) { Ly.off_m = slot; slot += (size_t)d.heads; }
             else if (d.mem_gates == GL3_MEM_CHANNEL_GATES) TRYM(hy_alloc(ctx, &Ly.mem_lower, (size_t)d.heads * d.dim * 4));
-            else {
+            else if (delta) {
+                Ly.off_tail = slot; slot += (size_t)(d.mem_conv - 1) * hy_delta_ch(d);
+                TRYM(hy_alloc(ctx, &Ly.mem_conv_w, (size_t)d.mem_conv * hy_delta_ch(d) * 4));
+                TRYM(hy_alloc(ctx, &Ly.a_log, (size_t)d.heads * 4));
+                TRYM(hy_alloc(ctx, &Ly.dt_bias, (size_t)d.heads * 4));
+                max_ch = std::max(max_ch, hy_delta_ch(d));
+            } else {
                 TRYM(hy_alloc(ctx, &Ly.decay, (size_t)d.heads * 4));
                 if (hipMemcpy(Ly.decay, d.mem_decay, (size_t)d.heads * 4, hipMemcpyHostToDevice) != hipSuccess) { ctx->err = "copy of mem_decay failed"; return GL3_E_HIP; }
             }
@@ -352,6 +396,7 @@ int32_t gl3_hy_create(const gl3_model_desc* desc, gl3_ctx** out, std::string& er
             TRYM(hy_alloc(ctx, &Ly.ssm_norm, (size_t)inner * 4));
             max_ch = std::max(max_ch, ch); max_inner = std::max(max_inner, inner);
         }
+        if (d.out_norm) TRYM(hy_alloc(ctx, &Ly.branch_norm, (size_t)W * 4));
 #undef TRYM
         Ly.d.mem_decay = nullptr;          // the caller's array is not kept
         Ly.d.beside = nullptr;
@@ -367,13 +412,19 @@ int32_t gl3_hy_create(const gl3_model_desc* desc, gl3_ctx** out, std::string& er
             Ly.side->d.ff = 0; Ly.side->d.experts = 0; Ly.side->d.shared_ff = 0;
         }
         const int np1 = hy_proj_rows(d), mo1 = hy_mix_out(d);
-        const int np = np1 + (bd ? hy_proj_rows(*bd) : 0), mo = mo1 + (bd ? hy_mix_out(*bd) : 0);
+        // two normed mixers: an output projection each, the second mixer's columns start at a 16-byte boundary of mixo
+        const bool apart = bd && d.out_norm;
+        const int o2 = apart ? hy_cdiv(mo1, 8) * 8 : mo1;
+        const int np = np1 + (bd ? hy_proj_rows(*bd) : 0), mo = apart ? hy_cdiv(o2 + hy_mix_out(*bd), 8) * 8 : mo1 + (bd ? hy_mix_out(*bd) : 0);
         const bool bias = hy_has_bias(d) || (bd && hy_has_bias(*bd));
         Ly.mo_total = mo;
         TRY(hy_alloc_mat(ctx, Ly.proj, np, W, W));
-        TRY(hy_alloc_mat(ctx, Ly.o, W, mo, mo));
+        if (apart) {
+            TRY(hy_alloc_mat(ctx, Ly.o, W, mo1, mo1));
+            TRY(hy_alloc_mat(ctx, Ly.side->o, W, hy_mix_out(*bd), hy_mix_out(*bd)));
+        } else TRY(hy_alloc_mat(ctx, Ly.o, W, mo, mo));
         if (bias) TRY(hy_alloc(ctx, &Ly.pbias, (size_t)np * 4));
-        TRY(hy_alloc(ctx, &Ly.norm1, (size_t)W * 4));
+        if (!h->no_pre) TRY(hy_alloc(ctx, &Ly.norm1, (size_t)W * 4));
         for (int q = 0; q < (d.ff > 0 ? 2 : 1) && !h->plain; ++q) {
             TRY(hy_alloc(ctx, &Ly.hc[q][0], (size_t)S * 4));
             TRY(hy_alloc(ctx, &Ly.hc[q][1], (size_t)S * 4));
@@ -391,11 +442,11 @@ int32_t gl3_hy_create(const gl3_model_desc* desc, gl3_ctx** out, std::string& er
         TRY(setup_mixer(Ly, 0, 0));
         if (Ly.side) {
             Ly.side->pbias = Ly.pbias; Ly.side->mo_total = mo;
-            TRY(setup_mixer(*Ly.side, np1, mo1));
+            TRY(setup_mixer(*Ly.side, np1, o2));
         }
         Ly.dense_ff = d.experts > 0 ? d.shared_ff : d.ff;
         Ly.dense_limit = d.experts > 0 ? d.shared_limit : d.ff_limit;
-        if (d.ff > 0 && !h->parallel) TRY(hy_alloc(ctx, &Ly.norm2, (size_t)W * 4));
+        if (d.ff > 0 && !h->parallel && !h->no_pre) TRY(hy_alloc(ctx, &Ly.norm2, (size_t)W * 4));
         if (h->post_norms) {
             TRY(hy_alloc(ctx, &Ly.norm1b, (size_t)W * 4));
             if (d.ff > 0) TRY(hy_alloc(ctx, &Ly.norm2b, (size_t)W * 4));
@@ -409,8 +460,8 @@ int32_t gl3_hy_create(const gl3_model_desc* desc, gl3_ctx** out, std::string& er
         }
         if (d.experts > 0) {
             Ly.eff_pad = hy_cdiv(d.ff, 32) * 32;
-            TRY(hy_alloc_mat(ctx, Ly.router, d.experts + (d.shared_ff > 0 && !d.shared_ungated ? 1 : 0), W, W));
-            if (d.route_bias) TRY(hy_alloc(ctx, &Ly.route_bias, (size_t)d.experts * 4));
+            TRY(hy_alloc_mat(ctx, Ly.router, d.experts + d.identity + (d.shared_ff > 0 && !d.shared_ungated ? 1 : 0), W, W));
+            if (d.route_bias) TRY(hy_alloc(ctx, &Ly.route_bias, (size_t)(d.experts + d.identity) * 4));
             TRY(hy_alloc_mat(ctx, Ly.egu, d.experts * (hy_ungated(d) ? 1 : 2) * Ly.eff_pad, W, W));
             TRY(hy_alloc_mat(ctx, Ly.edown, d.experts * W, Ly.eff_pad, Ly.eff_pad));
             max_rz = std::max(max_rz, Ly.router.rows); max_top = std::max(max_top, d.top); max_eff = std::max(max_eff, Ly.eff_pad); max_e = std::max(max_e, d.experts);
@@ -495,6 +546,9 @@ int32_t gl3_hy_create(const gl3_model_desc* desc, gl3_ctx** out, std::string& er
         HY_LDS(1, 1); HY_LDS(1, 2); HY_LDS(1, 4); HY_LDS(1, 8); HY_LDS(2, 1); HY_LDS(2, 2); HY_LDS(2, 4); HY_LDS(2, 8);
         HY_LDS(4, 1); HY_LDS(4, 2); HY_LDS(4, 4); HY_LDS(4, 8); HY_LDS(8, 1); HY_LDS(8, 2); HY_LDS(8, 4);
 #undef HY_LDS
+#define HY_LDS(KB, UA) TRYHIP(hipFuncSetAttribute((const void*)hy_heads_attn_kernel<KB, UA>, hipFuncAttributeMaxDynamicSharedMemorySize, 150 * 1024))
+        HY_LDS(1, 1); HY_LDS(1, 2); HY_LDS(1, 4); HY_LDS(1, 8); HY_LDS(2, 1); HY_LDS(2, 2); HY_LDS(2, 4); HY_LDS(2, 8); HY_LDS(4, 1); HY_LDS(4, 2); HY_LDS(4, 4); HY_LDS(4, 8);
+#undef HY_LDS
     }
     TRYHIP(hipDeviceSynchronize());
 #undef TRY
@@ -516,8 +570,9 @@ void gl3_hy_destroy(gl3_ctx* ctx) {
             if (!M) continue;
             f(M->lat_norm); f(M->wk); f(M->wv); f(M->wvT); f(M->conv_w); f(M->conv_b); f(M->dt_bias); f(M->a_log); f(M->dskip); f(M->ssm_norm);
             f(M->rot_freq); f(M->vrot_freq); f(M->qn); f(M->kn); f(M->sink); f(M->decay); f(M->uq.w); f(M->qlat_norm); f(M->lat_freq);
-            f(M->rot_freq64); f(M->qk_conv_w); f(M->mem_lower);
+            f(M->rot_freq64); f(M->qk_conv_w); f(M->mem_lower); f(M->head_temp); f(M->head_mixT); f(M->mem_conv_w); f(M->branch_norm);
         }
+        if (L.side) f(L.side->o.w);
         delete L.side;
         L.side = nullptr;
         f(L.norm1b); f(L.norm2b); f(L.route_bias); f(L.shift_mu); f(L.ls1); f(L.ls2); f(L.poly);
@@ -611,47 +666,68 @@ int32_t gl3_hy_upload(gl3_ctx* ctx, int32_t id, int32_t layer, const void* host,
     HyLayer& L = beside ? *L0.side : L0;             // the mixer the tensor belongs to
     const gl3_layer_desc& d = L.d;
     const bool att = d.mixer == GL3_MIX_ATTENTION, lat = d.mixer == GL3_MIX_LATENT, ssm = d.mixer == GL3_MIX_SSM, mem = d.mixer == GL3_MIX_MEMORY;
-    const bool memg = mem && d.mem_gates == GL3_MEM_EXP_GATES, memc = mem && d.mem_gates == GL3_MEM_CHANNEL_GATES;
+    const bool memg = mem && d.mem_gates == GL3_MEM_EXP_GATES, memc = mem && d.mem_gates == GL3_MEM_CHANNEL_GATES, memd = mem && d.mem_gates == GL3_MEM_DELTA;
     const int mo = hy_mix_out(d);
     HyMat& proj = L0.proj;
     const size_t tes = type == GL3_TYPE_BF16 ? 2 : 4;          // bytes per element of the source
     std::vector<float> f;
     switch (id) {
-        case GL3_T_ATTN_NORM: if (!beside) r = hy_put_vec(ctx, L.norm1, W, host, bytes, type, h->norm_offset); break;
+        case GL3_T_ATTN_NORM: if (!beside && L.norm1) r = hy_put_vec(ctx, L.norm1, W, host, bytes, type, h->norm_offset); break;
         case GL3_T_FFN_NORM: if (d.ff > 0 && L.norm2) r = hy_put_vec(ctx, L.norm2, W, host, bytes, type, h->norm_offset); break;
         case GL3_T_ATTN_POST_NORM: if (!beside && L.norm1b) r = hy_put_vec(ctx, L.norm1b, W, host, bytes, type, h->norm_offset); break;
         case GL3_T_FFN_POST_NORM: if (!beside && L.norm2b) r = hy_put_vec(ctx, L.norm2b, W, host, bytes, type, h->norm_offset); break;
         case GL3_T_WQ:
             if (lat && d.q_rank > 0) r = hy_put_rows(ctx, L.uq, 0, d.heads * L.De, d.q_rank, host, bytes, type, 0);
             else if (lat) r = hy_put_rows(ctx, proj, L.q_off, d.heads * L.De, W, host, bytes, type, 0);
-            else if (att || mem) r = hy_put_rows(ctx, proj, L.q_off, d.heads * d.dim, W, host, bytes, type, 0);
+            else if (att || mem) r = hy_put_rows(ctx, proj, L.q_off, (mem ? d.kv_heads : d.heads) * d.dim, W, host, bytes, type, 0);
             break;
         case GL3_T_Q_DOWN: if (lat && d.q_rank > 0) r = hy_put_rows(ctx, proj, L.q_off, d.q_rank, W, host, bytes, type, 0); break;
         case GL3_T_Q_DOWN_NORM: if (lat && d.q_rank > 0) r = hy_put_vec(ctx, L.qlat_norm, d.q_rank, host, bytes, type); break;
-        case GL3_T_FFN_ROUTE_BIAS: if (d.experts > 0 && d.route_bias) r = hy_put_vec(ctx, L.route_bias, d.experts, host, bytes, type); break;
+        case GL3_T_FFN_ROUTE_BIAS: if (d.experts > 0 && d.route_bias) r = hy_put_vec(ctx, L.route_bias, d.experts + d.identity, host, bytes, type); break;
         case GL3_T_WK: if (att || (mem && !memc)) r = hy_put_rows(ctx, proj, L.k_off, d.kv_heads * d.dim, W, host, bytes, type, 0); break;
-        case GL3_T_WV: if ((att && !d.v_from_k) || mem) r = hy_put_rows(ctx, proj, L.v_off, d.kv_heads * d.vdim, W, host, bytes, type, 0); break;
+        case GL3_T_WV: if ((att && !d.v_from_k) || mem) r = hy_put_rows(ctx, proj, L.v_off, (mem ? d.heads : d.kv_heads) * d.vdim, W, host, bytes, type, 0); break;
         case GL3_T_ATTN_GATE: if (hy_gate_rows(d) > 0 && !ssm) r = hy_put_rows(ctx, proj, L.g_off, hy_gate_rows(d), W, host, bytes, type, 0); break;
-        case GL3_T_WO: r = hy_put_rows(ctx, L0.o, 0, W, mo, host, bytes, type, 0, L.o0); break;
+        case GL3_T_WO: r = d.out_norm ? hy_put_rows(ctx, L.o, 0, W, mo, host, bytes, type, 0) : hy_put_rows(ctx, L0.o, 0, W, mo, host, bytes, type, 0, L.o0); break;
+        case GL3_T_BRANCH_NORM:          // the mixer's multiplier rides on the weight
+            if (d.out_norm) {
+                if (!hy_to_f32(host, bytes, type, W, f)) GL3_FAIL(GL3_E_ARG, "tensor size or type mismatch");
+                for (float& v : f) v = (v + h->norm_offset) * L.out_mul;
+                HY_HIP(hipMemcpy(L.branch_norm, f.data(), (size_t)W * 4, hipMemcpyHostToDevice));
+                r = GL3_OK;
+            }
+            break;
+        case GL3_T_ATTN_TEMP: if (att && d.head_temp) r = hy_put_vec(ctx, L.head_temp, d.heads, host, bytes, type); break;
+        case GL3_T_HEAD_MIX:
+            if (att && d.head_mix) {          // [h][g] -> [g][h], zero padded
+                const int H = d.heads;
+                if (!hy_to_f32(host, bytes, type, (size_t)H * H, f)) GL3_FAIL(GL3_E_ARG, "tensor size or type mismatch");
+                std::vector<float> tr((size_t)L.mix_ld * L.mix_ld, 0.f);
+                for (int a = 0; a < H; ++a)
+                    for (int b = 0; b < H; ++b) tr[(size_t)b * L.mix_ld + a] = f[(size_t)a * H + b];
+                HY_HIP(hipMemcpy(L.head_mixT, tr.data(), tr.size() * 4, hipMemcpyHostToDevice));
+                r = GL3_OK;
+            }
+            break;
         case GL3_T_BQ: if (att && d.qk_bias) r = hy_put_vec(ctx, L.pbias + L.q_off, (size_t)d.heads * d.dim, host, bytes, type); break;
         case GL3_T_BK: if (att && d.qk_bias) r = hy_put_vec(ctx, L.pbias + L.k_off, (size_t)d.kv_heads * d.dim, host, bytes, type); break;
         case GL3_T_BV: if (att && d.qk_bias) r = hy_put_vec(ctx, L.pbias + L.v_off, (size_t)d.kv_heads * d.vdim, host, bytes, type); break;
         case GL3_T_ATTN_Q_NORM: if (att && d.qk_unit_norm >= 2) r = hy_put_vec(ctx, L.qn, (size_t)(d.qk_unit_norm == 3 ? 1 : d.heads) * d.dim, host, bytes, type); break;
         case GL3_T_ATTN_K_NORM: if (att && d.qk_unit_norm >= 2) r = hy_put_vec(ctx, L.kn, (size_t)(d.qk_unit_norm == 3 ? 1 : d.kv_heads) * d.dim, host, bytes, type); break;
-        case GL3_T_ATTN_SINK: if (att && d.softmax_sink == 2) r = hy_put_vec(ctx, L.sink, d.heads, host, bytes, type); break;
-        case GL3_T_MEM_IGATE: if (memg) r = hy_put_rows(ctx, proj, L.i_off, d.heads, W, host, bytes, type, 0); break;
-        case GL3_T_MEM_FGATE: if (memg || memc) r = hy_put_rows(ctx, proj, L.f_off, memc ? d.heads * d.dim : d.heads, W, host, bytes, type, 0); break;
+        case GL3_T_ATTN_SINK: if ((att || lat) && d.softmax_sink == 2) r = hy_put_vec(ctx, L.sink, d.heads, host, bytes, type); break;
+        case GL3_T_MEM_IGATE: if (memg || memd) r = hy_put_rows(ctx, proj, L.i_off, d.heads, W, host, bytes, type, 0); break;
+        case GL3_T_MEM_FGATE: if (memg || memc || memd) r = hy_put_rows(ctx, proj, L.f_off, memc ? d.heads * d.dim : d.heads, W, host, bytes, type, 0); break;
         case GL3_T_MEM_IGATE_BIAS: if (memg) r = hy_put_vec(ctx, L.pbias + L.i_off, d.heads, host, bytes, type); break;
         case GL3_T_MEM_FGATE_BIAS: if (memg || memc) r = hy_put_vec(ctx, L.pbias + L.f_off, memc ? (size_t)d.heads * d.dim : d.heads, host, bytes, type); break;
         case GL3_T_MEM_LOWER: if (memc) r = hy_put_vec(ctx, L.mem_lower, (size_t)d.heads * d.dim, host, bytes, type); break;
-        case GL3_T_Q_CONV: case GL3_T_K_CONV:
-            if (att && d.qk_conv > 0) {          // [channels][taps] -> columns of [taps][all channels]
-                const int taps = d.qk_conv, C = hy_qk_ch(d), c0 = id == GL3_T_Q_CONV ? 0 : d.heads * d.dim, nc = (id == GL3_T_Q_CONV ? d.heads : d.kv_heads) * d.dim;
+        case GL3_T_Q_CONV: case GL3_T_K_CONV: case GL3_T_V_CONV:
+            if ((att && d.qk_conv > 0 && id != GL3_T_V_CONV) || memd) {          // [channels][taps] -> columns of [taps][all channels]
+                const int taps = memd ? d.mem_conv : d.qk_conv, nq = (memd ? d.kv_heads : d.heads) * d.dim, nk = d.kv_heads * d.dim, C = memd ? hy_delta_ch(d) : hy_qk_ch(d);
+                const int c0 = id == GL3_T_Q_CONV ? 0 : id == GL3_T_K_CONV ? nq : nq + nk, nc = id == GL3_T_Q_CONV ? nq : id == GL3_T_K_CONV ? nk : d.heads * d.vdim;
                 if (!hy_to_f32(host, bytes, type, (size_t)nc * taps, f)) GL3_FAIL(GL3_E_ARG, "tensor size or type mismatch");
                 std::vector<float> tr((size_t)nc * taps);
                 for (int c = 0; c < nc; ++c)
                     for (int j = 0; j < taps; ++j) tr[(size_t)j * nc + c] = f[(size_t)c * taps + j];
-                HY_HIP(hipMemcpy2D(L.qk_conv_w + c0, (size_t)C * 4, tr.data(), (size_t)nc * 4, (size_t)nc * 4, taps, hipMemcpyHostToDevice));
+                HY_HIP(hipMemcpy2D((memd ? L.mem_conv_w : L.qk_conv_w) + c0, (size_t)C * 4, tr.data(), (size_t)nc * 4, (size_t)nc * 4, taps, hipMemcpyHostToDevice));
                 r = GL3_OK;
             }
             break;
@@ -695,8 +771,8 @@ int32_t gl3_hy_upload(gl3_ctx* ctx, int32_t id, int32_t layer, const void* host,
         case GL3_T_SSM_IN: if (ssm) r = hy_put_rows(ctx, proj, L.q_off, hy_proj_rows(d), W, host, bytes, type, 0); break;
         case GL3_T_SSM_CONV: if (ssm) r = hy_put_vec(ctx, L.conv_w, (size_t)hy_conv_ch(d) * d.conv, host, bytes, type); break;
         case GL3_T_SSM_CONV_BIAS: if (ssm) r = hy_put_vec(ctx, L.conv_b, hy_conv_ch(d), host, bytes, type); break;
-        case GL3_T_SSM_DT_BIAS: if (ssm) r = hy_put_vec(ctx, L.dt_bias, d.heads, host, bytes, type); break;
-        case GL3_T_SSM_A_LOG: if (ssm) r = hy_put_vec(ctx, L.a_log, d.heads, host, bytes, type); break;
+        case GL3_T_SSM_DT_BIAS: if (ssm || memd) r = hy_put_vec(ctx, L.dt_bias, d.heads, host, bytes, type); break;
+        case GL3_T_SSM_A_LOG: if (ssm || memd) r = hy_put_vec(ctx, L.a_log, d.heads, host, bytes, type); break;
         case GL3_T_SSM_D: if (ssm) r = hy_put_vec(ctx, L.dskip, d.heads, host, bytes, type); break;
         case GL3_T_SSM_NORM: if (ssm || (mem && d.mem_norm_weight)) r = hy_put_vec(ctx, L.ssm_norm, (mem && d.mem_norm_weight == 2) ? d.vdim : mo, host, bytes, type); break;
         case GL3_T_W1: if (L.dense_ff > 0 && !hy_ungated(d)) r = hy_put_rows(ctx, L.gu, 0, L.dense_ff, W, host, bytes, type, 1); break;
@@ -710,8 +786,8 @@ int32_t gl3_hy_upload(gl3_ctx* ctx, int32_t id, int32_t layer, const void* host,
             }
             break;
         // mixture of experts: router rows, then (one more row) the shared expert's gate; the experts' matrices arrive stacked [experts][..]
-        case GL3_T_FFN_GATE_INP: if (d.experts > 0) r = hy_put_rows(ctx, L.router, 0, d.experts, W, host, bytes, type, 0); break;
-        case GL3_T_FFN_GATE_INP_SHEXP: if (d.experts > 0 && d.shared_ff > 0 && !d.shared_ungated) r = hy_put_rows(ctx, L.router, d.experts, 1, W, host, bytes, type, 0); break;
+        case GL3_T_FFN_GATE_INP: if (d.experts > 0) r = hy_put_rows(ctx, L.router, 0, d.experts + d.identity, W, host, bytes, type, 0); break;
+        case GL3_T_FFN_GATE_INP_SHEXP: if (d.experts > 0 && d.shared_ff > 0 && !d.shared_ungated) r = hy_put_rows(ctx, L.router, d.experts + d.identity, 1, W, host, bytes, type, 0); break;
         case GL3_T_FFN_GATE_EXPS: case GL3_T_FFN_UP_EXPS:
             if (d.experts > 0 && !(hy_ungated(d) && id == GL3_T_FFN_GATE_EXPS)) {
                 const size_t per = (size_t)d.ff * W * tes;
@@ -756,7 +832,12 @@ static HyHave hy_needed(const gl3_hybrid_state* h, const gl3_layer_desc& d, bool
     if (d.mixer == GL3_MIX_ATTENTION && d.qk_conv > 0) m |= HY_BIT(GL3_T_Q_CONV) | HY_BIT(GL3_T_K_CONV);
     if (d.mixer == GL3_MIX_ATTENTION && d.qk_bias) m |= (HY_BIT(GL3_T_BQ)) | (HY_BIT(GL3_T_BK)) | (HY_BIT(GL3_T_BV));
     if (d.mixer == GL3_MIX_ATTENTION && d.qk_unit_norm >= 2) m |= (HY_BIT(GL3_T_ATTN_Q_NORM)) | (HY_BIT(GL3_T_ATTN_K_NORM));
-    if (d.mixer == GL3_MIX_ATTENTION && d.softmax_sink == 2) m |= HY_BIT(GL3_T_ATTN_SINK);
+    if ((d.mixer == GL3_MIX_ATTENTION || d.mixer == GL3_MIX_LATENT) && d.softmax_sink == 2) m |= HY_BIT(GL3_T_ATTN_SINK);
+    if (d.head_temp) m.set(GL3_T_ATTN_TEMP);
+    if (d.head_mix) m.set(GL3_T_HEAD_MIX);
+    if (d.out_norm) m.set(GL3_T_BRANCH_NORM);
+    if (d.mixer == GL3_MIX_MEMORY && d.mem_gates == GL3_MEM_DELTA)
+        m |= HY_BIT(GL3_T_MEM_IGATE) | HY_BIT(GL3_T_MEM_FGATE) | HY_BIT(GL3_T_SSM_A_LOG) | HY_BIT(GL3_T_SSM_DT_BIAS) | HY_BIT(GL3_T_Q_CONV) | HY_BIT(GL3_T_K_CONV) | HY_BIT(GL3_T_V_CONV);
     if (d.mixer == GL3_MIX_MEMORY) m |= HY_BIT(GL3_T_WQ) | HY_BIT(GL3_T_WV);
     if (d.mixer == GL3_MIX_MEMORY && d.mem_gate_act != 2) m.set(GL3_T_ATTN_GATE);
     if (d.mixer == GL3_MIX_MEMORY && d.mem_gates != GL3_MEM_CHANNEL_GATES) m.set(GL3_T_WK);
@@ -765,7 +846,7 @@ static HyHave hy_needed(const gl3_hybrid_state* h, const gl3_layer_desc& d, bool
     if (d.mixer == GL3_MIX_MEMORY && d.mem_gates == GL3_MEM_EXP_GATES)
         m |= (HY_BIT(GL3_T_MEM_IGATE)) | (HY_BIT(GL3_T_MEM_FGATE)) | (HY_BIT(GL3_T_MEM_IGATE_BIAS)) | (HY_BIT(GL3_T_MEM_FGATE_BIAS));
     if (second) return m;
-    m |= HY_BIT(GL3_T_ATTN_NORM);
+    if (!h->no_pre) m |= HY_BIT(GL3_T_ATTN_NORM);
     if (!h->plain) m |= (HY_BIT(GL3_T_HC1_IN)) | (HY_BIT(GL3_T_HC1_OUT)) | (HY_BIT(GL3_T_HC1_MIX));
     if (h->depth) m |= HY_BIT(GL3_T_DEPTH_MIX);
     if (h->side_dim > 0) m |= (HY_BIT(GL3_T_SIDE_GATE)) | (HY_BIT(GL3_T_SIDE_PROJ)) | (HY_BIT(GL3_T_SIDE_NORM));
@@ -778,7 +859,7 @@ static HyHave hy_needed(const gl3_hybrid_state* h, const gl3_layer_desc& d, bool
     if (d.mixer == GL3_MIX_SSM)
         m |= (HY_BIT(GL3_T_SSM_IN)) | (HY_BIT(GL3_T_SSM_CONV)) | (HY_BIT(GL3_T_SSM_CONV_BIAS)) | (HY_BIT(GL3_T_SSM_DT_BIAS)) | (HY_BIT(GL3_T_SSM_A_LOG)) |
              (HY_BIT(GL3_T_SSM_D)) | (HY_BIT(GL3_T_SSM_NORM));
-    if (d.ff > 0 && !h->parallel) m |= HY_BIT(GL3_T_FFN_NORM);
+    if (d.ff > 0 && !h->parallel && !h->no_pre) m |= HY_BIT(GL3_T_FFN_NORM);
     if (h->shift) m.set(GL3_T_TOKEN_SHIFT);
     if (h->lscale) { m.set(GL3_T_ATTN_SCALE); if (d.ff > 0) m.set(GL3_T_FFN_SCALE); }
     if (d.ff > 0 && d.ff_act == 3) m.set(GL3_T_FFN_POLY);
@@ -926,6 +1007,63 @@ static int32_t hy_attention(gl3_ctx* ctx, const float* q, int ldq, const float* 
     return GL3_OK;
 }
 
+// Attention over all heads at once (hy_heads_attn_kernel): temperatures, capped and mixed scores, chunks.
+static int32_t hy_attention_heads(gl3_ctx* ctx, const HyLayer& L, const float* q, int ldq, const float* kc, const float* vc, int n, int pos0, int* nsplit_out) {
+    gl3_hybrid_state* h = ctx->hy;
+    const gl3_layer_desc& d = L.d;
+    const int H = d.heads, G = d.kv_heads, hpg = H / G;
+    // tokens per workgroup: enough for the rows of a key / value head to fill 16; 64 keys per tile for longer portions, 16 for a few tokens (more
+    // tiles to split over); both shrink until the scores fit two workgroups into a CU's LDS
+    int QT = 1, KB = n > 16 ? 4 : 1;
+    while (QT < n && QT * hpg < 16) QT *= 2;
+    HyHeadsArgs a;
+    auto lds = [&]() {
+        a.ts = 16 * KB + 4;
+        a.ss = QT * a.ts;
+        a.ss += (16 - a.ss % 64 + 64) % 64;          // a head's row starts 16 banks after the one before it
+        return ((size_t)H * a.ss + 3 * (size_t)H * QT) * 4;
+    };
+    while (lds() > 76 * 1024 && (KB > 1 || QT > 1)) { if (KB > 1) KB /= 2; else QT /= 2; }
+    if (lds() > 150 * 1024) GL3_FAIL(GL3_E_UNSUPPORTED, "attention: too many heads for the LDS tile");
+    const int KT = 16 * KB, RB = hy_cdiv(QT * hpg, 16), units = G * RB * hy_cdiv(d.vdim, 64), ny = hy_cdiv(units, 32), nx = hy_cdiv(n, QT);
+    a.ug = hy_cdiv(units, ny);
+    const int per = hy_cdiv(a.ug, 4), UA = per <= 1 ? 1 : per <= 2 ? 2 : per <= 4 ? 4 : 8;
+    a.ug = 4 * UA < a.ug ? 4 * UA : a.ug;
+    // key splits: one tile each for a few tokens; else as many as fill the chip twice
+    const long span = d.chunk > 0 ? std::min<long>(pos0 + n, (long)d.chunk + QT - 1) : pos0 + n;          // keys a workgroup walks at most
+    int nsplit = (int)std::min<long>(128, span / KT + 1 + (d.chunk > 0 ? 1 : 0));
+    if (n > 16) nsplit = std::min(nsplit, std::max(1, 512 / std::max(1, nx * ny)));
+    if ((size_t)n * nsplit > h->part_rows) nsplit = (int)std::max<size_t>(1, h->part_rows / n);
+    a.q = q; a.ldq = ldq; a.kc = kc; a.vc = vc; a.slot_stride = h->slot_floats; a.H = H; a.G = G; a.dk = d.dim; a.dv = d.vdim; a.scale = d.scale; a.cap = d.score_softcap;
+    a.temp = d.head_temp ? L.head_temp : nullptr; a.mixT = d.head_mix ? L.head_mixT : nullptr; a.mix_ld = L.mix_ld; a.chunk = d.chunk;
+    a.dyn = h->dyn; a.n = n; a.nsplit = nsplit; a.part_acc = h->part_acc; a.part_ml = h->part_ml; a.QT = QT;
+    const size_t smem = lds();
+    const dim3 grid(nx, ny, nsplit);
+#define HY_HA(KBT, UAT) hipLaunchKernelGGL((hy_heads_attn_kernel<KBT, UAT>), grid, dim3(256), smem, ctx->stream, a)
+#define HY_HA_U(KBT) do { if (UA == 1) HY_HA(KBT, 1); else if (UA == 2) HY_HA(KBT, 2); else if (UA == 4) HY_HA(KBT, 4); else HY_HA(KBT, 8); } while (0)
+    if (KB == 4) HY_HA_U(4); else if (KB == 2) HY_HA_U(2); else HY_HA_U(1);
+#undef HY_HA_U
+#undef HY_HA
+    *nsplit_out = nsplit;
+    return GL3_OK;
+}
+
+// The gated delta rule's recurrence: a column's states over NG lanes x NL registers (NG NL >= dim); tokens staged per round: what fits 48 KB of
+// LDS, at most 32.
+static void hy_delta_scan(gl3_ctx* ctx, HyDeltaScan& a) {
+#define HY_DS(NL, NG)                                                                                                                                    \
+    do {                                                                                                                                                 \
+        constexpr int cols = 4 * (64 / NG), Ns = NL * NG;                                                                                                  \
+        const size_t per = 2 * (size_t)Ns + cols + 2;                                                                                                      \
+        a.TB = (int)std::max<size_t>(1, std::min<size_t>(32, (48 * 1024 / 4 - per) / (per + 256)));                                                        \
+        const size_t smem = ((a.TB + 1) * per + (size_t)a.TB * 256) * 4;                                                                                   \
+        hipLaunchKernelGGL((hy_delta_scan_kernel<NL, NG>), dim3(hy_cdiv(a.P, cols), a.heads), dim3(256), smem, ctx->stream, a);                            \
+    } while (0)
+    if (a.N <= 16) HY_DS(4, 4); else if (a.N <= 32) HY_DS(4, 8); else if (a.N <= 64) HY_DS(8, 8); else if (a.N <= 128) HY_DS(8, 16);
+    else if (a.N <= 256) HY_DS(16, 16); else if (a.N <= 512) HY_DS(32, 16); else HY_DS(32, 32);
+#undef HY_DS
+}
+
 // The recurrence kernel: a column's states over NG lanes x NL registers: NL = 16 (32 for more than 1024 states, 8 / 4 for very small
 // ones), NG a power of two; tokens staged per round: what fits 48 KB of LDS, at most 32.  Fills in a.NG and a.TB.
 // With few workgroups (few heads, narrow values) NL = 16 is halved once so that more of them share the columns; below 8 every workgroup
@@ -952,6 +1090,27 @@ static void hy_scan(gl3_ctx* ctx, HyScanArgs& a) {
     } while (0)
     if (NL == 4) HY_SCAN(4); else if (NL == 8) HY_SCAN(8); else if (NL == 16) HY_SCAN(16); else HY_SCAN(32);
 #undef HY_SCAN
+}
+
+// What leaves a matrix memory: h->ssm_y (row stride ldy, P columns per head) normed, gated and written to the operand of the output projection.
+template <typename T>
+static void hy_mem_out(gl3_ctx* ctx, const HyLayer& L, int n, int ldy, int P, const float* ge, int np, T* mixo, int ldo) {
+    gl3_hybrid_state* h = ctx->hy;
+    const gl3_layer_desc& d = L.d;
+    const float* gate = d.mem_gate_act == 2 ? nullptr : h->proj;
+    const float* w = d.mem_norm_weight ? L.ssm_norm : nullptr;
+    const float mul = d.out_norm ? 1.f : L.out_mul;
+    const int w_stride = d.mem_norm_weight == 2 ? 0 : d.vdim;
+    // one norm over the heads side by side: the kernel's "head" is the token's whole row
+    const bool whole = d.mem_norm_whole && !ge;
+    const int heads = whole ? 1 : d.heads, V = whole ? ldy : d.vdim;
+    if (whole) P = ldy;
+#define HY_MO(NT) hipLaunchKernelGGL((hy_mem_out_kernel<T, NT>), dim3(n, heads), dim3(NT), 0, ctx->stream, h->ssm_y, ldy, P, V, ge, heads, w, gate, np, L.g_off, d.mem_gate_act, ctx->d.rms_eps, mul, mixo, ldo, w_stride)
+    // a whole row is heads x vdim wide: 1024 threads for a few tokens, 256 for many; a head: 256 / 64
+    if (whole ? (n <= 32 && V > 512) : false) HY_MO(1024);
+    else if (whole ? V > 128 : (n <= 32 && V > 128)) HY_MO(256);
+    else HY_MO(64);
+#undef HY_MO
 }
 
 // One mixer of a layer on the n rows of the fused projection in h->proj (row stride np): its heads land in mixo (row stride ldo) from
@@ -992,12 +1151,30 @@ static int32_t hy_mixer_core(gl3_ctx* ctx, HyLayer& L, int np, int ldo, int n, i
                 hipLaunchKernelGGL(hy_pool_kernel, dim3(done, 2, done <= 8 ? std::min(16, hy_cdiv(d.kv_heads * std::max(d.dim, d.vdim), 256)) : 1), dim3(256), 0, st, kc, vc, pk, pv,
                                    d.kv_heads * d.dim, d.kv_heads * d.vdim, d.pool, h->slot_floats, h->dyn, n);
         }
-        int32_t r = hy_attention(ctx, q, ldq, kc, vc, d.heads, d.kv_heads, d.dim, d.vdim, d.scale, d.slope_log2, n, pos0, &nsplit, true, d.window, d.keep_first,
-                                 pk, pv, d.pool);
+        int32_t r = hy_by_heads(d) ? hy_attention_heads(ctx, L, q, ldq, kc, vc, n, pos0, &nsplit)
+                                   : hy_attention(ctx, q, ldq, kc, vc, d.heads, d.kv_heads, d.dim, d.vdim, d.scale, d.slope_log2, n, pos0, &nsplit, true, d.window, d.keep_first,
+                                                  pk, pv, d.pool);
         if (r != GL3_OK) return r;
         hipLaunchKernelGGL((hy_attn_merge_kernel<T>), dim3(n, d.heads), dim3(64), 0, st, h->part_acc, h->part_ml, d.heads, d.vdim, nsplit, d.softmax_sink,
                            d.out_gate ? h->proj + L.g_off : nullptr, np, d.out_gate, mixo, ldo, d.v_rot ? L.vrot_freq : nullptr, h->dyn,
-                           d.softmax_sink == 2 ? L.sink : nullptr, L.out_mul);
+                           d.softmax_sink == 2 ? L.sink : nullptr, d.out_norm ? 1.f : L.out_mul);
+    } else if (d.mixer == GL3_MIX_MEMORY && d.mem_gates == GL3_MEM_DELTA) {
+        const int ch = hy_delta_ch(d), inner = d.heads * d.vdim, nk = d.kv_heads * d.dim;
+        float *ga = h->gates, *gb = ga + (size_t)h->mb * h->max_heads;
+        HyDeltaPrep x;
+        x.proj = h->proj; x.ld = np; x.c0 = L.q_off; x.G = d.kv_heads; x.H = d.heads; x.D = d.dim; x.V = d.vdim;
+        x.conv_w = L.mem_conv_w; x.taps = d.mem_conv; x.tail = h->slots + L.off_tail; x.slot_stride = h->slot_floats; x.dyn = h->dyn; x.n = n;
+        x.act = d.mem_qkv_act; x.unit = d.mem_qk_unit; x.q_mul = d.mem_q_mul != 0.f ? d.mem_q_mul : 1.f; x.k_mul = d.mem_k_mul != 0.f ? d.mem_k_mul : 1.f;
+        x.out = h->conv; x.a_off = L.f_off; x.b_off = L.i_off; x.A_log = L.a_log; x.dt_bias = L.dt_bias; x.ga = ga; x.gb = gb;
+        hipLaunchKernelGGL(hy_delta_prep_kernel, dim3(n, 2 * d.kv_heads + d.heads + 1), dim3(64), 0, st, x);
+        if (d.mem_conv > 1 && n > 1)
+            hipLaunchKernelGGL(hy_conv_tail_kernel, dim3(hy_cdiv(ch, 256)), dim3(256), 0, st, h->proj, np, L.q_off, ch, d.mem_conv, h->slots + L.off_tail, h->slot_floats, h->dyn, n);
+        HyDeltaScan a;
+        a.src = h->conv; a.ld = ch; a.k_off = nk; a.v_off = 2 * nk; a.ga = ga; a.gb = gb;
+        a.heads = d.heads; a.G = d.kv_heads; a.P = d.vdim; a.N = d.dim;
+        a.state = h->slots + L.off_state; a.slot_stride = h->slot_floats; a.dyn = h->dyn; a.n = n; a.y = h->ssm_y; a.ldy = inner;
+        hy_delta_scan(ctx, a);
+        hy_mem_out<T>(ctx, L, n, inner, d.vdim, nullptr, np, mixo, ldo);
     } else if (d.mixer == GL3_MIX_MEMORY) {
         const bool eg = d.mem_gates == GL3_MEM_EXP_GATES, cg = d.mem_gates == GL3_MEM_CHANNEL_GATES;
         const int P = d.vdim + (eg ? 1 : 0), ldy = d.heads * P;
@@ -1021,25 +1198,7 @@ static int32_t hy_mixer_core(gl3_ctx* ctx, HyLayer& L, int np, int ldo, int n, i
             a.act &= ~2; a.fbias = nullptr;
         }
         hy_scan(ctx, a);
-        const float* gate = d.mem_gate_act == 2 ? nullptr : h->proj;
-        const int w_stride = d.mem_norm_weight == 2 ? 0 : d.vdim;
-        if (d.mem_norm_whole && !eg) {          // one norm over the heads side by side: the kernel's "head" is the token's whole row
-            // (a row is heads x vdim wide: 1024 threads for a few tokens, 256 for many)
-            if (n <= 32 && ldy > 512)
-                hipLaunchKernelGGL((hy_mem_out_kernel<T, 1024>), dim3(n, 1), dim3(1024), 0, st, h->ssm_y, ldy, ldy, ldy, (const float*)nullptr, 1,
-                                   d.mem_norm_weight ? L.ssm_norm : nullptr, gate, np, L.g_off, d.mem_gate_act, eps, L.out_mul, mixo, ldo, w_stride);
-            else if (ldy > 128)
-                hipLaunchKernelGGL((hy_mem_out_kernel<T, 256>), dim3(n, 1), dim3(256), 0, st, h->ssm_y, ldy, ldy, ldy, (const float*)nullptr, 1,
-                                   d.mem_norm_weight ? L.ssm_norm : nullptr, gate, np, L.g_off, d.mem_gate_act, eps, L.out_mul, mixo, ldo, w_stride);
-            else
-                hipLaunchKernelGGL((hy_mem_out_kernel<T, 64>), dim3(n, 1), dim3(64), 0, st, h->ssm_y, ldy, ldy, ldy, (const float*)nullptr, 1,
-                                   d.mem_norm_weight ? L.ssm_norm : nullptr, gate, np, L.g_off, d.mem_gate_act, eps, L.out_mul, mixo, ldo, w_stride);
-        } else if (n <= 32 && d.vdim > 128)
-            hipLaunchKernelGGL((hy_mem_out_kernel<T, 256>), dim3(n, d.heads), dim3(256), 0, st, h->ssm_y, ldy, P, d.vdim, eg ? ge : nullptr, d.heads,
-                               d.mem_norm_weight ? L.ssm_norm : nullptr, gate, np, L.g_off, d.mem_gate_act, eps, L.out_mul, mixo, ldo, w_stride);
-        else
-            hipLaunchKernelGGL((hy_mem_out_kernel<T, 64>), dim3(n, d.heads), dim3(64), 0, st, h->ssm_y, ldy, P, d.vdim, eg ? ge : nullptr, d.heads,
-                               d.mem_norm_weight ? L.ssm_norm : nullptr, gate, np, L.g_off, d.mem_gate_act, eps, L.out_mul, mixo, ldo, w_stride);
+        hy_mem_out<T>(ctx, L, n, ldy, P, eg ? ge : nullptr, np, mixo, ldo);
     } else if (d.mixer == GL3_MIX_LATENT) {
         // De entries per query / key head, Re per cached row (= dim, kv_rank without a rotated part)
         float* cc = h->slots + L.off_k;
@@ -1070,7 +1229,7 @@ static int32_t hy_mixer_core(gl3_ctx* ctx, HyLayer& L, int np, int ldo, int n, i
             int32_t r = hy_attention(ctx, q, ldq, h->kx, h->vx, d.heads, d.heads, De, d.vdim, d.scale, 0.f, n, pos0, &nsplit, false);
             if (r != GL3_OK) return r;
             hipLaunchKernelGGL((hy_attn_merge_kernel<T>), dim3(n, d.heads), dim3(64), 0, st, h->part_acc, h->part_ml, d.heads, d.vdim, nsplit, d.softmax_sink,
-                               d.out_gate ? h->proj + L.g_off : nullptr, np, d.out_gate == 2 ? 2 : 1, mixo, ldo, (const float*)nullptr, h->dyn);
+                               d.out_gate ? h->proj + L.g_off : nullptr, np, d.out_gate == 2 ? 2 : 1, mixo, ldo, (const float*)nullptr, h->dyn, L.sink);
         } else {
             // A few tokens (decode): the query is carried into the latent's space and the attention core reads the latents themselves
             // (one shared key / value head, keys = values), then the weighted sum of latents is expanded.
@@ -1083,7 +1242,7 @@ static int32_t hy_mixer_core(gl3_ctx* ctx, HyLayer& L, int np, int ldo, int n, i
             int32_t r = hy_attention(ctx, h->qa, d.heads * R, cc, cc, d.heads, 1, R, R, d.scale, 0.f, n, pos0, &nsplit);
             if (r != GL3_OK) return r;
             hipLaunchKernelGGL((hy_attn_merge_kernel<float>), dim3(n, d.heads), dim3(64), 0, st, h->part_acc, h->part_ml, d.heads, R, nsplit, d.softmax_sink,
-                               (const float*)nullptr, 0, 0, h->oc, d.heads * R, (const float*)nullptr, h->dyn);
+                               (const float*)nullptr, 0, 0, h->oc, d.heads * R, (const float*)nullptr, h->dyn, L.sink);
             if (n == 1)
                 hipLaunchKernelGGL((hy_headmm_kernel<T, 1>), dim3(1, d.heads, hy_cdiv(d.vdim, 64)), dim3(256), 0, st, h->oc, d.heads * R, R, d.vdim, L.wvT,
                                    d.out_gate ? h->proj + L.g_off : nullptr, np, mixo, ldo, n, d.out_gate == 2 ? 2 : 1);
@@ -1133,7 +1292,13 @@ static int32_t hy_mixer(gl3_ctx* ctx, HyLayer& L, int n, int pos0, int seq) {
     int32_t r = hy_mixer_core<T>(ctx, L, np, L.mo_total, n, pos0, seq);
     if (r == GL3_OK && L.side) r = hy_mixer_core<T>(ctx, *L.side, np, L.mo_total, n, pos0, seq);
     if (r != GL3_OK) return r;
-    hy_gemm<T>(ctx, (T*)h->mixo, L.o.k, L.o, n, h->y, h->W, false, nullptr, 0, HyGlu{}, &h->y_parts);
+    hy_gemm<T>(ctx, (T*)h->mixo, L.mo_total, L.o, n, h->y, h->W, false, nullptr, 0, HyGlu{}, &h->y_parts);
+    h->y_first = h->y_parts;
+    if (L.d.out_norm) {          // two normed mixers: the second one's product behind the first one's parts
+        int p2 = 1;
+        hy_gemm<T>(ctx, (T*)h->mixo + L.side->o0, L.mo_total, L.side->o, n, h->y + (size_t)h->y_parts * n * h->W, h->W, false, nullptr, 0, HyGlu{}, &p2);
+        h->y_parts += p2;
+    }
     return GL3_OK;
 }
 
@@ -1160,7 +1325,7 @@ static void hy_ff_up(gl3_ctx* ctx, const T* hb, HyLayer& L, int n, T* act) {
 // expert read from h->sel; else the pairs ordered by expert (h->tiles) and one MFMA tile per HY_MOE_BM rows of an expert.
 template <typename T>
 static void hy_gemm_grouped(gl3_ctx* ctx, const T* A, int lda, const HyMat& w, size_t wstride, int P, int max_tiles, bool few, float* C, int ldc, bool glu, T* act, int ld_act, HyGlu gp,
-                            int a_div = 1, const float* row_scale = nullptr) {
+                            int n_sel, int a_div = 1, const float* row_scale = nullptr) {
     gl3_hybrid_state* h = ctx->hy;
     const T* Wt = (const T*)w.w;
     const int N = w.rows, K = w.k;
@@ -1171,9 +1336,9 @@ static void hy_gemm_grouped(gl3_ctx* ctx, const T* A, int lda, const HyMat& w, s
         const dim3 grid(ksplit ? pairs : hy_cdiv(pairs, 4), P);
 #define HY_GMV(KS)                                                                                                                                     \
     do {                                                                                                                                              \
-        if (glu) hipLaunchKernelGGL((hy_matvec_kernel<T, T, 1, HY_EPI_GLU, KS, 1>), grid, dim3(256), 0, st, A, lda, Wt, w.ld, 1, N, K, C, ldc, act, ld_act, gp, h->sel, wstride, a_div, row_scale);   \
-        else if (gp.act == 2) hipLaunchKernelGGL((hy_matvec_kernel<T, T, 1, HY_EPI_ACTMUL, KS, 1>), grid, dim3(256), 0, st, A, lda, Wt, w.ld, 1, N, K, C, ldc, act, ld_act, gp, h->sel, wstride, a_div, row_scale);    \
-        else hipLaunchKernelGGL((hy_matvec_kernel<T, T, 1, HY_EPI_STORE, KS, 1>), grid, dim3(256), 0, st, A, lda, Wt, w.ld, 1, N, K, C, ldc, act, ld_act, gp, h->sel, wstride, a_div, row_scale);    \
+        if (glu) hipLaunchKernelGGL((hy_matvec_kernel<T, T, 1, HY_EPI_GLU, KS, 1>), grid, dim3(256), 0, st, A, lda, Wt, w.ld, 1, N, K, C, ldc, act, ld_act, gp, h->sel, wstride, a_div, row_scale, n_sel);   \
+        else if (gp.act == 2) hipLaunchKernelGGL((hy_matvec_kernel<T, T, 1, HY_EPI_ACTMUL, KS, 1>), grid, dim3(256), 0, st, A, lda, Wt, w.ld, 1, N, K, C, ldc, act, ld_act, gp, h->sel, wstride, a_div, row_scale, n_sel);    \
+        else hipLaunchKernelGGL((hy_matvec_kernel<T, T, 1, HY_EPI_STORE, KS, 1>), grid, dim3(256), 0, st, A, lda, Wt, w.ld, 1, N, K, C, ldc, act, ld_act, gp, h->sel, wstride, a_div, row_scale, n_sel);    \
     } while (0)
         if (ksplit) HY_GMV(4); else HY_GMV(1);
 #undef HY_GMV
@@ -1193,15 +1358,15 @@ static void hy_moe(gl3_ctx* ctx, HyLayer& L, int n) {
     gl3_hybrid_state* h = ctx->hy;
     const gl3_layer_desc& d = L.d;
     hipStream_t st = ctx->stream;
-    const int W = h->W, E = d.experts, top = d.top, P = n * top, RZ = L.router.rows;
+    const int W = h->W, E = d.experts, top = d.top, P = n * top, RZ = L.router.rows;          // (choices >= E: identity, without products)
     T* hb = (T*)h->h;
     int zparts = 1;          // few result rows and a long K: the router's product comes in K-split parts that the route kernel adds
     hy_gemm<T>(ctx, hb, W, L.router, n, h->moe_z, RZ, false, nullptr, 0, HyGlu{}, &zparts, HY_ZSPLIT);
     const bool few = n <= 8;
     const int max_tiles = P / HY_MOE_BM + std::min(E, P);
     const bool on_out = d.route_on_output != 0;          // the weights multiply the experts' outputs (in the residual update) instead of their inputs
-    hipLaunchKernelGGL(hy_route_kernel, dim3(n), dim3(64), 0, st, h->moe_z, RZ, zparts, (size_t)n * RZ, E, top, h->sel, h->wsel, few ? h->pair_row : nullptr,
-                       (d.shared_ff > 0 && !d.shared_ungated) ? h->sgz : nullptr, HyRoute{d.route_softmax, L.route_bias, d.route_renorm, d.route_scale != 0.f ? d.route_scale : 1.f, d.route_groups, d.route_keep});
+    hipLaunchKernelGGL(hy_route_kernel, dim3(n), dim3(64), 0, st, h->moe_z, RZ, zparts, (size_t)n * RZ, E + d.identity, top, h->sel, h->wsel, few ? h->pair_row : nullptr,
+                       (d.shared_ff > 0 && !d.shared_ungated) ? h->sgz : nullptr, HyRoute{d.route_softmax, L.route_bias, d.route_renorm, d.route_scale != 0.f ? d.route_scale : 1.f, d.route_groups, d.route_keep, E, d.route_group_max});
     HyMat one_gu = L.egu, one_down = L.edown;
     const bool glu = !hy_ungated(d);
     one_gu.rows = (glu ? 2 : 1) * L.eff_pad; one_down.rows = W;
@@ -1209,14 +1374,14 @@ static void hy_moe(gl3_ctx* ctx, HyLayer& L, int n) {
     if (few) {
         // a few tokens: the pairs of a token read its normed row themselves and the score multiplies the products (W (s h) = s (W h))
         hy_gemm_grouped<T>(ctx, hb, W, one_gu, gu_stride, P, max_tiles, true, nullptr, 0, glu, (T*)h->eact, L.eff_pad,
-                           HyGlu{d.ff_limit, d.ff_alpha, d.ff_shift, nullptr, nullptr, 0, 0, d.ff_act}, top, on_out ? nullptr : h->wsel);
+                           HyGlu{d.ff_limit, d.ff_alpha, d.ff_shift, nullptr, nullptr, 0, 0, d.ff_act}, E, top, on_out ? nullptr : h->wsel);
     } else {
         hipLaunchKernelGGL(hy_moe_group_kernel, dim3(1), dim3(256), (size_t)2 * E * 4, st, h->sel, P, E, HY_MOE_BM, h->pair_row, h->tiles, h->ntiles);
         hipLaunchKernelGGL((hy_moe_scale_kernel<T>), dim3(P), dim3(256), 0, st, hb, W, top, on_out ? (const float*)nullptr : h->wsel, h->pair_row, (T*)h->ea);
         hy_gemm_grouped<T>(ctx, (const T*)h->ea, W, one_gu, gu_stride, P, max_tiles, false, nullptr, 0, glu, (T*)h->eact, L.eff_pad,
-                           HyGlu{d.ff_limit, d.ff_alpha, d.ff_shift, nullptr, nullptr, 0, 0, d.ff_act});
+                           HyGlu{d.ff_limit, d.ff_alpha, d.ff_shift, nullptr, nullptr, 0, 0, d.ff_act}, E);
     }
-    hy_gemm_grouped<T>(ctx, (const T*)h->eact, L.eff_pad, one_down, (size_t)W * L.edown.ld, P, max_tiles, few, h->eout, W, false, nullptr, 0, HyGlu{});
+    hy_gemm_grouped<T>(ctx, (const T*)h->eact, L.eff_pad, one_down, (size_t)W * L.edown.ld, P, max_tiles, few, h->eout, W, false, nullptr, 0, HyGlu{}, E);
     if (d.shared_ff > 0) {
         T* act = (T*)h->mixo;
         hy_ff_up<T>(ctx, hb, L, n, act);
@@ -1241,13 +1406,14 @@ static void hy_logits(gl3_ctx* ctx, int nw) {
 template <typename T>
 static void hy_resid(gl3_ctx* ctx, int n, const HyResid& r, T* xt, T* h_out) {
     const bool v4 = r.W % 4 == 0;
-    if (n <= 32) {
-        if (v4) hipLaunchKernelGGL((hy_resid_kernel<T, 1024, 4>), dim3(n), dim3(1024), 0, ctx->stream, r, xt, h_out);
-        else hipLaunchKernelGGL((hy_resid_kernel<T, 1024, 1>), dim3(n), dim3(1024), 0, ctx->stream, r, xt, h_out);
-    } else {
-        if (v4) hipLaunchKernelGGL((hy_resid_kernel<T, 256, 4>), dim3(n), dim3(256), 0, ctx->stream, r, xt, h_out);
-        else hipLaunchKernelGGL((hy_resid_kernel<T, 256, 1>), dim3(n), dim3(256), 0, ctx->stream, r, xt, h_out);
-    }
+#define HY_RS(NT, V)                                                                                                                   \
+    do {                                                                                                                               \
+        if (r.bw1) hipLaunchKernelGGL((hy_resid_kernel<T, NT, V, true>), dim3(n), dim3(NT), 0, ctx->stream, r, xt, h_out);               \
+        else hipLaunchKernelGGL((hy_resid_kernel<T, NT, V, false>), dim3(n), dim3(NT), 0, ctx->stream, r, xt, h_out);                    \
+    } while (0)
+    if (n <= 32) { if (v4) HY_RS(1024, 4); else HY_RS(1024, 1); }
+    else { if (v4) HY_RS(256, 4); else HY_RS(256, 1); }
+#undef HY_RS
 }
 
 // One portion of a plain-residual design: x <- x + mixer(norm1 x); x <- x + ff(norm2 x); x <- x + side input; what goes on is the depth
@@ -1272,11 +1438,11 @@ static int32_t hy_portion_plain(gl3_ctx* ctx, int seq, const int32_t* tokens, in
     auto resid_to_mixer = [&](HyResid r, int l) {
         if (l < nl) {
             HyLayer& N = h->L[l];
-            r.norm_w = N.norm1;
+            r.norm_w = N.norm1;          // (null where the sublayers read the residual itself)
             if (h->shift && n == 1) { r.shift_mu = N.shift_mu; r.shift_prev = h->slots + N.off_shift; r.slot_stride = h->slot_floats; r.dyn = h->dyn; }
             else if (h->shift) r.hf = h->hf;
         }
-        hy_resid<T>(ctx, n, r, (T*)nullptr, hb);
+        hy_resid<T>(ctx, n, r, h->no_pre ? hb : (T*)nullptr, hb);
         if (l < nl && r.hf) {
             float* prev = h->slots + h->L[l].off_shift;
             const int v = W % 4 == 0 ? 4 : 1;
@@ -1292,7 +1458,7 @@ static int32_t hy_portion_plain(gl3_ctx* ctx, int seq, const int32_t* tokens, in
         // the last residual update of the layer: [side input,] depth average, tap, the next layer's norm
         auto finish = [&](HyResid r) {
             if (h->side_dim > 0) {
-                hy_resid<T>(ctx, n, r, (T*)h->xb, (T*)nullptr);
+                hy_resid<T>(ctx, n, r, (T*)h->xb, hb);          // (no norm: hb is not written)
                 if (n <= 8) {        // gate product with gelu_tanh(.) * the token's side embedding in the epilogue -> the projection's operand
                     hy_gemm<T>(ctx, (const T*)h->xb, W, L.side_gate, n, nullptr, 0, false, (T*)h->side_g, h->side_ld,
                                HyGlu{0.f, 0.f, 0.f, h->side_emb.w, h->tokens, h->side_emb.ld, l * h->side_dim});
@@ -1330,11 +1496,12 @@ static int32_t hy_portion_plain(gl3_ctx* ctx, int seq, const int32_t* tokens, in
             hy_resid<T>(ctx, n, r, (T*)nullptr, hb);
             continue;
         }
+        if (L.d.out_norm) { r.bw1 = L.branch_norm; r.bw2 = L.side->branch_norm; r.ya_first = h->y_first; }
         r.post_w = L.norm1b;          // null without post norms
         r.lw = L.ls1;                 // null without layer scales
         if (L.d.ff > 0) {
             r.norm_w = L.norm2;
-            hy_resid<T>(ctx, n, r, (T*)nullptr, hb);
+            hy_resid<T>(ctx, n, r, h->no_pre ? hb : (T*)nullptr, hb);
             r = base;
             r.post_w = L.norm2b;
             r.lw = L.ls2;
@@ -1342,6 +1509,7 @@ static int32_t hy_portion_plain(gl3_ctx* ctx, int seq, const int32_t* tokens, in
                 hy_moe<T>(ctx, L, n);
                 r.eo = h->eout; r.pair_row = h->pair_row; r.top = L.d.top;
                 if (L.d.route_on_output) r.ew = h->wsel;
+                if (h->no_pre) r.id_x = h->X;          // what an identity choice returns
                 if (L.d.shared_ff > 0) {
                     r.ya = h->y; r.ya_parts = h->y_parts; r.ya_stride = (size_t)n * W;
                     if (!L.d.shared_ungated) { r.gate_z = h->sgz; r.gate_ld = 1; }

@@ -463,6 +463,30 @@ bool kosusun_tensor(const std::string& name, int32_t& id, int32_t& layer, int32_
     return true;
 }
 
+// latent attention with a query latent: its sizes, and the rotated part (rot_dim entries; rot.dims says the same number again)
+bool latent_sizes(const JVal& mx, gl3_layer_desc& ld, std::string& err) {
+    if (!get_int(mx, "kv_rank", ld.kv_rank, err) || !get_int(mx, "q_rank", ld.q_rank, err) || !get_float(mx, "scale", ld.scale, err)) return false;
+    if (mx.get("rot_dim") && !mx.get("rot_dim")->is_null() && !get_int(mx, "rot_dim", ld.rot_dim, err)) return false;
+    if (ld.q_rank < 1) { err = "config: q_rank must be positive"; return false; }
+    return true;
+}
+bool latent_rot(const JVal& mx, gl3_layer_desc& ld, std::string& err) {
+    if (ld.rot_dim <= 0) return true;
+    const JVal* rot = mx.get("rot");
+    int32_t dims = 0;
+    if (!rot || rot->kind != JVal::OBJ || !get_int(*rot, "dims", dims, err) || !get_float(*rot, "base", ld.rot_base, err)) {
+        if (err.empty()) err = "config: a latent attention with rot_dim needs rot.dims and rot.base";
+        return false;
+    }
+    if (dims != ld.rot_dim) { err = "config: rot.dims must equal rot_dim"; return false; }
+    if (const JVal* sc = rot->get("scaling"))
+        if (sc->kind == JVal::OBJ &&
+            (!get_float(*sc, "factor", ld.rot_yarn_factor, err) || !get_float(*sc, "original", ld.rot_yarn_original, err) ||
+             !get_float(*sc, "fast", ld.rot_yarn_fast, err) || !get_float(*sc, "slow", ld.rot_yarn_slow, err)))
+            return false;
+    return true;
+}
+
 // Kugadra: one plain residual stream with a norm in front of AND behind every sublayer, x <- x + rms_norm(sublayer(rms_norm(x, w)), w_post).
 // Two layer types.  "lightning": a matrix memory with a fixed decay per head behind silu-activated q / k / v (no rotation, no other
 // scale), the heads side by side through ONE RMS norm with a weight, times sigmoid(W_g h).  "latent_attention": queries through a normed
@@ -509,9 +533,7 @@ bool kugadra_describe(const JVal& cfg, gl3_model_desc& d, std::vector<gl3_layer_
         } else if (ty->str == "latent_attention") {
             ld.mixer = GL3_MIX_LATENT;
             ld.out_gate = 2;
-            if (!get_int(*mx, "kv_rank", ld.kv_rank, err) || !get_int(*mx, "q_rank", ld.q_rank, err) || !get_float(*mx, "scale", ld.scale, err)) return false;
-            if (mx->get("rot_dim") && !mx->get("rot_dim")->is_null() && !get_int(*mx, "rot_dim", ld.rot_dim, err)) return false;
-            if (ld.q_rank < 1) { err = "config: q_rank must be positive"; return false; }
+            if (!latent_sizes(*mx, ld, err)) return false;
             if (const JVal* kf = mx->get("kv_from"))
                 if (!kf->is_null()) {
                     int32_t j = -1;
@@ -519,20 +541,7 @@ bool kugadra_describe(const JVal& cfg, gl3_model_desc& d, std::vector<gl3_layer_
                     if (j < 0 || j >= (int32_t)layers.size()) { err = "config: kv_from must name an earlier layer"; return false; }
                     ld.kv_share = j + 1;
                 }
-            if (ld.rot_dim > 0) {
-                const JVal* rot = mx->get("rot");
-                int32_t dims = 0;
-                if (!rot || rot->kind != JVal::OBJ || !get_int(*rot, "dims", dims, err) || !get_float(*rot, "base", ld.rot_base, err)) {
-                    if (err.empty()) err = "config: a latent attention with rot_dim needs rot.dims and rot.base";
-                    return false;
-                }
-                if (dims != ld.rot_dim) { err = "config: rot.dims must equal rot_dim"; return false; }
-                if (const JVal* sc = rot->get("scaling"))
-                    if (sc->kind == JVal::OBJ &&
-                        (!get_float(*sc, "factor", ld.rot_yarn_factor, err) || !get_float(*sc, "original", ld.rot_yarn_original, err) ||
-                         !get_float(*sc, "fast", ld.rot_yarn_fast, err) || !get_float(*sc, "slow", ld.rot_yarn_slow, err)))
-                        return false;
-            }
+            if (!latent_rot(*mx, ld, err)) return false;
         } else { err = "config: unknown layer type '" + ty->str + "'"; return false; }
         if (mlp && !mlp->is_null()) {
             const JVal* kind = mlp->get("kind");
@@ -679,8 +688,123 @@ bool tutedra_tensor(const std::string& name, int32_t& id, int32_t& layer, int32_
     return expert_leaf(lf, id, expert);
 }
 
+// Ziginex: one plain residual stream whose sublayers read the residual itself and whose outputs are normed, x <- x + N(mixer(x), norm1),
+// x <- x + N(ff(x), norm2), x <- x + N(per-layer token input, side.norm); the head is the embedding table.  Two layer types.  "parallel": two
+// mixers side by side, each output normed over the width with a weight of its own, half their sum: `left` = grouped-query attention (RMS norm
+// per head with a shared weight on q and k, interleaved rotary pairs, scores times a number per head, capped, mixed over the heads, inside
+// chunks of the sequence, a learned sink per head), `right` = the gated delta rule (short convolutions with silu on q, k and v, unit q and k,
+// q times dim^(-1/2), heads normed with one shared weight, times silu(W_g h)).  "latent_attention": a query latent, one rotated key part with
+// blended frequencies, a learned sink per head, one sigmoid gate per output element.  Feed-forward: W_down (silu(W_gate x) * (W_up x)), or a
+// mixture of such experts and identity choices (softmax scores, chosen by score + correction among the groups with the largest choice
+// scores, the plain scores weight the outputs).  config.json gives every size and the constants; the forms are fixed here.
+bool ziginex_describe(const JVal& cfg, gl3_model_desc& d, std::vector<gl3_layer_desc>& layers, DescStore& store, std::string& err) {
+    d.arch = GL3_ARCH_LAYERLIST;
+    d.weight_type = GL3_TYPE_BF16;
+    if (!get_int(cfg, "vocab", d.vocab, err) || !get_int(cfg, "width", d.dim, err)) return false;
+    d.streams = 0;
+    d.post_norms = d.no_pre_norms = 1;
+    d.embedding_scale = 1.f;
+    if (const JVal* ts = cfg.get("token_side"))
+        if (ts->kind == JVal::OBJ && !get_int(*ts, "dim", d.side_dim, err)) return false;
+    const JVal* norm = cfg.get("norm");
+    if (!norm || !get_float(*norm, "eps", d.rms_eps, err)) { if (err.empty()) err = "config: missing norm.eps"; return false; }
+    const JVal* ls = cfg.get("layers");
+    if (!ls || ls->kind != JVal::ARR || ls->arr.empty()) { err = "config: 'layers' must be a non-empty list"; return false; }
+    for (const JVal& l : ls->arr) {
+        gl3_layer_desc ld{};
+        const JVal *ty = l.get("type"), *mx = l.get("mixer"), *mlp = l.get("mlp");
+        if (!ty || ty->kind != JVal::STR || !mx || mx->kind != JVal::OBJ) { err = "config: a layer needs 'type' and 'mixer'"; return false; }
+        if (ty->str == "parallel") {
+            const JVal *left = mx->get("left"), *right = mx->get("right");
+            if (!left || left->kind != JVal::OBJ || !right || right->kind != JVal::OBJ) { err = "config: a parallel mixer needs 'left' and 'right'"; return false; }
+            ld.mixer = GL3_MIX_ATTENTION;
+            if (!get_int(*left, "heads", ld.heads, err) || !get_int(*left, "kv_heads", ld.kv_heads, err) || !get_int(*left, "dim", ld.dim, err) || !get_int(*left, "vdim", ld.vdim, err) ||
+                !get_float(*left, "scale", ld.scale, err) || !get_rot(*left, ld, err))
+                return false;
+            ld.qk_unit_norm = 3; ld.rot_interleaved = 1; ld.softmax_sink = 2; ld.head_temp = ld.head_mix = 1; ld.out_norm = 1; ld.out_scale = 0.5f;
+            if (left->get("softcap") && !left->get("softcap")->is_null() && !get_float(*left, "softcap", ld.score_softcap, err)) return false;
+            if (const JVal* mask = left->get("mask"))
+                if (mask->kind == JVal::OBJ) {
+                    if (!get_int(*mask, "size", ld.chunk, err)) return false;
+                    if (ld.chunk < 1) { err = "config: mask.size must be positive"; return false; }
+                }
+            gl3_layer_desc rd{};
+            rd.mixer = GL3_MIX_MEMORY;
+            rd.mem_gates = GL3_MEM_DELTA;
+            if (!get_int(*right, "heads", rd.heads, err) || !get_int(*right, "kv_heads", rd.kv_heads, err) || !get_int(*right, "dim", rd.dim, err) || !get_int(*right, "vdim", rd.vdim, err) ||
+                !get_int(*right, "conv", rd.mem_conv, err))
+                return false;
+            rd.mem_qkv_act = 1; rd.mem_qk_unit = 1; rd.mem_norm_weight = 2; rd.mem_gate_act = 0; rd.out_norm = 1; rd.out_scale = 0.5f;
+            rd.mem_q_mul = (float)(1.0 / std::sqrt((double)std::max(1, rd.dim)));
+            store.descs.push_back(rd);
+            ld.beside = &store.descs.back();
+        } else if (ty->str == "latent_attention") {
+            ld.mixer = GL3_MIX_LATENT;
+            if (!get_int(*mx, "heads", ld.heads, err) || !get_int(*mx, "dim", ld.dim, err) || !get_int(*mx, "vdim", ld.vdim, err) || !latent_sizes(*mx, ld, err) || !latent_rot(*mx, ld, err)) return false;
+            ld.kv_heads = ld.heads;
+            ld.out_gate = 1; ld.softmax_sink = 2;
+        } else { err = "config: unknown layer type '" + ty->str + "'"; return false; }
+        if (mlp && !mlp->is_null()) {
+            const JVal* kind = mlp->get("kind");
+            if (!kind || kind->kind != JVal::STR) { err = "config: mlp needs 'kind'"; return false; }
+            ld.ff_alpha = 1.f; ld.ff_shift = 0.f;          // silu(g) u
+            if (kind->str == "dense") {
+                if (!get_int(*mlp, "ff", ld.ff, err)) return false;
+            } else if (kind->str == "moe") {
+                const JVal *ex = mlp->get("expert"), *ro = mlp->get("router");
+                if (!ex || !ro || !get_int(*ex, "ff", ld.ff, err) || !get_int(*ro, "experts", ld.experts, err) || !get_int(*ro, "top", ld.top, err)) {
+                    if (err.empty()) err = "config: a mixture of experts needs 'expert' and 'router'";
+                    return false;
+                }
+                if (ro->get("identity") && !ro->get("identity")->is_null() && !get_int(*ro, "identity", ld.identity, err)) return false;
+                if (const JVal* gr = ro->get("groups"))
+                    if (!gr->is_null() && (!get_int(*gr, "count", ld.route_groups, err) || !get_int(*gr, "keep", ld.route_keep, err))) return false;
+                ld.route_softmax = ld.route_bias = ld.route_on_output = ld.route_group_max = 1;
+            } else { err = "config: mlp.kind must be 'dense' or 'moe'"; return false; }
+        }
+        layers.push_back(ld);
+    }
+    d.n_layers = (int32_t)layers.size();
+    return true;
+}
+
+bool ziginex_tensor(const std::string& name, int32_t& id, int32_t& layer, int32_t& expert) {
+    static const std::map<std::string, int> global = {{"embed", GL3_T_TOKEN_EMBD}, {"side.embed", GL3_T_SIDE_EMBD}, {"final.norm", GL3_T_OUTPUT_NORM}};
+    static const std::map<std::string, int> leaf = {
+        {"norm1", GL3_T_ATTN_POST_NORM}, {"norm2", GL3_T_FFN_POST_NORM}, {"side.gate", GL3_T_SIDE_GATE}, {"side.proj", GL3_T_SIDE_PROJ}, {"side.norm", GL3_T_SIDE_NORM},
+        {"mlp.gate", GL3_T_W1}, {"mlp.up", GL3_T_W3}, {"mlp.down", GL3_T_W2}, {"mlp.router", GL3_T_FFN_GATE_INP}, {"mlp.correction", GL3_T_FFN_ROUTE_BIAS}};
+    // tensors of one mixer, after "mix." (latent attention), "mix.left." (attention) or "mix.right." (delta rule)
+    static const std::map<std::string, int> latent = {
+        {"dq", GL3_T_Q_DOWN}, {"dq.norm", GL3_T_Q_DOWN_NORM}, {"uq", GL3_T_WQ}, {"dkv", GL3_T_KV_DOWN}, {"dkv.norm", GL3_T_KV_DOWN_NORM}, {"uk", GL3_T_K_UP},
+        {"uv", GL3_T_V_UP}, {"sink", GL3_T_ATTN_SINK}, {"g", GL3_T_ATTN_GATE}, {"o", GL3_T_WO}};
+    static const std::map<std::string, int> left = {
+        {"q", GL3_T_WQ}, {"k", GL3_T_WK}, {"v", GL3_T_WV}, {"o", GL3_T_WO}, {"q.norm", GL3_T_ATTN_Q_NORM}, {"k.norm", GL3_T_ATTN_K_NORM}, {"talk", GL3_T_HEAD_MIX},
+        {"temp", GL3_T_ATTN_TEMP}, {"sink", GL3_T_ATTN_SINK}, {"out", GL3_T_BRANCH_NORM}};
+    static const std::map<std::string, int> right = {
+        {"q", GL3_T_WQ}, {"k", GL3_T_WK}, {"v", GL3_T_WV}, {"o", GL3_T_WO}, {"g", GL3_T_ATTN_GATE}, {"q.conv", GL3_T_Q_CONV}, {"k.conv", GL3_T_K_CONV},
+        {"v.conv", GL3_T_V_CONV}, {"b", GL3_T_MEM_IGATE}, {"a", GL3_T_MEM_FGATE}, {"A_log", GL3_T_SSM_A_LOG}, {"dt_bias", GL3_T_SSM_DT_BIAS}, {"norm", GL3_T_SSM_NORM},
+        {"out", GL3_T_BRANCH_NORM}};
+    expert = -1;
+    auto g = global.find(name);
+    if (g != global.end()) { id = g->second; layer = 0; return true; }
+    std::string lf;
+    if (!split_layer_name(name, layer, lf)) return false;
+    auto f = leaf.find(lf);
+    if (f != leaf.end()) { id = f->second; return true; }
+    if (lf.compare(0, 4, "mix.") != 0) return expert_leaf(lf, id, expert);
+    std::string rest = lf.substr(4);
+    const std::map<std::string, int>* table = &latent;
+    if (rest.compare(0, 5, "left.") == 0) { rest = rest.substr(5); table = &left; }
+    else if (rest.compare(0, 6, "right.") == 0) { rest = rest.substr(6); table = &right; layer |= GL3_LAYER_BESIDE; }
+    auto m = table->find(rest);
+    if (m == table->end()) return false;
+    id = m->second;
+    return true;
+}
+
 const Design DESIGNS[] = {{"Noditar", noditar_describe, noditar_tensor}, {"Vonulix", vonulix_describe, vonulix_tensor}, {"Kosusun", kosusun_describe, kosusun_tensor},
-                          {"Kugadra", kugadra_describe, kugadra_tensor}, {"Tutedra", tutedra_describe, tutedra_tensor}};
+                          {"Kugadra", kugadra_describe, kugadra_tensor}, {"Tutedra", tutedra_describe, tutedra_tensor},
+                          {"Ziginex", ziginex_describe, ziginex_tensor}};
 
 struct Mapping {
     void* p = MAP_FAILED; size_t n = 0;

@@ -22,7 +22,7 @@ FLAG_F32_COMPUTE = 128                         # layer-list family: float32 matr
 ARCH_NODITAR = ARCH_LAYERLIST = 6      # the layer-list family; its designs differ in parameters only
 TYPE_F32, TYPE_BF16 = 0, 30
 MIX_ATTENTION, MIX_LATENT, MIX_SSM, MIX_MEMORY = 0, 1, 2, 3
-MEM_DECAY, MEM_EXP_GATES = 0, 1
+MEM_DECAY, MEM_EXP_GATES, MEM_CHANNEL_GATES, MEM_DELTA = 0, 1, 2, 3
 LAYER_BESIDE = 1 << 30
 K_NAMES = ["matvec_qkv", "matvec_wo", "matvec_gateup", "matvec_down", "matvec_logits", "attention", "other", "collective"]
 
@@ -67,7 +67,9 @@ class LayerDesc(C.Structure):
                 ("mem_qkv_act", C.c_int32), ("mem_norm_whole", C.c_int32), ("route_softmax", C.c_int32), ("route_bias", C.c_int32),
                 ("route_renorm", C.c_int32), ("route_on_output", C.c_int32), ("shared_ungated", C.c_int32), ("route_scale", C.c_float),
                 ("qk_conv", C.c_int32), ("v_from_k", C.c_int32), ("rot_wave_factor", C.c_float), ("rot_wave_low", C.c_float),
-                ("rot_wave_high", C.c_float), ("rot_wave_original", C.c_float), ("route_groups", C.c_int32), ("route_keep", C.c_int32)]
+                ("rot_wave_high", C.c_float), ("rot_wave_original", C.c_float), ("route_groups", C.c_int32), ("route_keep", C.c_int32),
+                ("head_temp", C.c_int32), ("score_softcap", C.c_float), ("head_mix", C.c_int32), ("chunk", C.c_int32), ("mem_conv", C.c_int32),
+                ("mem_qk_unit", C.c_int32), ("out_norm", C.c_int32), ("identity", C.c_int32), ("route_group_max", C.c_int32)]
 
 
 class ModelDesc(C.Structure):
@@ -81,7 +83,7 @@ class ModelDesc(C.Structure):
                 ("streams", C.c_int32), ("layer_descs", C.POINTER(LayerDesc)),
                 ("norm_offset", C.c_float), ("side_dim", C.c_int32), ("depth_mix", C.c_int32), ("parallel_block", C.c_int32),
                 ("post_norms", C.c_int32), ("logit_softcap", C.c_float), ("bigram_buckets", C.c_int32), ("bigram_mul_prev", C.c_int32),
-                ("bigram_mul_cur", C.c_int32), ("token_shift", C.c_int32), ("layer_scale", C.c_int32)]
+                ("bigram_mul_cur", C.c_int32), ("token_shift", C.c_int32), ("layer_scale", C.c_int32), ("no_pre_norms", C.c_int32)]
 
 
 class KernelTimes(C.Structure):

@@ -71,7 +71,7 @@ enum { GL3_ARCH_LLAMA = 0, GL3_ARCH_QWEN3 = 1, GL3_ARCH_QWEN2 = 2,
                               * gl3_layer_desc; several residual streams mixed by per-sublayer tables, or one plain residual with an optional
                               * weighted average over all earlier layers' results; bfloat16 or float32 matrices
                               * (GL3_TYPE_BF16, GL3_FLAG_F32_COMPUTE); model folders with config.json + model.safetensors (gl3_load_model_dir) */
-       GL3_ARCH_LAYERLIST = 6 /* the same family under its own name: the registered designs (Noditar, Vonulix, Kosusun, Kugadra, Tutedra) differ only in
+       GL3_ARCH_LAYERLIST = 6 /* the same family under its own name: the registered designs (Noditar, Vonulix, Kosusun, Kugadra, Tutedra, Ziginex) differ only in
                               * the parameters of gl3_model_desc / gl3_layer_desc that their `describe` fills in */ };
 
 /* token mixers of a layer-list model (gl3_layer_desc.mixer) */
@@ -81,17 +81,21 @@ enum { GL3_MIX_ATTENTION = 0,   /* grouped-query softmax attention over cached k
        GL3_MIX_LATENT = 1,      /* attention whose keys and values are expanded from one cached low-rank latent per token */
        GL3_MIX_SSM = 2,         /* selective state-space recurrence (scalar decay per head) behind a short causal convolution */
        GL3_MIX_MEMORY = 3 };    /* matrix memory per head, S_t = a_t S_(t-1) + b_t k_t v_t^T, o_t = S_t^T q_t, float32 state carried per sequence:
-                                 * a fixed decay per head (retention), exponential gates with a running maximum and a normaliser (mLSTM), or a
-                                 * forget gate per head and channel whose complement is the key (HGRN2) */
+                                 * a fixed decay per head (retention), exponential gates with a running maximum and a normaliser (mLSTM), a
+                                 * forget gate per head and channel whose complement is the key (HGRN2), or the gated delta rule (writes what the key
+                                 * does not already recall) */
 
 /* gl3_layer_desc.mem_gates: how a matrix memory gets a_t and b_t */
 enum { GL3_MEM_DECAY = 0,       /* a = mem_decay[head], b = 1; no normaliser: o = S^T q */
        GL3_MEM_EXP_GATES = 1,  /* log gates from two projections with biases: i = cap tanh(z_i / cap), f = logsigmoid(cap tanh(z_f / cap));
                                  * m_t = max(f + m_(t-1), i), m_0 = 0; a = e^(f + m_(t-1) - m_t), b = e^(i - m_t); n_t = a n + b k;
                                  * o = S^T q / (max(|n . q|, e^(-m_t)) + 1e-6) */
-       GL3_MEM_CHANNEL_GATES = 2 }; /* one forget gate per head and key channel, f = l + (1 - l) sigmoid(z_f + bias); S_t = diag(f) S_(t-1) + (1 - f) v^T,
+       GL3_MEM_CHANNEL_GATES = 2, /* one forget gate per head and key channel, f = l + (1 - l) sigmoid(z_f + bias); S_t = diag(f) S_(t-1) + (1 - f) v^T,
                                  * o = S^T q: no key projection; z_f from GL3_T_MEM_FGATE [heads dim x width], GL3_T_MEM_FGATE_BIAS [heads dim], l from
                                  * GL3_T_MEM_LOWER [heads dim] */
+       GL3_MEM_DELTA = 3 };     /* gated delta rule: S <- a S; S <- S + k (b (v - S^T k))^T; o = S^T q, with a = exp(-exp(A_log) softplus(z_a + dt_bias)) and
+                                 * b = sigmoid(z_b) per head: z_a from GL3_T_MEM_FGATE, z_b from GL3_T_MEM_IGATE ([heads x width], no biases), A_log and dt_bias from
+                                 * GL3_T_SSM_A_LOG / GL3_T_SSM_DT_BIAS [heads].  kv_heads query / key heads serve the heads in equal runs; see mem_conv, mem_qk_unit */
 
 /* gl3_upload_tensor: `layer` + GL3_LAYER_BESIDE addresses the second mixer of a layer (gl3_layer_desc.beside) */
 #define GL3_LAYER_BESIDE (1 << 30)
@@ -194,6 +198,26 @@ typedef struct gl3_layer_desc {
      * route_groups > 0: the experts form that many equal runs of neighbours; a run's score is the sum of its two largest choice scores
      * (score + bias) and only experts of the best route_keep runs can be chosen */
     int32_t route_groups, route_keep;
+    /* attention, further switches (each usable alone; they go without windows, pooled blocks and a distance term; heads <= 128).  A head's score of a key is
+     * s = scale (q . k), times GL3_T_ATTN_TEMP[head] if head_temp != 0, then cap tanh(s / cap) if score_softcap > 0, then the heads' scores
+     * are mixed, s_h <- sum_g T[h][g] s_g with T = GL3_T_HEAD_MIX [heads x heads], if head_mix != 0.  chunk > 0: query i sees key j <= i
+     * only if both lie in the same run of `chunk` positions, counted from the sequence's position 0.  softmax_sink = 2 is also read by
+     * the latent attention */
+    int32_t head_temp;
+    float   score_softcap;
+    int32_t head_mix, chunk;
+    /* matrix memory with the gated delta rule: mem_conv (>= 1) taps of a causal depthwise convolution over time on every q, k and v channel, before
+     * mem_qkv_act (GL3_T_Q_CONV / K_CONV [kv_heads dim x mem_conv], GL3_T_V_CONV [heads vdim x mem_conv], last column = current token; the last
+     * mem_conv - 1 projected rows belong to the sequence slot); mem_qk_unit = 1: q and k of every head become x / sqrt(sum x^2 + 1e-6) behind it, before
+     * mem_q_mul / mem_k_mul */
+    int32_t mem_conv, mem_qk_unit;
+    /* Two mixers side by side, out_norm != 0 (on both or on neither): each mixer's projected output is RMS-normed over the model width with a weight
+     * of its own (GL3_T_BRANCH_NORM [width]) before out_scale multiplies it and the two are added */
+    int32_t out_norm;
+    /* mixture of experts with route_on_output, further switches.  identity: that many more router outputs behind the experts' (scores, bias, groups
+     * and choice run over experts + identity); the output of such a choice is the sublayer's input itself, it has no tensors.
+     * route_group_max = 1: a run's score is its largest choice score (else the sum of the two largest) */
+    int32_t identity, route_group_max;
 } gl3_layer_desc;
 
 /* ggml tensor types of the wire format (J/tensor/GGMLType.java:5-21) */
@@ -270,7 +294,11 @@ enum {
     GL3_T_Q_CONV = 62,             /* attention with qk_conv: taps of the q channels [heads * dim x qk_conv]             */
     GL3_T_K_CONV = 63,             /*                         taps of the k channels [kv_heads * dim x qk_conv]          */
     GL3_T_MEM_LOWER = 64,          /* matrix memory, channel gates: lower bound      [heads * dim]                       */
-    GL3_T_COUNT = 65
+    GL3_T_ATTN_TEMP = 65,          /* attention with head_temp: multiplier of a head's scores  [heads]                  */
+    GL3_T_HEAD_MIX = 66,           /* attention with head_mix: heads' scores from heads' scores [heads x heads]         */
+    GL3_T_V_CONV = 67,             /* gated delta rule: taps of the v channels       [heads * vdim x mem_conv] (its q and k channels: GL3_T_Q_CONV, GL3_T_K_CONV) */
+    GL3_T_BRANCH_NORM = 68,        /* one of two mixers side by side with out_norm: norm of its projected output  [width] */
+    GL3_T_COUNT = 69
 };
 
 /* gl3_model_desc.flags */
@@ -355,6 +383,9 @@ typedef struct {
      * GL3_T_FFN_SCALE before it joins the residual. */
     int32_t bigram_buckets, bigram_mul_prev, bigram_mul_cur;
     int32_t token_shift, layer_scale;
+    /* layer-list family with streams == 0 and post_norms: no_pre_norms != 0: the sublayers read the residual itself,
+     * x <- x + rms_norm(sublayer(x), w_post) (no GL3_T_ATTN_NORM / GL3_T_FFN_NORM) */
+    int32_t no_pre_norms;
 } gl3_model_desc;
 
 /* Per-kernel-class device time of one instrumented decode step (HIP events around every launch). */
