@@ -117,12 +117,17 @@ def main():
                     "prints its own JSON line instead of the tg/pp line")
     ap.add_argument("--tutedra", default="", help="layer-list family, Tutedra design (bfloat16: HGRN2, mLSTM and attention layers with a token shift in front "
                     "and a scale behind every sublayer, polynomial feed-forward, relu^2 experts): comma-separated sizes (1b, 8b); prints its own JSON line")
+    ap.add_argument("--ziginex", default="", help="layer-list family, Ziginex design (bfloat16: norms behind the sublayers only; attention with mixed head scores "
+                    "inside chunks beside a gated delta rule, latent attention, experts and identity choices, per-layer token input): comma-separated "
+                    "sizes (1b, 8b); prints its own JSON line")
     ap.add_argument("--kugadra", default="", help="layer-list family, Kugadra design (bfloat16: norms on both sides of every sublayer; lightning layers; "
                     "latent attention with a query latent, a shared rotated key part and a cache that the next layer reads; relu^2 feed-forward and a "
                     "mixture of experts with a softmax router): prefill and decode throughput at layer sizes of a real model beside the family's closest "
                     "design at equal size (Noditar latent-attention and state-space layers, same heads, row and state sizes, dense feed-forward of the "
                     "same active width); comma list of sizes from 1b,8b; prints its own JSON line instead of the tg/pp line")
     args = ap.parse_args()
+    if args.ziginex:
+        return bench_ziginex(args)
     if args.tutedra:
         return bench_tutedra(args)
     if args.kugadra:
@@ -851,6 +856,52 @@ def bench_tutedra(args):
     return bench_design_pair(args, "tutedra", "Tutedra", args.tutedra, TUTEDRA_SIZES, tutedra_config, tutedra_twin_config,
                              "twin = Noditar attention and state-space layers on one stream with the same heads and state sizes and a dense feed-forward of the "
                              "same active width, equal width / layers / vocabulary")
+
+
+ZIGINEX_SIZES = {   # width, dense feed-forward, layers (parallel, latent, parallel, parallel, ...; the first dense, the others experts), vocabulary; attention heads /
+                    # kv heads / head size, chunk; delta-rule heads / key heads x key size x value size; latent heads, unrotated + rotated key size, value
+                    # size, latent sizes; experts x width, identity choices, choices, groups (kept); token input
+    "1b": dict(width=2048, ff=8192, n_layers=8, vocab=32000, heads=32, kv_heads=8, dim=64, chunk=2048, d_heads=16, d_kv_heads=8, d_dim=128, d_vdim=128, conv=4,
+               l_heads=32, l_dim=64, l_rot=32, l_vdim=64, kv_rank=224, q_rank=768, experts=32, identity=8, top=8, groups=8, keep=4, expert_ff=1024, side=128),
+    "8b": dict(width=4096, ff=14336, n_layers=4, vocab=32000, heads=32, kv_heads=8, dim=128, chunk=2048, d_heads=32, d_kv_heads=16, d_dim=128, d_vdim=128, conv=4,
+               l_heads=32, l_dim=128, l_rot=64, l_vdim=128, kv_rank=448, q_rank=1536, experts=32, identity=8, top=8, groups=8, keep=4, expert_ff=1792, side=256),
+}
+
+
+def ziginex_config(z):
+    D = z["dim"]
+    moe = {"kind": "moe", "expert": {"ff": z["expert_ff"]},
+           "router": {"experts": z["experts"], "identity": z["identity"], "top": z["top"], "groups": {"count": z["groups"], "keep": z["keep"]}}}
+    par = {"type": "parallel",
+           "mixer": {"left": {"heads": z["heads"], "kv_heads": z["kv_heads"], "dim": D, "vdim": D, "scale": D ** -0.5, "softcap": 30.0, "mask": {"size": z["chunk"]},
+                              "rot": {"base": 500000.0, "dims": D // 2}},
+                     "right": {"heads": z["d_heads"], "kv_heads": z["d_kv_heads"], "dim": z["d_dim"], "vdim": z["d_vdim"], "conv": z["conv"]}}}
+    lat = {"type": "latent_attention",
+           "mixer": {"heads": z["l_heads"], "dim": z["l_dim"], "rot_dim": z["l_rot"], "vdim": z["l_vdim"], "kv_rank": z["kv_rank"], "q_rank": z["q_rank"],
+                     "scale": float(z["l_dim"] + z["l_rot"]) ** -0.5,
+                     "rot": {"base": 500000.0, "dims": z["l_rot"], "scaling": {"factor": 8.0, "original": 4096, "fast": 16.0, "slow": 2.0}}}}
+    return {"architecture": "Ziginex", "vocab": z["vocab"], "width": z["width"], "norm": {"eps": 1e-6}, "token_side": {"dim": z["side"]},
+            "layers": [dict(lat if i % 4 == 1 else par, mlp=moe if i else {"kind": "dense", "ff": z["ff"]}) for i in range(z["n_layers"])]}
+
+
+def ziginex_twin_config(z):
+    """The family's closest design at equal size: Kosusun layers — attention with the same heads and a window of the chunk's size beside retention with
+    the same heads, key and value sizes — with a dense gated feed-forward as wide as what a token uses; also in the place of the latent
+    layers, whose kernels Kugadra's latent layers of the same sizes stand beside (bench.py --kugadra)."""
+    D, n = z["dim"], z["d_heads"]
+    par = {"type": "parallel", "mlp": {"kind": "dense", "ff": z["ff"]},
+           "mixer": {"left": {"heads": z["heads"], "kv_heads": z["kv_heads"], "dim": D, "vdim": D, "scale": D ** -0.5, "mask": {"size": z["chunk"]},
+                              "rot": {"base": 500000.0, "dims": D // 2}},
+                     "right": {"heads": n, "dim": z["d_dim"], "vdim": z["d_vdim"], "rot": {"base": 10000.0, "dims": z["d_dim"]},
+                               "decay": [1.0 - 2.0 ** (-5.0 - 3.0 * i / max(1, n - 1)) for i in range(n)]}}}
+    return {"architecture": "Kosusun", "vocab": z["vocab"], "width": z["width"], "norm": {"eps": 1e-6}, "layers": [par] * z["n_layers"]}
+
+
+def bench_ziginex(args):
+    """As bench_vonulix, for the Ziginex design beside its twin."""
+    return bench_design_pair(args, "ziginex", "Ziginex", args.ziginex, ZIGINEX_SIZES, ziginex_config, ziginex_twin_config,
+                             "twin = Kosusun layers (windowed attention beside retention) with the same heads, key and value sizes and a dense feed-forward of the same "
+                             "active width, equal width / layers / vocabulary")
 
 
 def bench_design_pair(args, label_key, design, sizes_arg, SIZES, config_fn, twin_fn, twin_text):

@@ -50,6 +50,18 @@ __device__ __forceinline__ float hy_block_sum(float v, float* red) {
     return a;
 }
 
+// two sums at once (red: 2 NT / 64 floats)
+template <int NT>
+__device__ __forceinline__ void hy_block_sum2(float& a, float& b, float* red) {
+    a = hy_wave_sum(a); b = hy_wave_sum(b);
+    __syncthreads();
+    if ((threadIdx.x & 63) == 0) { red[threadIdx.x >> 6] = a; red[NT / 64 + (threadIdx.x >> 6)] = b; }
+    __syncthreads();
+    a = b = 0.f;
+#pragma unroll
+    for (int i = 0; i < NT / 64; ++i) { a += red[i]; b += red[NT / 64 + i]; }
+}
+
 // step record in device memory (read by the kernels, so that a captured step can be replayed at another position):
 // dyn[0] = position of the step's first token, dyn[1] = sequence slot, dyn[2] = the sequence's token before the step's first one
 constexpr int HY_MAX_STREAMS = 8;

@@ -62,7 +62,7 @@ template <int V> __device__ __forceinline__ void hy_stv(bf16_t* __restrict__ p, 
 constexpr int HY_RC = 2, HY_MAX_PARTS = 4, HY_MIX_UNROLL = 4;
 template <typename TO, int NT, int V, bool BR>
 static __global__ __launch_bounds__(NT) void hy_resid_kernel(HyResid a, TO* __restrict__ xt, TO* h_out) {
-    __shared__ float red[NT / 64];
+    __shared__ float red[2 * (NT / 64)];
     const int t = blockIdx.x, W = a.W;
     const size_t row = (size_t)t * W;
     float cr = 0.f;
@@ -98,28 +98,42 @@ static __global__ __launch_bounds__(NT) void hy_resid_kernel(HyResid a, TO* __re
             for (int i = 0; i < V; ++i) y[i] += q[i];
         }
     };
-    float b1 = 0.f, b2 = 0.f;          // two normed mixers: 1 / rms of each one's whole output
+    float b1 = 0.f, b2 = 0.f;          // two normed mixers: 1 / rms of each one's whole output; its first chunks stay in registers for `addend`
+    float by[BR ? HY_RC : 1][V], bz[BR ? HY_RC : 1][V];
     if constexpr (BR) {
-        for (int w = threadIdx.x * V; w < W; w += NT * V) {
+        int it = 0;
+        for (int w = threadIdx.x * V; w < W; w += NT * V, ++it) {
             float y[V], z[V];
             parts(w, 0, a.ya_first, y);
             parts(w, a.ya_first, a.ya_parts, z);
 #pragma unroll
             for (int i = 0; i < V; ++i) { b1 += y[i] * y[i]; b2 += z[i] * z[i]; }
+#pragma unroll
+            for (int q = 0; q < HY_RC; ++q)
+                if (q == it)
+#pragma unroll
+                    for (int i = 0; i < V; ++i) { by[q][i] = y[i]; bz[q][i] = z[i]; }
         }
-        b1 = hy_block_sum<NT>(b1, red);
-        b2 = hy_block_sum<NT>(b2, red);
+        hy_block_sum2<NT>(b1, b2, red);
         b1 = 1.f / sqrtf(b1 / (float)W + a.eps);
         b2 = 1.f / sqrtf(b2 / (float)W + a.eps);
     }
-    // column w of what joins the residual: y (the sublayer's output) and e (the routed experts')
-    auto addend = [&](int w, float* y, float* e) {
+    // column w (the thread's chunk it) of what joins the residual: y (the sublayer's output) and e (the routed experts')
+    auto addend = [&](int w, int it, float* y, float* e) {
 #pragma unroll
         for (int i = 0; i < V; ++i) y[i] = e[i] = 0.f;
         if constexpr (BR) {
             float z[V], w1[V], w2[V];
-            parts(w, 0, a.ya_first, y);
-            parts(w, a.ya_first, a.ya_parts, z);
+            if (it < HY_RC) {
+#pragma unroll
+                for (int q = 0; q < HY_RC; ++q)
+                    if (q == it)
+#pragma unroll
+                        for (int i = 0; i < V; ++i) { y[i] = by[q][i]; z[i] = bz[q][i]; }
+            } else {
+                parts(w, 0, a.ya_first, y);
+                parts(w, a.ya_first, a.ya_parts, z);
+            }
             hy_ldv<V>(a.bw1 + w, w1);
             hy_ldv<V>(a.bw2 + w, w2);
 #pragma unroll
@@ -143,7 +157,7 @@ static __global__ __launch_bounds__(NT) void hy_resid_kernel(HyResid a, TO* __re
         int it = 0;
         for (int w = threadIdx.x * V; w < W; w += NT * V, ++it) {
             float y[V], e[V];
-            addend(w, y, e);
+            addend(w, it, y, e);
 #pragma unroll
             for (int i = 0; i < V; ++i) { y[i] = ga * y[i] + e[i]; sd += y[i] * y[i]; }
 #pragma unroll
@@ -169,7 +183,7 @@ static __global__ __launch_bounds__(NT) void hy_resid_kernel(HyResid a, TO* __re
 #pragma unroll
                     for (int i = 0; i < V; ++i) y[i] = kept[q][i];
         } else {
-            addend(w, y, e);
+            addend(w, it, y, e);
             if (a.post_w)
 #pragma unroll
                 for (int i = 0; i < V; ++i) y[i] = ga * y[i] + e[i];
@@ -324,15 +338,16 @@ static __global__ __launch_bounds__(256) void hy_side_act_kernel(const float* __
 // expert's gate logit) is summed into extra_out[t].
 constexpr int HY_RT_PER = 16;
 struct HyRoute { int softmax; const float* bias; int renorm; float mul; int groups, keep; int real, group_max; };
+template <int PER>          // router rows per lane: rows <= 64 PER
 static __global__ __launch_bounds__(64) void hy_route_kernel(const float* __restrict__ z, int ldz, int parts, size_t pstride, int E, int top, int* __restrict__ sel,
                                                              float* __restrict__ wgt, int* __restrict__ pair_row, float* __restrict__ extra_out,
                                                              HyRoute rt) {
     const int t = blockIdx.x, lane = threadIdx.x;
     constexpr float GONE = -3.0e38f;
-    float s[HY_RT_PER], c[HY_RT_PER];          // score; what the choice goes by
+    float s[PER], c[PER];          // score; what the choice goes by
     float zmax = -INFINITY;
 #pragma unroll
-    for (int i = 0; i < HY_RT_PER; ++i) {
+    for (int i = 0; i < PER; ++i) {
         const int e = lane + 64 * i;
         float v = 0.f;
         if (e < E + (extra_out ? 1 : 0))
@@ -345,24 +360,24 @@ static __global__ __launch_bounds__(64) void hy_route_kernel(const float* __rest
         zmax = hy_wave_max(zmax);
         float den = 0.f;
 #pragma unroll
-        for (int i = 0; i < HY_RT_PER; ++i) { s[i] = lane + 64 * i < E ? expf(s[i] - zmax) : 0.f; den += s[i]; }
+        for (int i = 0; i < PER; ++i) { s[i] = lane + 64 * i < E ? expf(s[i] - zmax) : 0.f; den += s[i]; }
         den = hy_wave_sum(den);
 #pragma unroll
-        for (int i = 0; i < HY_RT_PER; ++i) s[i] = s[i] / den;
+        for (int i = 0; i < PER; ++i) s[i] = s[i] / den;
     } else {
 #pragma unroll
-        for (int i = 0; i < HY_RT_PER; ++i) s[i] = hy_sigmoid(s[i]);
+        for (int i = 0; i < PER; ++i) s[i] = hy_sigmoid(s[i]);
     }
 #pragma unroll
-    for (int i = 0; i < HY_RT_PER; ++i) {
+    for (int i = 0; i < PER; ++i) {
         const int e = lane + 64 * i;
         c[i] = e < E ? s[i] + (rt.bias ? rt.bias[e] : 0.f) : GONE;
     }
     if (rt.groups > 0) {
-        __shared__ float cs[64 * HY_RT_PER], gsc[64 * HY_RT_PER];
+        __shared__ float cs[64 * PER], gsc[64 * PER];
         const int gs = E / rt.groups;
 #pragma unroll
-        for (int i = 0; i < HY_RT_PER; ++i)
+        for (int i = 0; i < PER; ++i)
             if (lane + 64 * i < E) cs[lane + 64 * i] = c[i];
         __syncthreads();
         for (int g = lane; g < rt.groups; g += 64) {
@@ -376,7 +391,7 @@ static __global__ __launch_bounds__(64) void hy_route_kernel(const float* __rest
         __syncthreads();
         // an expert stays open if fewer than `keep` groups stand before its own
 #pragma unroll
-        for (int i = 0; i < HY_RT_PER; ++i) {
+        for (int i = 0; i < PER; ++i) {
             const int e = lane + 64 * i;
             if (e < E) {
                 const int g = e / gs;
@@ -393,7 +408,7 @@ static __global__ __launch_bounds__(64) void hy_route_kernel(const float* __rest
         float best = GONE, bs = 0.f;
         int bi = 0x7fffffff;
 #pragma unroll
-        for (int i = 0; i < HY_RT_PER; ++i)
+        for (int i = 0; i < PER; ++i)
             if (c[i] > best) { best = c[i]; bs = s[i]; bi = lane + 64 * i; }        // ascending index within a lane: strict > keeps the lowest
 #pragma unroll
         for (int o = 32; o > 0; o >>= 1) {
@@ -404,7 +419,7 @@ static __global__ __launch_bounds__(64) void hy_route_kernel(const float* __rest
         wsum += bs;
         if (lane == k) { myw = bs; mysel = bi; }
 #pragma unroll
-        for (int i = 0; i < HY_RT_PER; ++i)
+        for (int i = 0; i < PER; ++i)
             if (lane + 64 * i == bi) c[i] = GONE;
     }
     if (lane < top) {

@@ -546,8 +546,9 @@ int32_t gl3_hy_create(const gl3_model_desc* desc, gl3_ctx** out, std::string& er
         HY_LDS(1, 1); HY_LDS(1, 2); HY_LDS(1, 4); HY_LDS(1, 8); HY_LDS(2, 1); HY_LDS(2, 2); HY_LDS(2, 4); HY_LDS(2, 8);
         HY_LDS(4, 1); HY_LDS(4, 2); HY_LDS(4, 4); HY_LDS(4, 8); HY_LDS(8, 1); HY_LDS(8, 2); HY_LDS(8, 4);
 #undef HY_LDS
-#define HY_LDS(KB, UA) TRYHIP(hipFuncSetAttribute((const void*)hy_heads_attn_kernel<KB, UA>, hipFuncAttributeMaxDynamicSharedMemorySize, 150 * 1024))
-        HY_LDS(1, 1); HY_LDS(1, 2); HY_LDS(1, 4); HY_LDS(1, 8); HY_LDS(2, 1); HY_LDS(2, 2); HY_LDS(2, 4); HY_LDS(2, 8); HY_LDS(4, 1); HY_LDS(4, 2); HY_LDS(4, 4); HY_LDS(4, 8);
+#define HY_LDS(...) TRYHIP(hipFuncSetAttribute((const void*)hy_heads_attn_kernel<__VA_ARGS__>, hipFuncAttributeMaxDynamicSharedMemorySize, 150 * 1024))
+        HY_LDS(1, 1, true); HY_LDS(1, 2, true); HY_LDS(1, 4, true); HY_LDS(2, 1, true); HY_LDS(2, 2, true); HY_LDS(2, 4, true);
+        HY_LDS(4, 1, true); HY_LDS(4, 2, true); HY_LDS(4, 4, true); HY_LDS(1, 1, false); HY_LDS(1, 2, false); HY_LDS(1, 4, false);
 #undef HY_LDS
     }
     TRYHIP(hipDeviceSynchronize());
@@ -1014,21 +1015,21 @@ static int32_t hy_attention_heads(gl3_ctx* ctx, const HyLayer& L, const float* q
     const int H = d.heads, G = d.kv_heads, hpg = H / G;
     // tokens per workgroup: enough for the rows of a key / value head to fill 16; 64 keys per tile for longer portions, 16 for a few tokens (more
     // tiles to split over); both shrink until the scores fit two workgroups into a CU's LDS
-    int QT = 1, KB = n > 16 ? 4 : 1;
+    const bool vec = d.dim % 16 == 0 && d.vdim % 4 == 0 && ldq % 4 == 0 && (((uintptr_t)q | (uintptr_t)kc | (uintptr_t)vc) & 15) == 0;          // (slots are 256-byte aligned)
+    int QT = 1, KB = n > 16 && vec ? 4 : 1;
     while (QT < n && QT * hpg < 16) QT *= 2;
     HyHeadsArgs a;
     auto lds = [&]() {
         a.ts = 16 * KB + 4;
         a.ss = QT * a.ts;
         a.ss += (16 - a.ss % 64 + 64) % 64;          // a head's row starts 16 banks after the one before it
-        return ((size_t)H * a.ss + 3 * (size_t)H * QT) * 4;
+        return ((size_t)H * a.ss + 3 * (size_t)H * QT + (d.head_mix ? (size_t)H * L.mix_ld : 0)) * 4;
     };
     while (lds() > 76 * 1024 && (KB > 1 || QT > 1)) { if (KB > 1) KB /= 2; else QT /= 2; }
     if (lds() > 150 * 1024) GL3_FAIL(GL3_E_UNSUPPORTED, "attention: too many heads for the LDS tile");
     const int KT = 16 * KB, RB = hy_cdiv(QT * hpg, 16), units = G * RB * hy_cdiv(d.vdim, 64), ny = hy_cdiv(units, 32), nx = hy_cdiv(n, QT);
     a.ug = hy_cdiv(units, ny);
-    const int per = hy_cdiv(a.ug, 4), UA = per <= 1 ? 1 : per <= 2 ? 2 : per <= 4 ? 4 : 8;
-    a.ug = 4 * UA < a.ug ? 4 * UA : a.ug;
+    const int per = hy_cdiv(a.ug, 8), UA = per <= 1 ? 1 : per <= 2 ? 2 : 4;          // (32 units: 8 wavefronts x 4)
     // key splits: one tile each for a few tokens; else as many as fill the chip twice
     const long span = d.chunk > 0 ? std::min<long>(pos0 + n, (long)d.chunk + QT - 1) : pos0 + n;          // keys a workgroup walks at most
     int nsplit = (int)std::min<long>(128, span / KT + 1 + (d.chunk > 0 ? 1 : 0));
@@ -1039,27 +1040,20 @@ static int32_t hy_attention_heads(gl3_ctx* ctx, const HyLayer& L, const float* q
     a.dyn = h->dyn; a.n = n; a.nsplit = nsplit; a.part_acc = h->part_acc; a.part_ml = h->part_ml; a.QT = QT;
     const size_t smem = lds();
     const dim3 grid(nx, ny, nsplit);
-#define HY_HA(KBT, UAT) hipLaunchKernelGGL((hy_heads_attn_kernel<KBT, UAT>), grid, dim3(256), smem, ctx->stream, a)
-#define HY_HA_U(KBT) do { if (UA == 1) HY_HA(KBT, 1); else if (UA == 2) HY_HA(KBT, 2); else if (UA == 4) HY_HA(KBT, 4); else HY_HA(KBT, 8); } while (0)
-    if (KB == 4) HY_HA_U(4); else if (KB == 2) HY_HA_U(2); else HY_HA_U(1);
+#define HY_HA(...) hipLaunchKernelGGL((hy_heads_attn_kernel<__VA_ARGS__>), grid, dim3(512), smem, ctx->stream, a)
+#define HY_HA_U(KBT, VEC) do { if (UA == 1) HY_HA(KBT, 1, VEC); else if (UA == 2) HY_HA(KBT, 2, VEC); else HY_HA(KBT, 4, VEC); } while (0)
+    if (!vec) HY_HA_U(1, false);
+    else if (KB == 4) HY_HA_U(4, true); else if (KB == 2) HY_HA_U(2, true); else HY_HA_U(1, true);
 #undef HY_HA_U
 #undef HY_HA
     *nsplit_out = nsplit;
     return GL3_OK;
 }
 
-// The gated delta rule's recurrence: a column's states over NG lanes x NL registers (NG NL >= dim); tokens staged per round: what fits 48 KB of
-// LDS, at most 32.
-static void hy_delta_scan(gl3_ctx* ctx, HyDeltaScan& a) {
-#define HY_DS(NL, NG)                                                                                                                                    \
-    do {                                                                                                                                                 \
-        constexpr int cols = 4 * (64 / NG), Ns = NL * NG;                                                                                                  \
-        const size_t per = 2 * (size_t)Ns + cols + 2;                                                                                                      \
-        a.TB = (int)std::max<size_t>(1, std::min<size_t>(32, (48 * 1024 / 4 - per) / (per + 256)));                                                        \
-        const size_t smem = ((a.TB + 1) * per + (size_t)a.TB * 256) * 4;                                                                                   \
-        hipLaunchKernelGGL((hy_delta_scan_kernel<NL, NG>), dim3(hy_cdiv(a.P, cols), a.heads), dim3(256), smem, ctx->stream, a);                            \
-    } while (0)
-    if (a.N <= 16) HY_DS(4, 4); else if (a.N <= 32) HY_DS(4, 8); else if (a.N <= 64) HY_DS(8, 8); else if (a.N <= 128) HY_DS(8, 16);
+// The gated delta rule's recurrence: a column's states over NG lanes x NL registers (NG NL >= dim).
+static void hy_delta_scan(gl3_ctx* ctx, const HyDeltaScan& a) {
+#define HY_DS(NL, NG) hipLaunchKernelGGL((hy_delta_scan_kernel<NL, NG>), dim3(hy_cdiv(a.P, 4 * (64 / NG)), a.heads), dim3(256), 0, ctx->stream, a)
+    if (a.N <= 16) HY_DS(4, 4); else if (a.N <= 32) HY_DS(4, 8); else if (a.N <= 64) HY_DS(4, 16); else if (a.N <= 128) HY_DS(8, 16);
     else if (a.N <= 256) HY_DS(16, 16); else if (a.N <= 512) HY_DS(32, 16); else HY_DS(32, 32);
 #undef HY_DS
 }
@@ -1365,8 +1359,11 @@ static void hy_moe(gl3_ctx* ctx, HyLayer& L, int n) {
     const bool few = n <= 8;
     const int max_tiles = P / HY_MOE_BM + std::min(E, P);
     const bool on_out = d.route_on_output != 0;          // the weights multiply the experts' outputs (in the residual update) instead of their inputs
-    hipLaunchKernelGGL(hy_route_kernel, dim3(n), dim3(64), 0, st, h->moe_z, RZ, zparts, (size_t)n * RZ, E + d.identity, top, h->sel, h->wsel, few ? h->pair_row : nullptr,
-                       (d.shared_ff > 0 && !d.shared_ungated) ? h->sgz : nullptr, HyRoute{d.route_softmax, L.route_bias, d.route_renorm, d.route_scale != 0.f ? d.route_scale : 1.f, d.route_groups, d.route_keep, E, d.route_group_max});
+    const HyRoute rt{d.route_softmax, L.route_bias, d.route_renorm, d.route_scale != 0.f ? d.route_scale : 1.f, d.route_groups, d.route_keep, E, d.route_group_max};
+#define HY_RT(PER) hipLaunchKernelGGL((hy_route_kernel<PER>), dim3(n), dim3(64), 0, st, h->moe_z, RZ, zparts, (size_t)n * RZ, E + d.identity, top, h->sel, h->wsel,          \
+                                      few ? h->pair_row : nullptr, (d.shared_ff > 0 && !d.shared_ungated) ? h->sgz : nullptr, rt)
+    if (RZ <= 64) HY_RT(1); else if (RZ <= 256) HY_RT(4); else HY_RT(HY_RT_PER);
+#undef HY_RT
     HyMat one_gu = L.egu, one_down = L.edown;
     const bool glu = !hy_ungated(d);
     one_gu.rows = (glu ? 2 : 1) * L.eff_pad; one_down.rows = W;

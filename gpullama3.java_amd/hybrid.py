@@ -1,4 +1,4 @@
-"""Host side of the layer-list family (GL3_ARCH_LAYERLIST: the Noditar, Vonulix, Kosusun, Kugadra and Tutedra designs) over the C-ABI: model folders (config.json + model.safetensors), the step
+"""Host side of the layer-list family (GL3_ARCH_LAYERLIST: the Noditar, Vonulix, Kosusun, Kugadra, Tutedra and Ziginex designs) over the C-ABI: model folders (config.json + model.safetensors), the step
 function with sequence slots, greedy / sampled generation.  The compute path is csrc/gl3_hybrid.hip; nothing here computes.
 
     plan = HybridPlan.from_dir("model-folder", dtype="bfloat16", ctx=4096, max_batch=512, n_seqs=2)
@@ -322,15 +322,55 @@ def tutedra_tensor_shapes(config: dict) -> dict:
     return out
 
 
+def ziginex_tensor_shapes(config: dict) -> dict:
+    """{tensor name: shape} of a Ziginex configuration, in file order (the head is the embedding table)."""
+    W, V = config["width"], config["vocab"]
+    side = (config.get("token_side") or {}).get("dim", 0)
+    out = {"embed": (V, W)}
+    if side:
+        out["side.embed"] = (V, len(config["layers"]) * side)
+    for i, layer in enumerate(config["layers"]):
+        p, m, ff = "l%d." % i, layer["mixer"], layer.get("mlp")
+        out[p + "norm1"] = (W,)
+        if layer["type"] == "parallel":
+            a, d = m["left"], m["right"]
+            H, od = a["heads"], d["heads"] * d["vdim"]
+            left = {"q": (H * a["dim"], W), "k": (a["kv_heads"] * a["dim"], W), "v": (a["kv_heads"] * a["vdim"], W), "q.norm": (a["dim"],), "k.norm": (a["dim"],),
+                    "talk": (H, H), "temp": (H,), "sink": (H,), "o": (W, H * a["vdim"]), "out": (W,)}
+            nk, H = d["kv_heads"] * d["dim"], d["heads"]
+            right = {"q": (nk, W), "q.conv": (nk, d["conv"]), "k": (nk, W), "k.conv": (nk, d["conv"]), "v": (od, W), "v.conv": (od, d["conv"]), "b": (H, W), "a": (H, W),
+                     "A_log": (H,), "dt_bias": (H,), "norm": (d["vdim"],), "g": (od, W), "o": (W, od), "out": (W,)}
+            out.update({p + "mix.left." + k: v for k, v in left.items()})
+            out.update({p + "mix.right." + k: v for k, v in right.items()})
+        else:
+            P, R, od = m.get("rot_dim", 0), m["kv_rank"], m["heads"] * m["vdim"]
+            mix = {"dq": (m["q_rank"], W), "dq.norm": (m["q_rank"],), "uq": (m["heads"] * (m["dim"] + P), m["q_rank"]), "dkv": (R + P, W), "dkv.norm": (R,),
+                   "uk": (m["heads"] * m["dim"], R), "uv": (od, R), "sink": (m["heads"],), "g": (od, W), "o": (W, od)}
+            out.update({p + "mix." + k: v for k, v in mix.items()})
+        if ff:
+            out[p + "norm2"] = (W,)
+            if ff["kind"] == "dense":
+                out.update({p + "mlp.gate": (ff["ff"], W), p + "mlp.up": (ff["ff"], W), p + "mlp.down": (W, ff["ff"])})
+            else:
+                f, n = ff["expert"]["ff"], ff["router"]["experts"] + (ff["router"].get("identity") or 0)
+                for e in range(ff["router"]["experts"]):
+                    out.update({p + "mlp.e%d.gate" % e: (f, W), p + "mlp.e%d.up" % e: (f, W), p + "mlp.e%d.down" % e: (W, f)})
+                out.update({p + "mlp.router": (n, W), p + "mlp.correction": (n,)})
+        if side:
+            out.update({p + "side.gate": (side, W), p + "side.proj": (W, side), p + "side.norm": (W,)})
+    out["final.norm"] = (W,)
+    return out
+
+
 def random_model_dir(path: str, config: dict, seed: int = 0):
     """A model folder with random weights for timing: matrices are random bfloat16 bit patterns of magnitude 2^-9 .. 2^-6 / sqrt-free (cheap to
     make at billions of elements), vectors and tables are benign constants with noise."""
     rng = np.random.default_rng(seed)
     S = config.get("streams", 1)
     t = {}
-    vonulix, kosusun, kugadra, tutedra = (config["architecture"] == a for a in ("Vonulix", "Kosusun", "Kugadra", "Tutedra"))
+    vonulix, kosusun, kugadra, tutedra, ziginex = (config["architecture"] == a for a in ("Vonulix", "Kosusun", "Kugadra", "Tutedra", "Ziginex"))
     shapes = (vonulix_tensor_shapes(config) if vonulix else kosusun_tensor_shapes(config) if kosusun else kugadra_tensor_shapes(config) if kugadra
-              else tutedra_tensor_shapes(config) if tutedra else noditar_tensor_shapes(config))
+              else tutedra_tensor_shapes(config) if tutedra else ziginex_tensor_shapes(config) if ziginex else noditar_tensor_shapes(config))
     for name, shp in shapes.items():
         leaf = name.split(".", 1)[1] if name[0] == "l" and name[1].isdigit() else name
         if kosusun and leaf.endswith((".b", ".sink")):
@@ -338,7 +378,11 @@ def random_model_dir(path: str, config: dict, seed: int = 0):
         elif tutedra and leaf in ("mix.f.b", "mix.i.b", "shift", "mix.lower", "ls1", "ls2", "mlp.act"):
             v = {"mix.f.b": 3.0, "mix.i.b": 0.0, "shift": 0.25, "mix.lower": 0.5, "ls1": 1.0, "ls2": 1.0, "mlp.act": 0.3}[leaf]
             t[name] = np.full(shp, v, np.float32)
-        elif leaf in ("mix.q.conv", "mix.k.conv"):
+        elif ziginex and leaf == "mix.left.talk":
+            t[name] = (np.eye(shp[0]) + 0.1 * rng.standard_normal(shp)).astype(np.float32)
+        elif ziginex and (leaf.endswith((".norm", ".out")) or leaf in ("norm1", "norm2")):
+            t[name] = np.ones(shp, np.float32)
+        elif leaf in ("mix.q.conv", "mix.k.conv") or (ziginex and leaf.endswith(".conv")):
             t[name] = np.full(shp, 1.0 / shp[1], np.float32)
         elif (vonulix or tutedra) and leaf in ("norm1", "norm2", "final.norm"):
             t[name] = np.zeros(shp, np.float32)                  # the file holds weight - 1
@@ -356,7 +400,7 @@ def random_model_dir(path: str, config: dict, seed: int = 0):
             t[name] = (np.eye(S) + 0.05 * rng.standard_normal(shp)).astype(np.float32)
         elif leaf.endswith(".in") and leaf.startswith("hc"):
             t[name] = np.full(shp, 1.0 / S, np.float32)
-        elif leaf in ("mix.A_log", "mix.dt_bias"):
+        elif leaf.endswith((".A_log", ".dt_bias")):
             t[name] = rng.uniform(-1.0, 0.0, shp).astype(np.float32)
         elif leaf == "mix.conv":
             t[name] = (0.3 * rng.standard_normal(shp)).astype(np.float32)
