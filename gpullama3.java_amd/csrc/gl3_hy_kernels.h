@@ -1027,6 +1027,60 @@ static __global__ __launch_bounds__(64) void hy_attn_merge_kernel(const float* _
     }
 }
 
+// The same for a few tokens, whose keys are split over many workgroups (nsplit <= HY_MAX_SPLITS, dv <= 512): 256 threads per (token, head).  The splits'
+// weights are made side by side; the four wavefronts then share the splits of every column, eight loads in flight each, and meet in LDS.
+constexpr int HY_MAX_SPLITS = 128;
+template <typename TO>
+static __global__ __launch_bounds__(256) void hy_attn_merge_few_kernel(const float* __restrict__ part_acc, const float* __restrict__ part_ml, int H, int dv, int nsplit,
+                                                                       int sink, const float* __restrict__ gate, int ldg, int gate_mode, TO* __restrict__ out, int ldo,
+                                                                       const float* __restrict__ v_freq, const int* __restrict__ dyn, const float* __restrict__ sink_w, float out_mul) {
+    __shared__ float sw[HY_MAX_SPLITS], sm[4], red[4], part[4][512];
+    const int t = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const size_t o = ((size_t)t * H + h) * nsplit;
+    const float z = sink_w ? sink_w[h] : 0.f;
+    const float ms = tid < nsplit ? part_ml[2 * (o + tid)] : -INFINITY, ls = tid < nsplit ? part_ml[2 * (o + tid) + 1] : 0.f;
+    float M = hy_wave_max(ms);
+    if (lane == 0) sm[wave] = M;
+    __syncthreads();
+    M = fmaxf(fmaxf(sm[0], sm[1]), fmaxf(sm[2], sm[3]));
+    if (sink) M = fmaxf(M, z);
+    const float e = ms > -INFINITY ? expf(ms - M) : 0.f;
+    const float den = hy_block_sum<256>(e * ls, red) + (sink ? expf(z - M) : 0.f);
+    if (tid < nsplit) sw[tid] = e / den;
+    __syncthreads();
+    for (int c = lane; c < dv; c += 64) {
+        float v = 0.f;
+        for (int s0 = wave; s0 < nsplit; s0 += 32) {
+            float q[8];
+#pragma unroll
+            for (int u = 0; u < 8; ++u) q[u] = part_acc[(o + min(s0 + 4 * u, nsplit - 1)) * dv + c];
+#pragma unroll
+            for (int u = 0; u < 8; ++u) v = fmaf(s0 + 4 * u < nsplit ? sw[min(s0 + 4 * u, nsplit - 1)] : 0.f, q[u], v);
+        }
+        part[wave][c] = v;
+    }
+    __syncthreads();
+    auto column = [&](int c) { return (part[0][c] + part[1][c]) + (part[2][c] + part[3][c]); };
+    const float ghead = (gate && gate_mode == 2) ? hy_sigmoid(gate[(size_t)t * ldg + h]) : 1.f;
+    auto put = [&](int c, float v) {
+        if (gate && gate_mode != 2) v *= hy_sigmoid(gate[(size_t)t * ldg + h * dv + c]);
+        hy_st(out + (size_t)t * ldo + h * dv + c, v * ghead * out_mul);
+    };
+    if (v_freq) {
+        const int half = dv >> 1;
+        const float pos = (float)(dyn[0] + t);
+        for (int c = tid; c < half; c += 256) {
+            float sn, cs;
+            sincosf(pos * v_freq[c], &sn, &cs);
+            const float u = column(c), v = column(c + half);
+            put(c, u * cs + v * sn);
+            put(c + half, v * cs - u * sn);
+        }
+    } else {
+        for (int c = tid; c < dv; c += 256) put(c, column(c));
+    }
+}
+
 // ---- state-space mixer ------------------------------------------------------------------------------------------------------------
 // Causal depthwise convolution over the step's tokens; inputs before the step come from the slot's tail (the last taps - 1 inputs of
 // the sequence), zeros before position 0.  out = silu(bias + sum_k w[c][k] in(t - (taps - 1 - k))).

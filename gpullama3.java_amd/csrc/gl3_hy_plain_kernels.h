@@ -65,6 +65,13 @@ static __global__ __launch_bounds__(NT) void hy_resid_kernel(HyResid a, TO* __re
     __shared__ float red[2 * (NT / 64)];
     const int t = blockIdx.x, W = a.W;
     const size_t row = (size_t)t * W;
+    // the thread's first columns of the residual and of the post norm's weight travel with the first loads below (the sums put barriers between)
+    const int wf = threadIdx.x * V;
+    float x0[V], pw0[V];
+    if (wf < W) {
+        hy_ldv<V>(a.x + row + wf, x0);
+        if (a.post_w) hy_ldv<V>(a.post_w + wf, pw0);
+    }
     float cr = 0.f;
     if (a.yc) {
         float ss = 0.f;
@@ -98,12 +105,14 @@ static __global__ __launch_bounds__(NT) void hy_resid_kernel(HyResid a, TO* __re
             for (int i = 0; i < V; ++i) y[i] += q[i];
         }
     };
-    float b1 = 0.f, b2 = 0.f;          // two normed mixers: 1 / rms of each one's whole output; its first chunks stay in registers for `addend`
+    float b1 = 0.f, b2 = 0.f;          // two normed mixers: 1 / rms of each one's whole output; its first chunks, times their weights, stay in registers
     float by[BR ? HY_RC : 1][V], bz[BR ? HY_RC : 1][V];
     if constexpr (BR) {
         int it = 0;
         for (int w = threadIdx.x * V; w < W; w += NT * V, ++it) {
-            float y[V], z[V];
+            float y[V], z[V], w1[V], w2[V];
+            hy_ldv<V>(a.bw1 + w, w1);
+            hy_ldv<V>(a.bw2 + w, w2);
             parts(w, 0, a.ya_first, y);
             parts(w, a.ya_first, a.ya_parts, z);
 #pragma unroll
@@ -112,7 +121,7 @@ static __global__ __launch_bounds__(NT) void hy_resid_kernel(HyResid a, TO* __re
             for (int q = 0; q < HY_RC; ++q)
                 if (q == it)
 #pragma unroll
-                    for (int i = 0; i < V; ++i) { by[q][i] = y[i]; bz[q][i] = z[i]; }
+                    for (int i = 0; i < V; ++i) { by[q][i] = y[i] * w1[i]; bz[q][i] = z[i] * w2[i]; }
         }
         hy_block_sum2<NT>(b1, b2, red);
         b1 = 1.f / sqrtf(b1 / (float)W + a.eps);
@@ -123,7 +132,7 @@ static __global__ __launch_bounds__(NT) void hy_resid_kernel(HyResid a, TO* __re
 #pragma unroll
         for (int i = 0; i < V; ++i) y[i] = e[i] = 0.f;
         if constexpr (BR) {
-            float z[V], w1[V], w2[V];
+            float z[V];
             if (it < HY_RC) {
 #pragma unroll
                 for (int q = 0; q < HY_RC; ++q)
@@ -131,13 +140,16 @@ static __global__ __launch_bounds__(NT) void hy_resid_kernel(HyResid a, TO* __re
 #pragma unroll
                         for (int i = 0; i < V; ++i) { y[i] = by[q][i]; z[i] = bz[q][i]; }
             } else {
+                float w1[V], w2[V];
+                hy_ldv<V>(a.bw1 + w, w1);
+                hy_ldv<V>(a.bw2 + w, w2);
                 parts(w, 0, a.ya_first, y);
                 parts(w, a.ya_first, a.ya_parts, z);
-            }
-            hy_ldv<V>(a.bw1 + w, w1);
-            hy_ldv<V>(a.bw2 + w, w2);
 #pragma unroll
-            for (int i = 0; i < V; ++i) y[i] = y[i] * b1 * w1[i] + z[i] * b2 * w2[i];
+                for (int i = 0; i < V; ++i) { y[i] *= w1[i]; z[i] *= w2[i]; }
+            }
+#pragma unroll
+            for (int i = 0; i < V; ++i) y[i] = y[i] * b1 + z[i] * b2;
         } else if (a.ya) parts(w, 0, a.ya_parts, y);
         if (a.eo)
             for (int k = 0; k < a.top; ++k) {
@@ -173,7 +185,10 @@ static __global__ __launch_bounds__(NT) void hy_resid_kernel(HyResid a, TO* __re
     int it = 0;
     for (int w = threadIdx.x * V; w < W; w += NT * V, ++it) {
         float x[V], y[V], e[V], c[V], cw[V];
-        hy_ldv<V>(a.x + row + w, x);
+        if (it == 0) {
+#pragma unroll
+            for (int i = 0; i < V; ++i) x[i] = x0[i];
+        } else hy_ldv<V>(a.x + row + w, x);
 #pragma unroll
         for (int i = 0; i < V; ++i) c[i] = 0.f;
         if (a.post_w && it < HY_RC) {
@@ -191,7 +206,10 @@ static __global__ __launch_bounds__(NT) void hy_resid_kernel(HyResid a, TO* __re
         if (a.yc) { hy_ldv<V>(a.yc + row + w, c); hy_ldv<V>(a.cw + w, cw); }
         if (a.post_w) {
             float pw[V];
-            hy_ldv<V>(a.post_w + w, pw);
+            if (it == 0) {
+#pragma unroll
+                for (int i = 0; i < V; ++i) pw[i] = pw0[i];
+            } else hy_ldv<V>(a.post_w + w, pw);
 #pragma unroll
             for (int i = 0; i < V; ++i) y[i] = y[i] * pr * pw[i];
             if (a.lw) {
@@ -344,6 +362,9 @@ static __global__ __launch_bounds__(64) void hy_route_kernel(const float* __rest
                                                              HyRoute rt) {
     const int t = blockIdx.x, lane = threadIdx.x;
     constexpr float GONE = -3.0e38f;
+    __shared__ float pick_w[64];
+    __shared__ int pick_e[64];
+    if constexpr (PER == 1) { pick_w[lane] = 0.f; pick_e[lane] = 0; __syncthreads(); }
     float s[PER], c[PER];          // score; what the choice goes by
     float zmax = -INFINITY;
 #pragma unroll
@@ -404,6 +425,18 @@ static __global__ __launch_bounds__(64) void hy_route_kernel(const float* __rest
     }
     float wsum = 0.f, myw = 0.f;          // lane k keeps the weight of choice k (top <= 64) until the sum is known
     int mysel = 0;
+    if constexpr (PER == 1) {          // an output per lane: its rank is the number of outputs before it, the lane of rank k hands choice k over
+        int rank = 0;
+        for (int j = 0; j < E; ++j) {
+            const float o = __int_as_float(__builtin_amdgcn_readlane(__float_as_int(c[0]), j));
+            rank += (o > c[0] || (o == c[0] && j < lane)) ? 1 : 0;
+        }
+        const bool mine = lane < E && rank < top;
+        wsum = hy_wave_sum(mine ? s[0] : 0.f);
+        if (mine) { pick_w[rank] = s[0]; pick_e[rank] = lane; }
+        __syncthreads();
+        if (lane < top) { myw = pick_w[lane]; mysel = pick_e[lane]; }
+    } else
     for (int k = 0; k < top; ++k) {
         float best = GONE, bs = 0.f;
         int bi = 0x7fffffff;

@@ -990,7 +990,7 @@ static int32_t hy_attention(gl3_ctx* ctx, const float* q, int ldq, const float* 
         int tiles = hy_cdiv(pos0 + n, p.kt);
         if (window > 0) tiles = std::min<long>(tiles, hy_cdiv(keep, p.kt) + ((long)window + n) / p.kt + 2);      // kept first keys + the window's tiles
         if (pool > 0) tiles += hy_cdiv(std::max(0, pos0 + n - window) / pool, p.kt);                               // + the tiles of pooled rows
-        nsplit = std::min(128, std::max(1, tiles));
+        nsplit = std::min(HY_MAX_SPLITS, std::max(1, tiles));
     }
     if ((size_t)n * nsplit > h->part_rows) nsplit = std::max<size_t>(1, h->part_rows / n);
     HyAttnArgs a;
@@ -1006,6 +1006,20 @@ static int32_t hy_attention(gl3_ctx* ctx, const float* q, int ldq, const float* 
 #undef HY_AT
     *nsplit_out = nsplit;
     return GL3_OK;
+}
+
+// Joins the key splits of an attention core's launch: out[n][heads dv] (row stride ldo), gated and turned back where the layer asks for it.
+template <typename TO>
+static void hy_merge(gl3_ctx* ctx, const HyLayer& L, int n, int dv, int nsplit, const float* gate, int ldg, int gate_mode, TO* out, int ldo, const float* v_freq = nullptr, float out_mul = 1.f) {
+    gl3_hybrid_state* h = ctx->hy;
+    const gl3_layer_desc& d = L.d;
+    const float* sink_w = d.softmax_sink == 2 ? L.sink : nullptr;
+    if (nsplit > 2 && nsplit <= HY_MAX_SPLITS && n <= 16)
+        hipLaunchKernelGGL((hy_attn_merge_few_kernel<TO>), dim3(n, d.heads), dim3(256), 0, ctx->stream, h->part_acc, h->part_ml, d.heads, dv, nsplit, d.softmax_sink, gate, ldg, gate_mode, out, ldo,
+                           v_freq, h->dyn, sink_w, out_mul);
+    else
+        hipLaunchKernelGGL((hy_attn_merge_kernel<TO>), dim3(n, d.heads), dim3(64), 0, ctx->stream, h->part_acc, h->part_ml, d.heads, dv, nsplit, d.softmax_sink, gate, ldg, gate_mode, out, ldo,
+                           v_freq, h->dyn, sink_w, out_mul);
 }
 
 // Attention over all heads at once (hy_heads_attn_kernel): temperatures, capped and mixed scores, chunks.
@@ -1032,7 +1046,7 @@ static int32_t hy_attention_heads(gl3_ctx* ctx, const HyLayer& L, const float* q
     const int per = hy_cdiv(a.ug, 8), UA = per <= 1 ? 1 : per <= 2 ? 2 : 4;          // (32 units: 8 wavefronts x 4)
     // key splits: one tile each for a few tokens; else as many as fill the chip twice
     const long span = d.chunk > 0 ? std::min<long>(pos0 + n, (long)d.chunk + QT - 1) : pos0 + n;          // keys a workgroup walks at most
-    int nsplit = (int)std::min<long>(128, span / KT + 1 + (d.chunk > 0 ? 1 : 0));
+    int nsplit = (int)std::min<long>(HY_MAX_SPLITS, span / KT + 1 + (d.chunk > 0 ? 1 : 0));
     if (n > 16) nsplit = std::min(nsplit, std::max(1, 512 / std::max(1, nx * ny)));
     if ((size_t)n * nsplit > h->part_rows) nsplit = (int)std::max<size_t>(1, h->part_rows / n);
     a.q = q; a.ldq = ldq; a.kc = kc; a.vc = vc; a.slot_stride = h->slot_floats; a.H = H; a.G = G; a.dk = d.dim; a.dv = d.vdim; a.scale = d.scale; a.cap = d.score_softcap;
@@ -1149,9 +1163,8 @@ static int32_t hy_mixer_core(gl3_ctx* ctx, HyLayer& L, int np, int ldo, int n, i
                                    : hy_attention(ctx, q, ldq, kc, vc, d.heads, d.kv_heads, d.dim, d.vdim, d.scale, d.slope_log2, n, pos0, &nsplit, true, d.window, d.keep_first,
                                                   pk, pv, d.pool);
         if (r != GL3_OK) return r;
-        hipLaunchKernelGGL((hy_attn_merge_kernel<T>), dim3(n, d.heads), dim3(64), 0, st, h->part_acc, h->part_ml, d.heads, d.vdim, nsplit, d.softmax_sink,
-                           d.out_gate ? h->proj + L.g_off : nullptr, np, d.out_gate, mixo, ldo, d.v_rot ? L.vrot_freq : nullptr, h->dyn,
-                           d.softmax_sink == 2 ? L.sink : nullptr, d.out_norm ? 1.f : L.out_mul);
+        hy_merge<T>(ctx, L, n, d.vdim, nsplit, d.out_gate ? h->proj + L.g_off : nullptr, np, d.out_gate, mixo, ldo, d.v_rot ? L.vrot_freq : nullptr,
+                    d.out_norm ? 1.f : L.out_mul);
     } else if (d.mixer == GL3_MIX_MEMORY && d.mem_gates == GL3_MEM_DELTA) {
         const int ch = hy_delta_ch(d), inner = d.heads * d.vdim, nk = d.kv_heads * d.dim;
         float *ga = h->gates, *gb = ga + (size_t)h->mb * h->max_heads;
@@ -1222,8 +1235,7 @@ static int32_t hy_mixer_core(gl3_ctx* ctx, HyLayer& L, int np, int ldo, int n, i
             hy_gemm<float>(ctx, lat, R, wvm, M, h->vx, d.heads * d.vdim, false, nullptr, 0, HyGlu{});
             int32_t r = hy_attention(ctx, q, ldq, h->kx, h->vx, d.heads, d.heads, De, d.vdim, d.scale, 0.f, n, pos0, &nsplit, false);
             if (r != GL3_OK) return r;
-            hipLaunchKernelGGL((hy_attn_merge_kernel<T>), dim3(n, d.heads), dim3(64), 0, st, h->part_acc, h->part_ml, d.heads, d.vdim, nsplit, d.softmax_sink,
-                               d.out_gate ? h->proj + L.g_off : nullptr, np, d.out_gate == 2 ? 2 : 1, mixo, ldo, (const float*)nullptr, h->dyn, L.sink);
+            hy_merge<T>(ctx, L, n, d.vdim, nsplit, d.out_gate ? h->proj + L.g_off : nullptr, np, d.out_gate == 2 ? 2 : 1, mixo, ldo);
         } else {
             // A few tokens (decode): the query is carried into the latent's space and the attention core reads the latents themselves
             // (one shared key / value head, keys = values), then the weighted sum of latents is expanded.
@@ -1235,8 +1247,7 @@ static int32_t hy_mixer_core(gl3_ctx* ctx, HyLayer& L, int np, int ldo, int n, i
                                    (const float*)nullptr, 0, h->qa, d.heads * R, n);
             int32_t r = hy_attention(ctx, h->qa, d.heads * R, cc, cc, d.heads, 1, R, R, d.scale, 0.f, n, pos0, &nsplit);
             if (r != GL3_OK) return r;
-            hipLaunchKernelGGL((hy_attn_merge_kernel<float>), dim3(n, d.heads), dim3(64), 0, st, h->part_acc, h->part_ml, d.heads, R, nsplit, d.softmax_sink,
-                               (const float*)nullptr, 0, 0, h->oc, d.heads * R, (const float*)nullptr, h->dyn, L.sink);
+            hy_merge<float>(ctx, L, n, R, nsplit, nullptr, 0, 0, h->oc, d.heads * R);
             if (n == 1)
                 hipLaunchKernelGGL((hy_headmm_kernel<T, 1>), dim3(1, d.heads, hy_cdiv(d.vdim, 64)), dim3(256), 0, st, h->oc, d.heads * R, R, d.vdim, L.wvT,
                                    d.out_gate ? h->proj + L.g_off : nullptr, np, mixo, ldo, n, d.out_gate == 2 ? 2 : 1);
